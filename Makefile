@@ -9,10 +9,12 @@
 #                   does not change
 #   make layer      libvmi_gpt2_layer.so (include/vmi_gpt2_layer.h): the decode harness's own library — the GPT-2 block's
 #                   linear layers; one unit, part of `make` / `all`
+#   make hybrid     libvmi_hybrid.so (include/vmi_hybrid.h): the layers of decoders with recurrent blocks and latent
+#                   attention; three units, part of `make` / `all`
 HIPCC  ?= hipcc
 ARCH   ?= gfx950
 # -ffp-contract=off: the fp16 p*v products are rounded before the fp16 adds (the reference's rounding points)
-FLAGS  := --offload-arch=$(ARCH) -O3 -std=c++17 -ffp-contract=off -fPIC -fvisibility=hidden -fno-gpu-rdc -Iinclude
+FLAGS  := --offload-arch=$(ARCH) -O3 -std=c++17 -ffp-contract=off -fPIC -fvisibility=hidden -fno-gpu-rdc -Xclang -target-feature -Xclang -packed-fp32-ops -Iinclude
 CSRC   := vllmini_amd/csrc
 OUTDIR := vllmini_amd/_C
 CORE_UNITS := paged_attention pa_variants_extra pa_append_core pa_append_extra pa_variants_fp8 pa_queue pa_split
@@ -32,7 +34,17 @@ DEPS   := $(wildcard $(CSRC)/*.hpp) $(wildcard $(CSRC)/*.inc) include/vmi_paged_
 
 LAYER_LIB := $(OUTDIR)/libvmi_gpt2_layer.so
 
-all: $(LIB) $(LAYER_LIB) oracle
+HYBRID_LIB := $(OUTDIR)/libvmi_hybrid.so
+HYBRID_UNITS := hybrid_linear hybrid_rglru hybrid_latent
+HYBRID_SRCS := $(HYBRID_UNITS:%=$(CSRC)/%.hip)
+
+all: $(LIB) $(LAYER_LIB) $(HYBRID_LIB) oracle
+
+hybrid: $(HYBRID_LIB)
+
+$(HYBRID_LIB): $(HYBRID_SRCS) $(CSRC)/hybrid_common.hpp include/vmi_hybrid.h
+	mkdir -p $(OUTDIR)
+	$(HIPCC) $(filter-out -ffp-contract=off,$(FLAGS)) -shared $(HYBRID_SRCS) -o $@
 
 layer: $(LAYER_LIB)
 

@@ -84,6 +84,10 @@ EXTRAS_LIB_PATH = os.path.join(OUT_DIR, "libvmi_paged_attention_extras.so")
 SRC_LAYER = os.path.join(CSRC, "gpt2_layer.hip")
 LAYER_LIB_PATH = os.path.join(OUT_DIR, "libvmi_gpt2_layer.so")
 
+# the layers of decoders with recurrent blocks and latent attention (include/vmi_hybrid.h): three units, loaded by hybrid_ops.py only
+SRC_HYBRID = [os.path.join(CSRC, f"hybrid_{t}.hip") for t in ("linear", "rglru", "latent")]
+HYBRID_LIB_PATH = os.path.join(OUT_DIR, "libvmi_hybrid.so")
+
 ARCH = "gfx950"
 # -ffp-contract=off: the fp16 p*v products must be rounded before the fp16 adds (reference
 # rounding points, dtype_float16.cuh:252-260, 451-457) — no v_pk_fma_f16 contraction.
@@ -95,6 +99,8 @@ HIPCC_FLAGS = [
     "-fPIC",
     "-fvisibility=hidden",          # only the extern "C" entries (VMI_API in the headers) leave the library
     "-fno-gpu-rdc", *os.environ.get("VMI_EXTRA_FLAGS", "").split(),
+    # no packed fp32 arithmetic (v_pk_add / mul / fma_f32): some of its forms have given wrong results on these parts
+    "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     f"-I{INCLUDE}",
 ]
 
@@ -137,6 +143,8 @@ def _obj_of(src: str, flavor="") -> str:
 
 def _flags(flavor="") -> list[str]:
     flavor = {False: "", True: "diag"}.get(flavor, flavor)
+    if flavor == "fma":      # no reference rounding points to keep: products and sums may contract
+        return [f for f in HIPCC_FLAGS if f != "-ffp-contract=off"]
     extra = {"": [], "extras": ["-DVMI_EXTRAS"], "diag": ["-DVMI_DIAG", "-DVMI_EXTRAS"]}[flavor]
     return [*HIPCC_FLAGS, *extra]
 
@@ -206,7 +214,7 @@ def build_layer(force: bool = False, verbose: bool = False) -> str:
         return LAYER_LIB_PATH      # a tree with libraries and no objects is the GPU box: complete as it is (see build())
     if force or layer_is_stale():
         tmp = LAYER_LIB_PATH + ".tmp"
-        cmd = [_hipcc(), *[f for f in HIPCC_FLAGS if f != "-ffp-contract=off"], "-shared", SRC_LAYER, "-o", tmp]
+        cmd = [_hipcc(), *_flags("fma"), "-shared", SRC_LAYER, "-o", tmp]
         if verbose:
             print(" ".join(cmd), file=sys.stderr)
         proc = subprocess.run(cmd, capture_output=True, text=True)
@@ -214,6 +222,26 @@ def build_layer(force: bool = False, verbose: bool = False) -> str:
             raise RuntimeError(f"hipcc failed ({proc.returncode}): {' '.join(cmd)}\n{proc.stdout}\n{proc.stderr}")
         os.replace(tmp, LAYER_LIB_PATH)
     return LAYER_LIB_PATH
+
+
+def hybrid_is_stale() -> bool:
+    if not os.path.exists(HYBRID_LIB_PATH):
+        return True
+    t = os.path.getmtime(HYBRID_LIB_PATH)
+    deps = [*SRC_HYBRID, os.path.join(CSRC, "hybrid_common.hpp"), os.path.join(INCLUDE, "vmi_hybrid.h")]
+    return any(os.path.getmtime(d) > t for d in deps)
+
+
+def build_hybrid(force: bool = False, verbose: bool = False) -> str:
+    """libvmi_hybrid.so: its units compiled concurrently, one link (~40 s; all a checkout needs to run the hybrid decoders)."""
+    os.makedirs(OUT_DIR, exist_ok=True)
+    if not force and os.path.exists(HYBRID_LIB_PATH) and not _have_objects():
+        return HYBRID_LIB_PATH
+    if force or hybrid_is_stale():
+        units = [(s, "fma") for s in SRC_HYBRID]
+        _compile([u for u in units if force or _obj_stale(*u)], verbose)
+        _link([_obj_of(*u) for u in units], HYBRID_LIB_PATH, verbose)
+    return HYBRID_LIB_PATH
 
 
 def _have_objects() -> bool:
@@ -229,6 +257,7 @@ def build(force: bool = False, verbose: bool = False, diag: bool = False, extras
     complete as it is: nothing is recompiled there."""
     os.makedirs(OUT_DIR, exist_ok=True)
     build_layer(force, verbose)
+    build_hybrid(force, verbose)
     kinds = ["product"] + (["extras"] if (extras or diag) else []) + (["diag"] if diag else [])
     if not force and not _have_objects() and not any(is_stale(k) for k in kinds):
         return _lib_of(kinds[-1])
