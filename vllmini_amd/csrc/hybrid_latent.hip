@@ -1,0 +1,403 @@
+// Latent attention over a paged cache of latents (include/vmi_hybrid.h): the queries are taken into the latent space (the key
+// up-projection is folded into them), so a cache row [rank | rot] is at once the key of ALL heads and, its first `rank` columns,
+// their value: one page read serves every head, and the rows of a query tile are (token, head) pairs.
+//
+// A workgroup takes 16 * RT query rows and walks its keys in tiles of KT cache rows.  A tile comes from the pages into LDS once
+// (requested one tile ahead, held in registers meanwhile) and is used three ways: wave w scores the 16 keys 16 w ..; softmax
+// statistics meet in LDS; then wave w adds the value columns w, w + 4, ... (tiles of 16) of all rows, the value operand read
+// column-wise from the same LDS rows (ds_read_b64_tr_b16).  Scores, softmax and accumulators are fp32.  A sequence whose rows do
+// not fill the chip has its keys dealt to `splits` workgroups, whose unnormalised parts a second kernel adds up.
+#include "hybrid_common.hpp"
+
+namespace vmi_hybrid {
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+
+// 8 consecutive rows (keys) of one column of an LDS tile, as a matrix operand's fragment: lane = (kc, column r16)
+__device__ __forceinline__ b16x8 column8(const b16* tile, int ld, int row0, int col0, int r16) {
+  const b16* a = tile + (row0 + (r16 >> 2)) * ld + col0 + 4 * (r16 & 3);
+  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a);
+  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a + 4 * ld));
+  // (whole vectors are cast: a bit_cast of one vector element takes element 0 on this compiler)
+  return __builtin_shufflevector(__builtin_bit_cast(b16x4, lo), __builtin_bit_cast(b16x4, hi), 0, 1, 2, 3, 4, 5, 6, 7);
+}
+__device__ __forceinline__ f32x8 column8(const float* tile, int ld, int row0, int col0, int r16) {
+  f32x8 r;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) r[e] = tile[(row0 + e) * ld + col0 + r16];
+  return r;
+}
+
+__device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+
+template <typename T>
+constexpr int pad_of() {
+  return 16 / (int)sizeof(T);
+}
+
+template <typename T, int KT, int RT>
+inline size_t attention_lds(int D) {
+  return ((size_t)(KT + 16 * RT) * (D + pad_of<T>()) + (size_t)16 * RT * (KT + pad_of<T>())) * sizeof(T) + (size_t)4 * 16 * RT * 4;
+}
+
+// RT row tiles, NT value tiles (of 16 columns) per wave, U 16-byte-element units of a cache row per thread
+template <typename T, int KT, int RT, int NT, int U>
+__global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_latent_attention_args p, const vmi_hy_step s) {
+  constexpr int R = 16 * RT, TPK = 256 / KT, PAD = pad_of<T>(), LDP = KT + PAD, SW = KT / 16;   // SW waves score
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+  const int D = p.rank + p.rot, LDK = D + PAD;
+  T* ks = reinterpret_cast<T*>(smem);              // [KT][LDK]
+  T* qs = ks + (size_t)KT * LDK;                   // [R][LDK]
+  T* ps = qs + (size_t)R * LDK;                    // [R][LDP]
+  float* sx = reinterpret_cast<float*>(ps + (size_t)R * LDP);   // [4][R]
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), kc = lane >> 4, r16 = lane & 15;
+  const int e = p.tiles[2 * blockIdx.x], r0 = p.tiles[2 * blockIdx.x + 1], split = blockIdx.y;
+  if (e < 0) return;
+  const int H = p.heads, ctx = s.ctx[e];
+  const int nrows = min(R, s.q_len[e] * H - r0);
+  if (nrows <= 0) return;
+  const int64_t grow0 = (int64_t)s.q_start[e] * H + r0;          // row of q / out
+  const int kv_end = ctx + (r0 + nrows - 1) / H + 1;
+  const int nkt = (kv_end + KT - 1) / KT, tps = (nkt + p.splits - 1) / p.splits;
+  const int kt0 = split * tps, kt1 = min(nkt, kt0 + tps);
+  const int n16 = p.rank >> 4, d0 = (int)blockIdx.z * (NT * 4);   // this workgroup's value tiles: d0 + wave + 4 nt
+  float* part = p.partial ? p.partial + ((int64_t)split * s.T * H + grow0) * (p.rank + 2) : nullptr;
+  if (kt0 >= kt1) {   // (splits > 1 only: split 0 always has keys)
+    if (blockIdx.z == 0 && tid < nrows) {
+      part[(int64_t)tid * (p.rank + 2) + p.rank] = -1e30f;
+      part[(int64_t)tid * (p.rank + 2) + p.rank + 1] = 0.f;
+    }
+    return;
+  }
+
+  const T* cache = static_cast<const T*>(p.cache);
+  const int* tab = s.table + (int64_t)e * s.table_ld;
+  const int kj = tid / TPK, kcol = (tid % TPK) * 8;   // this thread's key of a tile, first column
+  auto page_of = [&](int kt) -> int64_t {              // cache row of the thread's key, -1 past the end
+    const int pos = kt * KT + kj;
+    return pos < kv_end ? (int64_t)tab[pos / s.page_size] * s.page_size + pos % s.page_size : -1;
+  };
+  V8<T> kr[U];
+  auto load_tile = [&](int64_t row) {
+    const T* src = cache + row * D + kcol;
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+      kr[i] = row >= 0 && kcol + i * TPK * 8 < D ? load8(src + i * TPK * 8) : zero8<T>();
+  };
+  load_tile(page_of(kt0));
+  int64_t next_row = kt0 + 1 < kt1 ? page_of(kt0 + 1) : -1;
+
+  for (int u = tid; u < R * (D >> 3); u += 256) {   // the query rows
+    const int m = u / (D >> 3), k = (u - m * (D >> 3)) * 8;
+    *reinterpret_cast<V8<T>*>(qs + m * LDK + k) = m < nrows ? load8(static_cast<const T*>(p.q) + (grow0 + m) * D + k) : zero8<T>();
+  }
+
+  f32x4 o[RT][NT];
+  float mrun[RT][4], lrun[RT][4];
+  int lim[RT][4];   // last key row m sees
+#pragma unroll
+  for (int rt = 0; rt < RT; ++rt) {
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) o[rt][nt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      mrun[rt][r] = -1e30f;
+      lrun[rt][r] = 0.f;
+      lim[rt][r] = ctx + (r0 + rt * 16 + 4 * kc + r) / H;
+    }
+  }
+  const float sc2 = p.scale * 1.4426950408889634f;   // scores in units of log 2
+
+  for (int kt = kt0; kt < kt1; ++kt) {
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+      if (kcol + i * TPK * 8 < D) *reinterpret_cast<V8<T>*>(ks + kj * LDK + kcol + i * TPK * 8) = kr[i];
+    if (kt + 1 < kt1) {
+      load_tile(next_row);
+      next_row = kt + 2 < kt1 ? page_of(kt + 2) : -1;
+    }
+    __syncthreads();
+    f32x4 sc[RT];
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) sc[rt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (wave < SW) {
+      const T* krow = ks + (wave * 16 + r16) * LDK + 8 * kc;
+      const T* qrow = qs + r16 * LDK + 8 * kc;
+#pragma unroll 4
+      for (int k = 0; k < D; k += 32) {
+        const V8<T> kf = load8(krow + k);
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt) mma(sc[rt], load8(qrow + rt * 16 * LDK + k), kf);
+      }
+      const int key = kt * KT + wave * 16 + r16;
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          sc[rt][r] = key <= lim[rt][r] ? sc[rt][r] * sc2 : -INFINITY;   // (keys past kv_end are past every row's limit)
+          float v = sc[rt][r];
+#pragma unroll
+          for (int x = 1; x < 16; x <<= 1) v = fmaxf(v, __shfl_xor(v, x, 64));
+          if (r16 == 0) sx[wave * R + rt * 16 + 4 * kc + r] = v;
+        }
+      }
+    }
+    __syncthreads();
+    bool moved = false;
+    float alpha[RT][4];
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+      f32x4 mx = *reinterpret_cast<const f32x4*>(sx + rt * 16 + 4 * kc);
+#pragma unroll
+      for (int w = 1; w < SW; ++w) {
+        const f32x4 v = *reinterpret_cast<const f32x4*>(sx + w * R + rt * 16 + 4 * kc);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mx[r] = fmaxf(mx[r], v[r]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float mn = fmaxf(mrun[rt][r], mx[r]);
+        alpha[rt][r] = exp2_hw(mrun[rt][r] - mn);
+        moved |= mn != mrun[rt][r];
+        mrun[rt][r] = mn;
+        if (wave < SW) {
+          const T pr = (T)exp2_hw(sc[rt][r] - mn);
+          lrun[rt][r] = fmaf(lrun[rt][r], alpha[rt][r], (float)pr);   // (what is summed is what multiplies the values)
+          ps[(rt * 16 + 4 * kc + r) * LDP + wave * 16 + r16] = pr;
+        }
+      }
+    }
+    if (__ballot(moved)) {
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o[rt][nt][r] *= alpha[rt][r];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < KT; k += 32) {
+      V8<T> pf[RT];
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt) pf[rt] = load8(ps + (rt * 16 + r16) * LDP + k + 8 * kc);
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) {
+        const int dt = d0 + wave + 4 * nt;
+        if (dt < n16) {
+          const V8<T> vf = column8(ks, LDK, k + 8 * kc, dt * 16, r16);
+#pragma unroll
+          for (int rt = 0; rt < RT; ++rt) mma(o[rt][nt], pf[rt], vf);
+        }
+      }
+    }
+    __syncthreads();
+  }
+
+  // the rows' sums: over the 16 keys a lane group held, then over the waves
+#pragma unroll
+  for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      float v = lrun[rt][r];
+#pragma unroll
+      for (int x = 1; x < 16; x <<= 1) v += __shfl_xor(v, x, 64);
+      if (r16 == 0) sx[wave * R + rt * 16 + 4 * kc + r] = v;
+    }
+  __syncthreads();
+#pragma unroll
+  for (int rt = 0; rt < RT; ++rt) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int m = rt * 16 + 4 * kc + r;
+      if (m >= nrows) continue;
+      const float l = sx[m] + sx[R + m] + sx[2 * R + m] + sx[3 * R + m];
+      if (p.splits == 1) {
+        const float inv = 1.f / l;
+        T* out = static_cast<T*>(p.out) + (grow0 + m) * p.rank + r16;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          const int dt = d0 + wave + 4 * nt;
+          if (dt < n16) out[dt * 16] = (T)(o[rt][nt][r] * inv);
+        }
+      } else {
+        float* out = part + (int64_t)m * (p.rank + 2);
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          const int dt = d0 + wave + 4 * nt;
+          if (dt < n16) out[dt * 16 + r16] = o[rt][nt][r];
+        }
+        if (blockIdx.z == 0 && wave == 0 && r16 == 0) {
+          out[p.rank] = mrun[rt][r];
+          out[p.rank + 1] = l;
+        }
+      }
+    }
+  }
+}
+
+// out[row] = sum over splits of 2^(m_s - m) part_s / sum of 2^(m_s - m) l_s; one workgroup per (token, head)
+template <typename T>
+__global__ __launch_bounds__(256) void latent_combine_kernel(const vmi_hy_latent_attention_args p, const vmi_hy_step s) {
+  const int64_t row = blockIdx.x, n = (int64_t)s.T * p.heads;
+  if (s.tok_seq[row / p.heads] < 0) return;
+  const int ld = p.rank + 2;
+  float m = -1e30f;
+  for (int i = 0; i < p.splits; ++i) m = fmaxf(m, p.partial[(i * n + row) * ld + p.rank]);
+  float l = 0.f;
+  for (int i = 0; i < p.splits; ++i) {
+    const float* q = p.partial + (i * n + row) * ld + p.rank;
+    l += exp2_hw(q[0] - m) * q[1];
+  }
+  const float inv = 1.f / l;
+  for (int k = threadIdx.x; k < p.rank; k += blockDim.x) {
+    float a = 0.f;
+#pragma unroll 4
+    for (int i = 0; i < p.splits; ++i) {
+      const float* q = p.partial + (i * n + row) * ld;
+      if (q[p.rank + 1] > 0.f) a = fmaf(exp2_hw(q[p.rank] - m), q[k], a);   // (a part without keys holds no values)
+    }
+    static_cast<T*>(p.out)[row * p.rank + k] = (T)(a * inv);
+  }
+}
+
+// RMS norm of the latent, rotation of the shared key and of the query parts; one workgroup per token
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_prep_args p, const vmi_hy_step s) {
+  extern __shared__ float cs[];   // [rot_n / 2][2]
+  __shared__ float part[4];
+  const int t = blockIdx.x, tid = threadIdx.x, half = p.rot_n >> 1, hd = p.dim + p.rot, D = p.rank + p.rot;
+  if (s.tok_seq[t] < 0) return;
+  const double pos = (double)s.tok_pos[t];
+  for (int i = tid; i < half; i += 256) {   // the angle reduced in fp64: exact to fp32 at any position
+    const double a = pos * p.freq[i];
+    const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
+    cs[2 * i] = cosf(r);
+    cs[2 * i + 1] = sinf(r);
+  }
+  const T* row = static_cast<const T*>(p.proj) + (int64_t)t * p.ldp;
+  const T* lat = row + p.heads * hd;
+  float ss = 0.f;
+  for (int k = tid * 8; k < p.rank; k += 2048) {
+    const f32x8 v = to_f32<T>(load8(lat + k));
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) part[tid >> 6] = ss;
+  __syncthreads();
+  const float rms = 1.f / sqrtf((part[0] + part[1] + part[2] + part[3]) / (float)p.rank_n + p.eps);
+  const int64_t slot = s.tok_slot[t];
+  T* crow = slot >= 0 ? static_cast<T*>(p.cache) + slot * D : nullptr;
+  if (crow) {
+    for (int k = tid * 8; k < p.rank; k += 2048) {
+      f32x8 v = to_f32<T>(load8(lat + k));
+      const f32x8 w = load8(p.norm_w + k);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = v[e] * rms * w[e];
+      *reinterpret_cast<V8<T>*>(crow + k) = from_f32<T>(v);
+    }
+  }
+  // heads 0 .. heads - 1: the query's rotated part; "head" `heads`: the shared key
+  T* qrow = static_cast<T*>(p.q) + (int64_t)t * p.heads * D;
+  for (int u = tid; u < (p.heads + 1) * p.rot; u += 256) {
+    const int h = u / p.rot, i = u - h * p.rot;
+    const T* src = h < p.heads ? row + h * hd + p.dim : lat + p.rank;
+    T* dst = h < p.heads ? qrow + (int64_t)h * D + p.rank : (crow ? crow + p.rank : nullptr);
+    if (!dst) continue;
+    if (i >= p.rot_n) {
+      dst[i] = src[i];   // passes unrotated (padding: zeros)
+    } else if (i < half) {
+      dst[i] = (T)((float)src[i] * cs[2 * i] - (float)src[i + half] * cs[2 * i + 1]);
+    } else {
+      const int j = i - half;
+      dst[i] = (T)((float)src[i] * cs[2 * j] + (float)src[j] * cs[2 * j + 1]);
+    }
+  }
+}
+
+template <typename T, int KT, int RT, int NT, int U>
+static int launch_attention(const vmi_hy_latent_attention_args& p, const vmi_hy_step& s, hipStream_t st) {
+  auto* fn = latent_attention_kernel<T, KT, RT, NT, U>;
+  const size_t lds = attention_lds<T, KT, RT>(p.rank + p.rot);
+  if (int rc = allow_lds(fn, lds, "vmi_hy_latent_attention")) return rc;
+  const int zb = ((p.rank >> 4) + 4 * NT - 1) / (4 * NT);
+  hipLaunchKernelGGL(fn, dim3(p.n_tiles, p.splits, zb), dim3(256), lds, st, p, s);
+  if (p.splits > 1)
+    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3((int64_t)s.T * p.heads), dim3(p.rank > 128 ? 256 : 128), 0, st, p, s);
+  return launched("vmi_hy_latent_attention");
+}
+
+template <typename T, int KT, int RT>
+static int attention_width(const vmi_hy_latent_attention_args& p, const vmi_hy_step& s, hipStream_t st) {
+  const int units = (p.rank + p.rot + 2048 / KT - 1) / (2048 / KT);   // of 8 elements of a cache row, per thread
+  if (p.rank <= 128 && units <= 8) return launch_attention<T, KT, RT, 2, 8>(p, s, st);
+  if (p.rank <= 256 && units <= 12) return launch_attention<T, KT, RT, 4, 12>(p, s, st);
+  if (units <= 20) return launch_attention<T, KT, RT, 8, 20>(p, s, st);
+  if constexpr (RT == 1)
+    if (units <= 32) return launch_attention<T, KT, RT, 8, 32>(p, s, st);
+  return fail(VMI_HY_E_SHAPE, "vmi_hy_latent_attention", "cache rows this long are not built");
+}
+
+// the most row tiles (1, 2, 4; at most `want`) a workgroup can hold beside a tile of 64 keys; fp32 is built for one
+static int row_tiles_for(int D, int want, int dtype) {
+  if (dtype == VMI_HY_BF16 && D <= 640) {
+    if (want >= 4 && attention_lds<b16, 64, 4>(D) <= LDS_PER_CU) return 4;
+    if (want >= 2 && attention_lds<b16, 64, 2>(D) <= LDS_PER_CU) return 2;
+  }
+  return 1;
+}
+
+template <typename T>
+static int run_attention(const vmi_hy_latent_attention_args& p, const vmi_hy_step& s, hipStream_t st) {
+  const int D = p.rank + p.rot;
+  if constexpr (sizeof(T) == 2) {
+    if (p.row_tiles == 4) return attention_width<T, 64, 4>(p, s, st);
+    if (p.row_tiles == 2) return attention_width<T, 64, 2>(p, s, st);
+  }
+  if (p.row_tiles != 1) return fail(VMI_HY_E_ARG, "vmi_hy_latent_attention", "row_tiles is what vmi_hy_latent_row_tiles returns");
+  // tiles of 64 keys where they fit LDS beside the query rows, of 32 otherwise
+  return attention_lds<T, 64, 1>(D) <= LDS_PER_CU ? attention_width<T, 64, 1>(p, s, st) : attention_width<T, 32, 1>(p, s, st);
+}
+
+}  // namespace vmi_hybrid
+
+using namespace vmi_hybrid;
+
+extern "C" {
+
+int vmi_hy_latent_prep(const vmi_hy_latent_prep_args* a, const vmi_hy_step* s, void* stream) {
+  static const char* who = "vmi_hy_latent_prep";
+  if (!a || !s || !a->proj || !a->q || !a->cache || !a->norm_w || !a->freq || !s->tok_seq || !s->tok_pos || !s->tok_slot || s->T <= 0 ||
+      a->heads <= 0 || a->dim <= 0 || a->rot <= 0 || a->rank <= 0 || a->rot_n <= 0 || a->rot_n > a->rot || (a->rot_n & 1) ||
+      a->rank_n <= 0 || a->rank_n > a->rank)
+    return fail(VMI_HY_E_ARG, who, "null pointer or a size out of range");
+  if ((a->dim & 31) || (a->rot & 31) || (a->rank & 31) || (a->ldp & 7) || a->rot_n > 8192)
+    return fail(VMI_HY_E_SHAPE, who, "needs sizes that are multiples of 32");
+  DeviceScope dev(a->device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  const size_t lds = (size_t)a->rot_n * 4;
+  if (a->dtype == VMI_HY_BF16)
+    hipLaunchKernelGGL(latent_prep_kernel<b16>, dim3(s->T), dim3(256), lds, st, *a, *s);
+  else
+    hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(s->T), dim3(256), lds, st, *a, *s);
+  return launched(who);
+}
+
+int32_t vmi_hy_latent_row_tiles(int32_t row_dim, int32_t want, int32_t dtype) { return row_tiles_for(row_dim, want, dtype); }
+
+int vmi_hy_latent_attention(const vmi_hy_latent_attention_args* a, const vmi_hy_step* s, void* stream) {
+  static const char* who = "vmi_hy_latent_attention";
+  if (!a || !s || !a->q || !a->cache || !a->out || !a->tiles || !s->tok_seq || !s->q_start || !s->q_len || !s->ctx || !s->table ||
+      s->T <= 0 || s->table_ld <= 0 || s->page_size <= 0 || a->heads <= 0 || a->rank <= 0 || a->rot <= 0 || a->n_tiles <= 0 ||
+      a->splits <= 0 || a->splits > 65535 || (a->splits > 1 && !a->partial))
+    return fail(VMI_HY_E_ARG, who, "null pointer or a size out of range");
+  if ((a->rank & 31) || (a->rot & 31)) return fail(VMI_HY_E_SHAPE, who, "needs sizes that are multiples of 32");
+  DeviceScope dev(a->device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  return a->dtype == VMI_HY_BF16 ? run_attention<b16>(*a, *s, st) : run_attention<float>(*a, *s, st);
+}
+
+}  // extern "C"

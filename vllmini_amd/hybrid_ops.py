@@ -1,0 +1,313 @@
+"""Operators of libvmi_hybrid.so (include/vmi_hybrid.h): what decoders with recurrent blocks and latent attention are made of.
+
+Thin ctypes wrappers over csrc/hybrid_*.hip that check operands on the host (devices, dtypes, shapes, strides — a kernel never
+sees sizes that do not fit its buffers) and launch on torch's current stream.  There is no torch fallback: a missing library or
+an unsupported shape raises.  Two element types: torch.bfloat16 (what models are served in) and torch.float32 (every product in
+full 32 bits).
+
+    linear            y = epilogue(prologue(x) W^T): layer norm / concatenation in front, residual add / gated unit / head gate behind
+    embed, add_norm, glu, argmax
+    rglru             causal convolution + block-diagonal gates + gated linear recurrence + gelu(y) product
+    latent_prep       RMS norm of the latent, rotary parts, cache write
+    latent_attention  softmax attention in the latent space over the paged cache
+
+StepLayout describes the tokens of one step to the last three.
+"""
+from __future__ import annotations
+
+import ctypes
+import os
+import threading
+from typing import Optional, Tuple
+
+import torch
+
+from . import build as _build
+
+ABI_VERSION = 1
+DTYPES = {torch.bfloat16: 0, torch.float32: 1}
+X_ROWS, X_NORM, X_CONCAT = 0, 1, 2
+E_STORE, E_RESIDUAL, E_FLOAT, E_GLU, E_GATED = 0, 1, 2, 3, 4
+
+_vp, _i32, _i64, _f32 = ctypes.c_void_p, ctypes.c_int32, ctypes.c_int64, ctypes.c_float
+
+
+def _struct(name, fields):
+    return type(name, (ctypes.Structure,), {"_fields_": [(n, t) for t, names in fields for n in names.split()]})
+
+
+LinearArgs = _struct("LinearArgs", [(_vp, "x x2 rows norm_w w bias gate y"), (_i64, "ldx ldy ldg x_gstride y_gstride"),
+                                    (_i32, "M N K groups norm_n n_out"), (_f32, "eps scale"), (_i32, "x_kind epilogue dtype device")])
+StepArgs = _struct("StepArgs", [(_vp, "tok_seq tok_pos tok_slot q_start q_len ctx state_slot flip table"),
+                                (_i32, "T B table_ld page_size")])
+RglruArgs = _struct("RglruArgs", [(_vp, "yx out conv_w conv_b gates gate_b decay state tail scratch carry"), (_i64, "ldx ldo"),
+                                  (_i32, "width blocks taps single spans dtype device")])
+PrepArgs = _struct("PrepArgs", [(_vp, "proj q cache norm_w freq"), (_i64, "ldp"), (_i32, "heads dim rot rank rot_n rank_n"),
+                                (_f32, "eps"), (_i32, "dtype device")])
+AttentionArgs = _struct("AttentionArgs", [(_vp, "q cache out tiles partial"), (_i32, "heads rank rot n_tiles row_tiles splits"),
+                                          (_f32, "scale"), (_i32, "dtype device")])
+
+SIGNATURES = {
+    "vmi_hy_linear": (ctypes.c_int, [ctypes.POINTER(LinearArgs), _vp]),
+    "vmi_hy_embed": (ctypes.c_int, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "vmi_hy_add_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_glu": (ctypes.c_int, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_argmax": (ctypes.c_int, [_vp, _i64, _i32, _i32, _vp, _i32, _vp]),
+    "vmi_hy_rglru": (ctypes.c_int, [ctypes.POINTER(RglruArgs), ctypes.POINTER(StepArgs), _vp]),
+    "vmi_hy_latent_prep": (ctypes.c_int, [ctypes.POINTER(PrepArgs), ctypes.POINTER(StepArgs), _vp]),
+    "vmi_hy_latent_row_tiles": (_i32, [_i32, _i32, _i32]),
+    "vmi_hy_latent_attention": (ctypes.c_int, [ctypes.POINTER(AttentionArgs), ctypes.POINTER(StepArgs), _vp]),
+    "vmi_hybrid_last_error": (ctypes.c_char_p, []),
+    "vmi_hybrid_abi_version": (_i32, []),
+    "vmi_hybrid_target_arch": (ctypes.c_char_p, []),
+}
+
+_lock = threading.Lock()
+_lib = None
+
+
+class HybridLibraryError(RuntimeError):
+    """libvmi_hybrid.so is missing / stale / does not match the header."""
+
+
+def load() -> ctypes.CDLL:
+    global _lib
+    if _lib is None:
+        with _lock:
+            if _lib is None:
+                path = _build.HYBRID_LIB_PATH
+                if not os.path.exists(path):
+                    raise HybridLibraryError(f"{path} not found: build it with `python -m vllmini_amd.build` (or `make hybrid`)")
+                try:
+                    lib = ctypes.CDLL(path)
+                except OSError as e:
+                    raise HybridLibraryError(f"cannot load {path}: {e}") from e
+                for name, (restype, argtypes) in SIGNATURES.items():
+                    try:
+                        fn = getattr(lib, name)
+                    except AttributeError as e:
+                        raise HybridLibraryError(f"{path} does not export {name}") from e
+                    fn.restype, fn.argtypes = restype, argtypes
+                if lib.vmi_hybrid_abi_version() != ABI_VERSION:
+                    raise HybridLibraryError(f"{path}: ABI {lib.vmi_hybrid_abi_version()}, expected {ABI_VERSION}")
+                _lib = lib
+    return _lib
+
+
+def _check(rc: int) -> None:
+    if rc != 0:
+        raise RuntimeError(load().vmi_hybrid_last_error().decode("utf-8", "replace"))
+
+
+def _need(cond: bool, what: str) -> None:
+    if not cond:
+        raise RuntimeError(what)
+
+
+def _ptr(t: Optional[torch.Tensor]):
+    return None if t is None else t.data_ptr()
+
+
+def _on(t: torch.Tensor) -> Tuple[int, int]:
+    _need(t.device.type == "cuda", "hybrid_ops: there is no CPU path")
+    idx = t.device.index if t.device.index is not None else torch.cuda.current_device()
+    return idx, torch.cuda.current_stream(t.device).cuda_stream
+
+
+def pad32(n: int) -> int:
+    return (n + 31) // 32 * 32
+
+
+class MatrixTiles:
+    """Linear weights [N, K] (or a group of them, [G, N, K]) as the tiles the kernels stream, zero-padded to N % 32 == K % 32 == 0:
+    tiles[g][s][t][kc * 16 + r][e] = w[g][16 s + r][32 t + 8 kc + e].  `dense=True` keeps the padded [N, K] as well (steps of many
+    tokens go through the vendor's matrix product)."""
+
+    def __init__(self, weight: torch.Tensor, dtype: torch.dtype, dense: bool = False):
+        w = weight if weight.dim() == 3 else weight[None]
+        G, N, K = w.shape
+        self.groups, self.N, self.K = G, pad32(N), pad32(K)
+        p = torch.zeros((G, self.N, self.K), dtype=dtype, device=w.device)
+        p[:, :N, :K] = w.to(dtype)
+        self.tiles = p.view(G, self.N // 16, 16, self.K // 32, 4, 8).permute(0, 1, 3, 4, 2, 5).contiguous()
+        self.dense = p[0].contiguous() if dense and G == 1 else None
+
+
+def linear(x: torch.Tensor, w: MatrixTiles, *, norm: Optional[Tuple[torch.Tensor, int, float]] = None, x2: Optional[torch.Tensor] = None,
+           rows: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
+           residual: bool = False, float_out: Optional[Tuple[int, float]] = None, glu_limit: Optional[float] = None,
+           gate: Optional[torch.Tensor] = None, x_gstride: int = 0, y_gstride: int = 0) -> torch.Tensor:
+    """One linear layer over the rows of x.
+        input     x [M, K] of the element type | norm=(weight, n, eps): x float32, layer norm over its first n columns, optionally
+                  of `rows` only | x2: x and x2 float32 side by side
+        output    element type (+ bias) | residual=True: out (float32) += | float_out=(columns, scale): float32 | glu_limit: the
+                  clamped gated unit of interleaved (gate, up) columns | gate [M, groups ...]: times sigmoid of the group's column
+        groups    group g reads x at column g * x_gstride, writes out at column g * y_gstride"""
+    lib = load()
+    device, stream = _on(x)
+    T = w.tiles.dtype
+    kind = X_NORM if norm is not None else X_CONCAT if x2 is not None else X_ROWS
+    epi = E_RESIDUAL if residual else E_FLOAT if float_out else E_GLU if glu_limit is not None else E_GATED if gate is not None else E_STORE
+    M = int(rows.numel()) if rows is not None else int(x.shape[0])
+    K, N = w.K, w.N
+    span = (w.groups - 1) * x_gstride + (K // 2 if kind == X_CONCAT else K)
+    _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[1] >= span and x.dtype == (T if kind == X_ROWS else torch.float32),
+          f"hybrid_ops.linear: x {tuple(x.shape)} {x.dtype} does not hold {w.groups} x {K} columns")
+    if x2 is not None:
+        _need(x2.shape == x.shape and x2.stride() == x.stride() and x2.dtype == torch.float32 and x2.device == x.device,
+              "hybrid_ops.linear: x2 must match x")
+    if norm is not None:
+        _need(norm[0].dtype == torch.float32 and norm[0].numel() >= K and 0 < norm[1] <= K, "hybrid_ops.linear: norm weight float32 [K]")
+    if rows is not None:
+        _need(kind == X_NORM and rows.dtype == torch.int32 and rows.is_contiguous(), "hybrid_ops.linear: rows int32, with norm")
+    if bias is not None:
+        _need(bias.dtype == torch.float32 and bias.numel() >= N, "hybrid_ops.linear: bias float32 [N]")
+    if gate is not None:
+        _need(gate.dtype == T and gate.shape[0] == M and gate.stride(1) == 1 and gate.shape[1] >= w.groups, "hybrid_ops.linear: gate")
+    cols = float_out[0] if epi == E_FLOAT else N // 2 if epi == E_GLU else (w.groups - 1) * y_gstride + N
+    odt = torch.float32 if epi in (E_RESIDUAL, E_FLOAT) else T
+    if out is None:
+        out = torch.empty((M, cols), dtype=odt, device=x.device)
+    _need(out.dim() == 2 and out.shape[0] == M and out.shape[1] >= cols and out.stride(1) == 1 and out.dtype == odt
+          and out.data_ptr() != x.data_ptr(), f"hybrid_ops.linear: out {tuple(out.shape)} {out.dtype} for {M} x {cols}")
+    a = LinearArgs(x=x.data_ptr(), x2=_ptr(x2), rows=_ptr(rows), norm_w=norm[0].data_ptr() if norm else None, w=w.tiles.data_ptr(),
+                   bias=_ptr(bias), gate=_ptr(gate), y=out.data_ptr(), ldx=x.stride(0), ldy=out.stride(0),
+                   ldg=gate.stride(0) if gate is not None else 0, x_gstride=x_gstride, y_gstride=y_gstride, M=M, N=N, K=K,
+                   groups=w.groups, norm_n=norm[1] if norm else 0, n_out=float_out[0] if float_out else 0,
+                   eps=norm[2] if norm else 0.0, scale=float_out[1] if float_out else glu_limit if glu_limit is not None else 1.0,
+                   x_kind=kind, epilogue=epi, dtype=DTYPES[T], device=device)
+    _check(lib.vmi_hy_linear(ctypes.byref(a), stream))
+    return out
+
+
+def embed(ids: torch.Tensor, table: torch.Tensor, width: int, scale: float) -> torch.Tensor:
+    """float32 [T, ld] = table[ids] * scale, zero past `width` (table bfloat16 [vocab, ld])."""
+    device, stream = _on(ids)
+    _need(ids.dtype == torch.int64 and ids.dim() == 1 and ids.is_contiguous() and table.dtype == torch.bfloat16
+          and table.is_contiguous() and table.device == ids.device, "hybrid_ops.embed: int64 ids, bfloat16 table on one device")
+    T, ld = ids.numel(), table.shape[1]
+    x = torch.empty((T, ld), dtype=torch.float32, device=ids.device)
+    _check(load().vmi_hy_embed(ids.data_ptr(), table.data_ptr(), x.data_ptr(), T, width, ld, table.shape[0], float(scale), device, stream))
+    return x
+
+
+def add_norm(x: torch.Tensor, add: Optional[torch.Tensor], norm: Optional[Tuple[torch.Tensor, int, float]],
+             dtype: torch.dtype) -> Optional[torch.Tensor]:
+    """x += add (if given), then the layer norm of x in `dtype` (if asked for)."""
+    device, stream = _on(x)
+    T, ld = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "hybrid_ops.add_norm: x float32, contiguous")
+    if add is not None:
+        _need(add.shape[0] == T and add.shape[1] >= ld and add.stride(1) == 1 and add.dtype == dtype, "hybrid_ops.add_norm: add")
+    out = None
+    if norm is not None:
+        _need(norm[0].dtype == torch.float32 and norm[0].numel() >= ld, "hybrid_ops.add_norm: norm weight float32 [ld]")
+        out = torch.empty((T, ld), dtype=dtype, device=x.device)
+    _check(load().vmi_hy_add_norm(x.data_ptr(), _ptr(add), add.stride(0) if add is not None else 0, norm[0].data_ptr() if norm else None,
+                                  _ptr(out), T, norm[1] if norm else ld, ld, norm[2] if norm else 0.0, DTYPES[dtype], device, stream))
+    return out
+
+
+def glu(x: torch.Tensor, limit: float) -> torch.Tensor:
+    """The clamped gated unit of interleaved (gate, up) columns: [T, 2 n] -> [T, n]."""
+    device, stream = _on(x)
+    T, n = x.shape[0], x.shape[1] // 2
+    _need(x.stride(1) == 1 and x.dtype in DTYPES, "hybrid_ops.glu: rows of unit stride")
+    out = torch.empty((T, n), dtype=x.dtype, device=x.device)
+    for t in range(0, T, 65535):      # (a launch's grid holds that many rows)
+        m = min(65535, T - t)
+        _check(load().vmi_hy_glu(x[t:].data_ptr(), x.stride(0), out[t:].data_ptr(), n, m, n, float(limit), DTYPES[x.dtype], device, stream))
+    return out
+
+
+def argmax(logits: torch.Tensor) -> torch.Tensor:
+    device, stream = _on(logits)
+    _need(logits.dim() == 2 and logits.dtype == torch.float32 and logits.stride(1) == 1, "hybrid_ops.argmax: float32 [B, V]")
+    out = torch.empty((logits.shape[0],), dtype=torch.int64, device=logits.device)
+    _check(load().vmi_hy_argmax(logits.data_ptr(), logits.stride(0), logits.shape[0], logits.shape[1], out.data_ptr(), device, stream))
+    return out
+
+
+ROW_TILE = 64      # rows of a tile of the recurrence's kernel
+
+
+class StepLayout:
+    """The tokens of a step on the device: `fields` maps the names of vmi_hy_step to int32 tensors; `single`: every portion is one
+    token; `spans`: some portion crosses a row tile."""
+
+    def __init__(self, fields: dict, T: int, B: int, page_size: int, single: bool, spans: bool, max_len: int, max_keys: int):
+        for name in ("tok_seq", "tok_pos", "tok_slot"):
+            _need(fields[name].dtype == torch.int32 and fields[name].numel() >= T and fields[name].is_contiguous(), f"StepLayout: {name}")
+        for name in ("q_start", "q_len", "ctx", "state_slot", "flip"):
+            _need(fields[name].dtype == torch.int32 and fields[name].numel() >= B and fields[name].is_contiguous(), f"StepLayout: {name}")
+        tab = fields["table"]
+        _need(tab.dtype == torch.int32 and tab.dim() == 2 and tab.shape[0] >= B and tab.is_contiguous(), "StepLayout: table")
+        self.fields = fields      # (keeps the tensors alive)
+        self.T, self.B, self.single, self.spans = T, B, single, spans
+        self.max_len, self.max_keys = max_len, max_keys      # longest portion, most keys any token sees
+        self.args = StepArgs(**{k: fields[k].data_ptr() for k in ("tok_seq", "tok_pos", "tok_slot", "q_start", "q_len", "ctx",
+                                                                  "state_slot", "flip", "table")},
+                             T=T, B=B, table_ld=tab.shape[1], page_size=page_size)
+        self.ref = ctypes.byref(self.args)
+
+
+def rglru(yx: torch.Tensor, step: StepLayout, *, conv_w: torch.Tensor, conv_b: torch.Tensor, gates: torch.Tensor, gate_b: torch.Tensor,
+          decay: torch.Tensor, blocks: int, state: torch.Tensor, tail: Optional[torch.Tensor]) -> torch.Tensor:
+    """yx [T, 2 width] -> [T, width]; state float32 [slots, width] and tail [slots, 2, taps - 1, width] are updated."""
+    device, stream = _on(yx)
+    T, width, taps = step.T, state.shape[1], conv_w.shape[0]
+    bw = width // blocks
+    _need(yx.shape == (T, 2 * width) and yx.is_contiguous() and width % blocks == 0 and conv_w.shape == (taps, width)
+          and conv_b.numel() == width and gates.numel() == 2 * blocks * bw * bw and gates.dtype == yx.dtype and gate_b.numel() == 2 * width
+          and decay.numel() == width and state.dtype == torch.float32 and state.is_contiguous(), "hybrid_ops.rglru: operand sizes")
+    for t in (conv_w, conv_b, gate_b, decay):
+        _need(t.dtype == torch.float32 and t.is_contiguous(), "hybrid_ops.rglru: float32 constants")
+    if taps > 1:
+        _need(tail is not None and tail.shape == (state.shape[0], 2, taps - 1, width) and tail.dtype == yx.dtype and tail.is_contiguous(),
+              "hybrid_ops.rglru: tail [slots, 2, taps - 1, width]")
+    out = torch.empty((T, width), dtype=yx.dtype, device=yx.device)
+    scratch = carry = None
+    if not step.single:
+        scratch = torch.empty((2, T, width), dtype=torch.float32, device=yx.device)
+        carry = torch.empty((-(-T // ROW_TILE), width), dtype=torch.float32, device=yx.device)
+    a = RglruArgs(yx=yx.data_ptr(), out=out.data_ptr(), conv_w=conv_w.data_ptr(), conv_b=conv_b.data_ptr(), gates=gates.data_ptr(),
+                  gate_b=gate_b.data_ptr(), decay=decay.data_ptr(), state=state.data_ptr(), tail=_ptr(tail) if taps > 1 else None,
+                  scratch=_ptr(scratch), carry=_ptr(carry), ldx=yx.stride(0), ldo=width, width=width, blocks=blocks, taps=taps,
+                  single=int(step.single), spans=int(step.spans), dtype=DTYPES[yx.dtype], device=device)
+    _check(load().vmi_hy_rglru(ctypes.byref(a), step.ref, stream))
+    return out
+
+
+def latent_prep(proj: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, step: StepLayout, *, norm_w: torch.Tensor, freq: torch.Tensor,
+                heads: int, dim: int, rot: int, rank: int, rot_n: int, rank_n: int, eps: float) -> None:
+    device, stream = _on(proj)
+    D = rank + rot
+    _need(proj.shape[0] == step.T and proj.shape[1] >= heads * (dim + rot) + D and proj.stride(1) == 1 and q.dtype == proj.dtype
+          and q.shape == (step.T, heads * D) and q.is_contiguous() and cache.dtype == proj.dtype and cache.shape[-1] == D
+          and cache.is_contiguous() and norm_w.numel() == rank and norm_w.dtype == torch.float32 and freq.dtype == torch.float64
+          and freq.numel() == rot_n // 2, "hybrid_ops.latent_prep: operand sizes")
+    a = PrepArgs(proj=proj.data_ptr(), q=q.data_ptr(), cache=cache.data_ptr(), norm_w=norm_w.data_ptr(), freq=freq.data_ptr(),
+                 ldp=proj.stride(0), heads=heads, dim=dim, rot=rot, rank=rank, rot_n=rot_n, rank_n=rank_n, eps=eps,
+                 dtype=DTYPES[proj.dtype], device=device)
+    _check(load().vmi_hy_latent_prep(ctypes.byref(a), step.ref, stream))
+
+
+def latent_row_tiles(row_dim: int, want: int, dtype: torch.dtype) -> int:
+    return int(load().vmi_hy_latent_row_tiles(row_dim, want, DTYPES[dtype]))
+
+
+def latent_attention(q: torch.Tensor, cache: torch.Tensor, step: StepLayout, tiles: torch.Tensor, *, heads: int, rank: int, rot: int,
+                     scale: float, row_tiles: int, splits: int) -> torch.Tensor:
+    """q [T, heads * (rank + rot)] -> [T, heads * rank] over the cache's pages."""
+    device, stream = _on(q)
+    _need(q.shape == (step.T, heads * (rank + rot)) and q.is_contiguous() and cache.dtype == q.dtype and cache.dim() == 3
+          and cache.shape[1] == step.args.page_size and cache.shape[2] == rank + rot and cache.is_contiguous()
+          and tiles.dtype == torch.int32 and tiles.dim() == 2 and tiles.shape[1] == 2 and tiles.is_contiguous(),
+          "hybrid_ops.latent_attention: operand sizes")
+    out = torch.empty((step.T, heads * rank), dtype=q.dtype, device=q.device)
+    partial = torch.empty((splits, step.T * heads, rank + 2), dtype=torch.float32, device=q.device) if splits > 1 else None
+    a = AttentionArgs(q=q.data_ptr(), cache=cache.data_ptr(), out=out.data_ptr(), tiles=tiles.data_ptr(), partial=_ptr(partial),
+                      heads=heads, rank=rank, rot=rot, n_tiles=tiles.shape[0], row_tiles=row_tiles, splits=splits, scale=scale,
+                      dtype=DTYPES[q.dtype], device=device)
+    _check(load().vmi_hy_latent_attention(ctypes.byref(a), step.ref, stream))
+    return out

@@ -31,10 +31,20 @@ Reference quirks that are reproduced or flagged, not silently changed:
     sequence can use at most max_blocks_per_seq-1 blocks per layer before the next step fails; that
     raises here (the reference dies with UnboundLocalError);
   * exhaustion raises RuntimeError with the reference's messages (kv_cache.py:22-23, 57-58).
+
+Two things a model other than GPT-2 may ask of the same pool (vllmini_amd/hybrid_decoder.py):
+  * `page_rows=[n, ...]`: instead of key / value pages, one tensor [num_blocks, block_size, n] of row pages per cache the model
+    keeps (a latent row per token, say).  Every sequence then has ONE block list (num_layers = 1): block b holds the same
+    tokens in all of those tensors;
+  * `state=[(shape, dtype), ...]`, `state_slots=n`: fixed-size per-sequence state (a recurrence's, a convolution's tail),
+    one tensor [n, *shape] each; a sequence holds one slot from open() to free().  `state_parity` counts its steps modulo 2,
+    for state that is written to the half a step does not read.
+open() + append() advance sequences by portions of any length: what a decode step (one token each), a whole prompt and a piece
+of a prompt have in common.  append() is all or nothing: when blocks run out it has changed nothing.
 """
 from __future__ import annotations
 
-from typing import Dict, List, Sequence, Tuple
+from typing import Dict, List, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
@@ -46,7 +56,9 @@ class PagedKVPool:
     def __init__(self, num_blocks: int, num_heads: int, head_size: int, block_size: int,
                  max_blocks_per_seq: int, num_layers: int, device: torch.device | str = "cuda",
                  allocate_tensors: bool = True, max_seqs: int = 64, multi_block_prefill: bool = True,
-                 kv_cache_dtype: str = "auto", kv_scale: float = 1.0, host_blocks: int = 0):
+                 kv_cache_dtype: str = "auto", kv_scale: float = 1.0, host_blocks: int = 0,
+                 page_rows: Optional[Sequence[int]] = None, page_dtype: torch.dtype = torch.bfloat16,
+                 state: Sequence[Tuple[Sequence[int], torch.dtype]] = (), state_slots: int = 0):
         self.num_blocks = num_blocks
         self.num_heads = num_heads
         self.head_size = head_size
@@ -62,7 +74,21 @@ class PagedKVPool:
             # E5M2 pages are outside the hot path (include/vmi_paged_attention_extras.h): say so HERE, not at the first launch
             from . import _lib
             _lib.require_extras("PagedKVPool(kv_cache_dtype='fp8_e5m2'): operators over fp8-E5M2 pages")
-        if allocate_tensors:
+        self.page_rows = None if page_rows is None else [int(n) for n in page_rows]
+        self.page_dtype = page_dtype
+        self.row_pages: List[torch.Tensor] = []
+        self.state: List[torch.Tensor] = []
+        self.state_slots = int(state_slots)
+        self._free_slots: List[int] = list(range(self.state_slots))
+        self._slot_of: Dict[int, int] = {}
+        if page_rows is not None:
+            if num_layers != 1:
+                raise ValueError("row pages share one block list per sequence: num_layers must be 1")
+            self.key_cache = self.value_cache = None
+            if allocate_tensors:
+                self.row_pages = [torch.zeros(num_blocks, block_size, n, dtype=page_dtype, device=self.device) for n in self.page_rows]
+                self.state = [torch.zeros((self.state_slots, *shape), dtype=dt, device=self.device) for shape, dt in state]
+        elif allocate_tensors:
             # kv_cache.py:13-14 — ONE pool shared by all layers
             x, dt = (16, torch.uint8) if kv_cache_dtype in ("fp8", "fp8_e4m3", "fp8_e5m2") else (X, torch.float16)
             self.key_cache = torch.zeros(num_blocks, num_heads, head_size // x, block_size, x,
@@ -77,6 +103,7 @@ class PagedKVPool:
         # swap_out; host_blocks = 0 -> as many as the device pool.  swapped[seq_id] = everything needed to put the sequence back
         self.host_blocks = int(host_blocks) or num_blocks
         self.host_key_cache = self.host_value_cache = None
+        self.host_row_pages: List[torch.Tensor] = []
         self._host_free: List[int] = list(range(self.host_blocks))
         self.swapped: Dict[int, dict] = {}
         self.swap_stats = {"swap_outs": 0, "swap_ins": 0, "blocks_out": 0, "blocks_in": 0, "bytes_out": 0, "bytes_in": 0}
@@ -92,13 +119,15 @@ class PagedKVPool:
         nblocks = np.zeros((L, n), dtype=np.int64)
         filled = np.zeros((L, n), dtype=np.int64)
         seq_len = np.zeros(n, dtype=np.int64)
+        parity = np.zeros(n, dtype=np.int64)
         if self._rows:
             tables[:, : self._rows] = self._tables
             nblocks[:, : self._rows] = self._nblocks
             filled[:, : self._rows] = self._filled
             seq_len[: self._rows] = self._seq_len
+            parity[: self._rows] = self._parity
         self._free_rows.extend(range(self._rows, n))
-        self._tables, self._nblocks, self._filled, self._seq_len = tables, nblocks, filled, seq_len
+        self._tables, self._nblocks, self._filled, self._seq_len, self._parity = tables, nblocks, filled, seq_len, parity
         self._rows = n
 
     def _new_row(self, seq_id: int) -> int:
@@ -159,17 +188,86 @@ class PagedKVPool:
             self._tables[:, row, :] = -1
             self._nblocks[:, row] = 0
             self._free_rows.append(row)
+            slot = self._slot_of.pop(seq_id, None)
+            if slot is not None:
+                self._free_slots.append(slot)
+
+    # ---- portions of any length ----------------------------------------------------------------------------------------
+    @property
+    def free_state_slots(self) -> int:
+        return len(self._free_slots)
+
+    def _take_slot(self, seq_id: int) -> None:
+        if self.state_slots:
+            if not self._free_slots:
+                raise RuntimeError(f"Not enough free blocks: all {self.state_slots} state slots are taken")
+            self._slot_of[seq_id] = self._free_slots.pop(0)
+
+    def open(self, seq_id: int) -> None:
+        """A new sequence without tokens: a table row and, where the model keeps state, a slot (its contents are whatever the
+        last owner left: a portion that starts at position 0 starts from zeros by itself)."""
+        if seq_id in self.allocated_blocks:
+            raise ValueError(f"sequence {seq_id} already allocated")
+        self._take_slot(seq_id)
+        self.allocated_blocks[seq_id] = []
+        row = self._new_row(seq_id)
+        self._tables[:, row, :] = -1
+        self._nblocks[:, row] = 0
+        self._filled[:, row] = self.block_size       # (full: the first token opens a block)
+        self._seq_len[row] = 0
+        self._parity[row] = 0
+
+    def append(self, seq_ids: Sequence[int], counts: Sequence[int]) -> dict:
+        """counts[i] more tokens for seq_ids[i] -> what a step over those tokens needs (numpy):
+             tables [layers, B, MB] int32, slots [layers, sum(counts)] int64 (entry by entry), ctx [B] the lengths before,
+             state_slot [B], parity [B] (before this step)
+        All or nothing: RuntimeError("No free blocks available") / a full table leaves the pool as it was."""
+        B, bs, L, MB = len(seq_ids), self.block_size, self.num_layers, self.max_blocks_per_seq
+        rows = np.fromiter((self._row_of[s] for s in seq_ids), dtype=np.int64, count=B)
+        n = np.asarray(counts, dtype=np.int64)
+        if (n <= 0).any() or len(set(seq_ids)) != B:
+            raise ValueError("append: every sequence once, with at least one token")
+        ctx = self._seq_len[rows].copy()
+        total = ctx + n
+        have = self._nblocks[0, rows]                # (the layers advance together)
+        more = -(-total // bs) - have
+        if (have + more > MB).any():
+            b = int(np.argmax(have + more))
+            raise RuntimeError(f"sequence {seq_ids[b]}: {int(total[b])} tokens need more than the {MB} blocks per layer of its table")
+        if int(more.sum()) * L > len(self.free_blocks):
+            raise RuntimeError("No free blocks available")
+        for b in np.flatnonzero(more):
+            k = int(more[b])
+            new = np.asarray(self._take(k * L), dtype=np.int32)
+            self._tables[:, rows[b], have[b]:have[b] + k] = new.reshape(k, L).T
+            self.allocated_blocks[seq_ids[b]].extend(int(x) for x in new)
+        self._nblocks[:, rows] += more
+        self._filled[:, rows] = total - (-(-total // bs) - 1) * bs
+        self._seq_len[rows] = total
+        parity = self._parity[rows].copy()
+        self._parity[rows] ^= 1
+        tables = self._tables[:, rows, :]
+        of = np.repeat(np.arange(B), n)
+        pos = np.arange(int(n.sum()), dtype=np.int64) - np.repeat(np.cumsum(n) - n, n) + np.repeat(ctx, n)
+        slots = tables[:, of, pos // bs].astype(np.int64) * bs + pos % bs
+        slot = np.fromiter((self._slot_of.get(s, 0) for s in seq_ids), dtype=np.int64, count=B)
+        return {"tables": tables, "slots": slots, "ctx": ctx, "pos": pos, "entry": of, "state_slot": slot, "parity": parity}
 
     # ---- preemption: a sequence's blocks to host memory and back (block_manager.py:70-87) -------------------------------
     @property
     def block_bytes(self) -> int:
-        """Bytes of one block of ONE cache (K and V blocks have the same size)."""
+        """Bytes of one block of ONE cache (K and V blocks have the same size; row pages: half of a block of all tensors)."""
+        if self.page_rows is not None:
+            return sum(self.page_rows) * self.block_size * torch.empty((), dtype=self.page_dtype).element_size() // 2
         esz = 1 if self.kv_cache_dtype in ("fp8", "fp8_e4m3", "fp8_e5m2") else 2
         return self.num_heads * self.head_size * self.block_size * esz
 
     def reserve_host(self) -> None:
         """Allocate the pinned host pool now (else at the first swap_out: pinning host_blocks x 2 x block_bytes takes a
         fraction of a second per GB — a server does it at start-up, not under its first preemption)."""
+        if self.row_pages and not self.host_row_pages:
+            self.host_row_pages = [torch.empty((self.host_blocks,) + tuple(t.shape[1:]), dtype=t.dtype,
+                                               pin_memory=self.device.type == "cuda") for t in self.row_pages]
         if self.key_cache is not None and self.host_key_cache is None:
             pin = self.device.type == "cuda"    # pinned: the GPU reads / writes these pages directly (one launch per swap)
             self.host_key_cache = torch.empty((self.host_blocks,) + tuple(self.key_cache.shape[1:]),
@@ -177,7 +275,24 @@ class PagedKVPool:
             self.host_value_cache = torch.empty((self.host_blocks,) + tuple(self.value_cache.shape[1:]),
                                                 dtype=self.value_cache.dtype, pin_memory=pin)
 
+    def _move_row_pages(self, to_host: bool, pairs: np.ndarray) -> None:
+        """The same move for row pages: the batched launch takes two tensors of one block size, so tensors go in pairs (an odd
+        one out rides with itself)."""
+        from . import cache_ops
+        self.reserve_host()
+        by_size: Dict[int, List[int]] = {}
+        for i, t in enumerate(self.row_pages):
+            by_size.setdefault(t[0].numel(), []).append(i)
+        m = torch.from_numpy(np.ascontiguousarray(pairs))
+        for idx in by_size.values():
+            for j in range(0, len(idx), 2):
+                a, b = idx[j], idx[min(j + 1, len(idx) - 1)]
+                src, dst = (self.row_pages, self.host_row_pages) if to_host else (self.host_row_pages, self.row_pages)
+                cache_ops.swap_blocks_batched(src[a], src[b], dst[a], dst[b], m)
+
     def _move_blocks(self, to_host: bool, pairs: np.ndarray) -> None:
+        if len(pairs) and self.row_pages:
+            self._move_row_pages(to_host, pairs)
         if self.key_cache is None:          # bookkeeping only (CPU tests)
             return
         from . import cache_ops
@@ -203,7 +318,9 @@ class PagedKVPool:
         row = self._row_of[seq_id]
         self.swapped[seq_id] = {"host": host, "dev": list(blocks), "tables": self._tables[:, row, :].copy(),
                                 "nblocks": self._nblocks[:, row].copy(), "filled": self._filled[:, row].copy(),
-                                "seq_len": int(self._seq_len[row])}
+                                "seq_len": int(self._seq_len[row]), "parity": int(self._parity[row]),
+                                # (a slot's state is a few rows: it waits in device memory of its own)
+                                "state": [t[self._slot_of[seq_id]].clone() for t in self.state]}
         self._move_blocks(True, np.stack([np.asarray(blocks, dtype=np.int64), np.asarray(host, dtype=np.int64)], axis=1))
         self.free(seq_id)
         st = self.swap_stats
@@ -220,8 +337,11 @@ class PagedKVPool:
         if st is None:
             return False                                                    # :76-77
         n = len(st["host"])
-        if len(self.free_blocks) < n:
+        if len(self.free_blocks) < n or (self.state_slots and not self._free_slots):
             return False                                                    # :86-87
+        self._take_slot(seq_id)
+        for t, kept in zip(self.state, st["state"]):
+            t[self._slot_of[seq_id]].copy_(kept)
         new = self._take(n)
         lut = np.full(self.num_blocks, -1, dtype=np.int32)
         lut[np.asarray(st["dev"], dtype=np.int64)] = np.asarray(new, dtype=np.int32)
@@ -231,6 +351,7 @@ class PagedKVPool:
         self._nblocks[:, row] = st["nblocks"]
         self._filled[:, row] = st["filled"]
         self._seq_len[row] = st["seq_len"]
+        self._parity[row] = st["parity"]
         self.allocated_blocks[seq_id] = list(new)
         self._move_blocks(False, np.stack([np.asarray(st["host"], dtype=np.int64), np.asarray(new, dtype=np.int64)], axis=1))
         self._host_free.extend(st["host"])
