@@ -131,6 +131,13 @@ def build_parser():
     ap.add_argument("--serve-no-deferred-scatter", action="store_true", help="the reference's call pair per layer instead")
     ap.add_argument("--serve-eager", action="store_true", help="plain launches instead of hipGraph replay")
     ap.add_argument("--no-serve", action="store_true", help="skip the extra serving-loop measurement")
+    ap.add_argument("--design", default="", choices=("", "voduvik"),
+                    help="prefill and decode throughput of another registered design at sizes of a real model's layers, beside GPT-2 "
+                         "of equal width and depth (random weights; its own JSON, not the headline line)")
+    ap.add_argument("--design-width", type=int, default=0, help="one width only (default: 1024, 2048 and 4096)")
+    ap.add_argument("--design-part", default="all", choices=("all", "decode", "prefill"))
+    ap.add_argument("--design-model", default="both", choices=("both", "design", "gpt2"))
+    ap.add_argument("--design-batch", type=int, default=0, help="one decode batch only (default: 1, 32 and 256)")
     ap.add_argument("--min-timed-ms", type=float, default=50.0,
                     help="repeat the K-step timed region until the regions hold this many ms in all; the line reports the MEDIAN region")
     ap.add_argument("--headline-only", action="store_true",
@@ -865,6 +872,112 @@ def run_serve(args, dev, rank):
             json.dump(res, f, indent=1)
 
 
+DESIGN_CONTEXT, DESIGN_PROMPTS, DESIGN_VOCAB = 1024, 4, 50257
+
+
+def voduvik_config(width):
+    """Six layers in the proportions of a small production model (per head 128 + 64 query dimensions over latents of 512 + 64, gate
+    blocks of 256 channels, a feed-forward of three widths), the first two of them run twice: eight layer runs."""
+    ff = {"kind": "dense", "ff": 3 * width, "limit": 7.0}
+    rec = {"type": "rglru", "mixer": {"width": width, "blocks": width // 256, "conv": 4}, "mlp": ff}
+    att = {"type": "latent_attention", "mlp": ff,
+           "mixer": {"heads": width // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                     "rot": {"base": 10000.0, "dims": 64}}}
+    return {"architecture": "Voduvik", "vocab": DESIGN_VOCAB, "width": width, "layers": [rec, rec, att, rec, rec, att],
+            "loop": {"start": 0, "stop": 2, "times": 2}, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5}, "logit_scale": 1.0}
+
+
+def design_decoders(width, batch, dev, which):
+    """(name, decoder) of the design and of GPT-2 with the same width and as many layers as the design has runs; pools sized for
+    `batch` sequences of DESIGN_CONTEXT tokens and for the prompts."""
+    tokens = max(batch * (DESIGN_CONTEXT + 128), DESIGN_PROMPTS * (DESIGN_CONTEXT + 64))
+    if which == "design":
+        from vllmini_amd.hybrid_decoder import HybridDecoder
+        from vllmini_amd.voduvik import VoduvikConfig, build_model, random_tensors
+
+        cfg = VoduvikConfig.from_json(voduvik_config(width))
+        model = build_model(cfg, random_tensors(cfg, dev), torch.bfloat16, dev)
+        return HybridDecoder(model, model.make_pool(tokens, max(batch, DESIGN_PROMPTS), 64, DESIGN_CONTEXT + 128))
+    from vllmini_amd.gpt2_decode import GPT2Dims, GPT2PagedDecoder, random_state_dict
+    from vllmini_amd.kv_pool import PagedKVPool
+
+    dims = GPT2Dims(vocab_size=DESIGN_VOCAB, n_positions=DESIGN_CONTEXT + 128, n_embd=width, n_layer=8, n_head=width // 64)
+    pool = PagedKVPool(-(-tokens // 16) * dims.n_layer, dims.n_head, 64, 16, (DESIGN_CONTEXT + 128) // 16 + 1, dims.n_layer, device=dev,
+                       max_seqs=max(batch, DESIGN_PROMPTS))
+    return GPT2PagedDecoder(dims, random_state_dict(dims, dev), pool)
+
+
+def design_decode(dec, batch, dev, steps):
+    """ms per decode step of `batch` sequences around DESIGN_CONTEXT tokens (synthetic contexts: the pages hold random rows),
+    replayed from a hipGraph."""
+    pool, ids = dec.pool, list(range(batch))
+    if getattr(pool, "page_rows", None) is not None:
+        for t in pool.row_pages:
+            t.normal_()
+        for s in ids:
+            pool.open(s)
+            pool.append([s], [DESIGN_CONTEXT])
+    else:
+        pool.key_cache.uniform_(-1, 1)
+        pool.value_cache.uniform_(-1, 1)
+        for s in ids:
+            pool.allocate_for_prefill(s, DESIGN_CONTEXT)
+    tok = torch.randint(0, DESIGN_VOCAB, (batch,), device=dev)
+    for _ in range(4):
+        dec.decode(ids, tok, use_graph=True)
+    times = []
+    for _ in range(3):
+        torch.cuda.synchronize(dev)
+        t0 = time.perf_counter()
+        for _ in range(steps):
+            dec.decode(ids, tok, use_graph=True)
+        torch.cuda.synchronize(dev)
+        times.append((time.perf_counter() - t0) / steps * 1e3)
+    for s in ids:
+        pool.free(s)
+    return statistics.median(times)
+
+
+def design_prefill(dec, dev, repeats=3):
+    """ms for DESIGN_PROMPTS prompts of DESIGN_CONTEXT tokens in one prefill call."""
+    prompts = [torch.randint(0, DESIGN_VOCAB, (DESIGN_CONTEXT,)).tolist() for _ in range(DESIGN_PROMPTS)]
+    times = []
+    for r in range(repeats + 1):
+        ids = [10_000 + r * DESIGN_PROMPTS + i for i in range(DESIGN_PROMPTS)]
+        torch.cuda.synchronize(dev)
+        t0 = time.perf_counter()
+        dec.prefill_batch(ids, prompts)
+        torch.cuda.synchronize(dev)
+        times.append((time.perf_counter() - t0) * 1e3)
+        for s in ids:
+            dec.pool.free(s)
+    return statistics.median(times[1:])
+
+
+def run_design(args, dev):
+    rows = []
+    for width in [args.design_width] if args.design_width else [1024, 2048, 4096]:
+        for which in ("design", "gpt2") if args.design_model == "both" else (args.design_model,):
+            for batch in [args.design_batch] if args.design_batch else [1, 32, 256]:
+                dec = design_decoders(width, batch, dev, which)
+                row = {"model": args.design if which == "design" else "gpt2", "width": width, "layer_runs": 8, "batch": batch,
+                       "context": DESIGN_CONTEXT, "dtype": "bf16" if which == "design" else "f16", "data": "synthetic"}
+                if args.design_part != "prefill":
+                    ms = design_decode(dec, batch, dev, min(args.steps, 30))
+                    row.update(decode_ms_per_step=ms, decode_tokens_per_s=batch / ms * 1e3)
+                if args.design_part != "decode" and batch == (args.design_batch or 32):
+                    ms = design_prefill(dec, dev)
+                    row.update(prefill_ms=ms, prefill_tokens=DESIGN_PROMPTS * DESIGN_CONTEXT,
+                               prefill_tokens_per_s=DESIGN_PROMPTS * DESIGN_CONTEXT / ms * 1e3)
+                rows.append(row)
+                print(json.dumps(row), flush=True)
+                del dec
+                torch.cuda.empty_cache()
+    os.makedirs(os.path.join(REPO, "gpurun_out"), exist_ok=True)
+    with open(os.path.join(REPO, "gpurun_out", f"design_{args.design}.json"), "w") as f:
+        json.dump(rows, f, indent=1)
+
+
 def run_e2e(args, cfg, dist, rank, world, dev):
     res = e2e_measure(args, cfg, dist, rank, world, dev, kv=args.kv, fused=args.e2e_fused, ragged=args.e2e_ragged, deferred=args.e2e_deferred,
                       eager=args.e2e_eager, ctx0=args.e2e_context, native_layers=not args.e2e_torch_layers,
@@ -1207,6 +1320,9 @@ def main(argv=None):
         per = -(-l_ // cfg.block_size)
         cfg = dataclasses.replace(cfg, name=f"{cfg.name}_b{b_}_l{l_}", batch=b_, seq_len=l_,
                                   num_blocks=max(2 * b_ * per, 64))
+    if args.design:
+        run_design(args, dev)
+        return
     if args.serve:
         run_serve(args, dev, rank)
         if dist is not None:

@@ -36,7 +36,7 @@ def test_library_builds_loads_and_exports_every_declared_symbol():
     assert os.path.exists(path)
     lib = ctypes.CDLL(path)
     assert sorted(os.path.basename(h) for h in glob.glob(os.path.join(REPO, "include", "*.h"))) == \
-        ["vmi_gpt2_layer.h", "vmi_paged_attention.h", "vmi_paged_attention_diag.h", "vmi_paged_attention_extras.h"]
+        ["vmi_gpt2_layer.h", "vmi_hybrid.h", "vmi_paged_attention.h", "vmi_paged_attention_diag.h", "vmi_paged_attention_extras.h"]
     declared = _declared_symbols()
     assert {"vmi_paged_attention_v1_f16", "vmi_reshape_and_cache_f16", "vmi_last_error_string",
             "vmi_abi_version"} <= set(declared)

@@ -26,6 +26,10 @@ at once, step() admits queued requests while a batch slot and blocks are free â€
 the sampled ids come back through a pinned buffer requested BEFORE the decode launches are queued, so the bookkeeping of
 step k+1 runs while the GPU executes step k.
 
+prefill_chunk=n (decoders with step(), vllmini_amd/hybrid_decoder.py): admitted prompts run in portions of at most n tokens per
+step, in the SAME batch as the running sequences' single tokens â€” a long prompt costs the others n tokens of a step at a time
+instead of the whole prompt at once.
+
 Across GPUs (vllmini_amd/shard.py): one scheduler per rank over a private KV pool; requests are dealt to
 ranks by arrival index, and the only per-step exchange is the all_gather of the sampled token ids.
 
@@ -77,8 +81,13 @@ class BatchScheduler:
     def __init__(self, decoder, max_length: int, eos_token_id: int, max_batch: int = 256,
                  sampler: Callable[..., torch.Tensor] = sample_top_k, use_graph: bool = False,
                  generator: Optional[torch.Generator] = None, preempt: str = "swap", record_latency: bool = False,
-                 max_prefill_tokens: int = 8192, admit_every: int = 1, headroom_blocks: Optional[int] = None):
+                 max_prefill_tokens: int = 8192, admit_every: int = 1, headroom_blocks: Optional[int] = None,
+                 prefill_chunk: int = 0):
         self.decoder = decoder
+        if prefill_chunk and not hasattr(decoder, "step"):
+            raise ValueError("prefill_chunk needs a decoder that runs portions of prompts (step())")
+        self.prefill_chunk = int(prefill_chunk)
+        self.prefilling: Dict[int, int] = {}                 # admitted, prompt not finished: seq_id -> tokens run so far
         # a sequence may grow to max_length tokens; the pool's table must hold them (the reference crashes at that
         # point, block_manager.py:41-63 â€” here ONE such sequence would abort the step of every sequence in its batch)
         pool = getattr(decoder, "pool", None)
@@ -176,6 +185,12 @@ class BatchScheduler:
                 self.stop_at.pop(seq_id, None)
                 self._t_submit.pop(seq_id, None)
                 return True
+        if seq_id in self.prefilling:
+            del self.prefilling[seq_id]
+            self.decoder.pool.free(seq_id)
+            self.stop_at.pop(seq_id, None)
+            self._t_submit.pop(seq_id, None)
+            return True
         if seq_id in self.swapped:
             self.decoder.pool.drop_swapped(seq_id)
             del self.swapped[seq_id]
@@ -246,10 +261,10 @@ class BatchScheduler:
         the headroom of everything running (without it the newcomer would be the next victim at the next block boundary)."""
         pool = self.decoder.pool
         for sid in sorted(self.swapped, key=self.swapped.get):
-            if len(self.active) >= self.max_batch:
+            if len(self.active) + len(self.prefilling) >= self.max_batch:
                 break
             need = pool.blocks_of(sid)
-            forced = not self.active          # nothing runs: the oldest swapped sequence must, whatever the headroom
+            forced = not self.active and not self.prefilling          # nothing runs: the oldest swapped sequence must, whatever the headroom
             if len(pool.free_blocks) < need + (0 if forced else self._headroom(1)):
                 break                         # strictly oldest first: a younger, smaller sequence does not overtake
             if not pool.swap_in(sid):
@@ -270,8 +285,11 @@ class BatchScheduler:
         pool = self.decoder.pool
         L, bs = getattr(pool, "num_layers", 1), getattr(pool, "block_size", 16)
         free = len(pool.free_blocks) - self._headroom()
+        for sid, done in self.prefilling.items():            # what admitted prompts have still to take
+            free -= L * (-(-len(self.sequences[sid]) // bs) - (-(-done // bs)) + 1)
+        slots = getattr(pool, "free_state_slots", 0) if getattr(pool, "state_slots", 0) else self.max_batch
         group, tokens = [], 0
-        while self.waiting and len(self.active) + len(group) < self.max_batch:
+        while self.waiting and len(self.active) + len(self.prefilling) + len(group) < self.max_batch and len(group) < slots:
             sid, ids = self.waiting[0]
             need = L * (-(-len(ids) // bs)) + L
             if need > free or (group and tokens + len(ids) > self.max_prefill_tokens):
@@ -281,7 +299,7 @@ class BatchScheduler:
             free -= need
             tokens += len(ids)
         alone = False
-        if not group and not self.active and self.waiting:      # nothing runs and the head of the queue does not "fit": try it alone
+        if not group and not self.active and not self.prefilling and self.waiting:      # nothing runs and the head of the queue does not "fit": try it alone
             group.append(self.waiting.popleft())
             alone = True
         if not group:
@@ -300,6 +318,14 @@ class BatchScheduler:
             self._t_submit.pop(sid, None)
 
     def _prefill_group(self, group) -> None:
+        if self.prefill_chunk:
+            for sid, ids in group:
+                usable = self.decoder.pool.max_blocks_per_seq * self.decoder.pool.block_size
+                if len(ids) > min(usable, self.decoder.pool.num_blocks * self.decoder.pool.block_size):
+                    raise RuntimeError(f"prompt of {len(ids)} tokens: not enough free blocks even in an empty pool")
+                self.decoder.pool.open(sid)
+                self.prefilling[sid] = 0
+            return
         if hasattr(self.decoder, "prefill_batch") and (len(group) > 1 or getattr(self.decoder, "paged_prefill", False)):
             logits = self.decoder.prefill_batch([g[0] for g in group], [g[1] for g in group])
             self.stats["prefill_calls"] += 1
@@ -309,6 +335,51 @@ class BatchScheduler:
             for sid, ids in group:
                 self._started(sid, ids, self.decoder.prefill(sid, ids))
                 self.stats["prefill_calls"] += 1
+
+    # ---- portions of prompts beside single tokens ---------------------------------------------------------------------------
+    def _portions(self) -> List[tuple]:
+        """(seq_id, first token, tokens) of this step, oldest prompt first, prefill_chunk tokens in all."""
+        room, out = self.prefill_chunk, []
+        for sid in sorted(self.prefilling):
+            done = self.prefilling[sid]
+            n = min(room, len(self.sequences[sid]) - done)
+            if n <= 0:
+                break
+            out.append((sid, done, n))
+            room -= n
+        return out
+
+    def _advance(self, batch: List[int], tokens, portions: List[tuple]):
+        """The decoder call of a step: single tokens of `batch`, and the portions; the batch's logits (None without a batch)."""
+        if not portions:
+            return self.decoder.decode(batch, tokens, use_graph=self.use_graph) if self.use_graph else self.decoder.decode(batch, tokens)
+        ends = [d + n == len(self.sequences[s]) for s, d, n in portions]
+        lg = self.decoder.step(batch + [s for s, _, _ in portions],
+                               ([tokens[i:i + 1] for i in range(len(batch))] if batch else [])
+                               + [self.sequences[s][d:d + n] for s, d, n in portions],
+                               [[0]] * len(batch) + [[n - 1] if e else [] for (_, _, n), e in zip(portions, ends)])
+        self.stats["prefill_calls"] += 1
+        row = len(batch)
+        for (s, d, n), e in zip(portions, ends):
+            self.prefilling[s] = d + n
+            if e:
+                del self.prefilling[s]
+                self._started(s, self.sequences[s], lg[row])
+                row += 1
+        return lg[: len(batch)] if batch else None
+
+    def _give_back_prompt(self) -> None:
+        """Out of blocks with no running sequence to preempt: the youngest unfinished prompt returns to the queue â€” unless it is
+        the only one, which then can never fit."""
+        sid = max(self.prefilling)
+        del self.prefilling[sid]
+        self.decoder.pool.free(sid)
+        if self.prefilling:
+            self.waiting.appendleft((sid, self.sequences[sid]))
+        else:
+            self.rejected[sid] = "not enough free blocks even in an empty pool"
+            self.stop_at.pop(sid, None)
+            self._t_submit.pop(sid, None)
 
     # ---- one decode step for every running sequence ------------------------------------------------------
     def _batch_logits(self, batch: List[int]) -> torch.Tensor:
@@ -368,7 +439,16 @@ class BatchScheduler:
             self.stats["admit_s"] += ta
             t0 += ta                                   # (prefill calls are accounted apart from the decode step's host time)
         batch = sorted(self.active, key=self.active.get)[: self.max_batch]      # oldest first (PriorityQueue, :16)
+        portions = self._portions()
         if not batch:
+            if portions:
+                try:
+                    self._advance([], None, portions)
+                    self.steps += 1
+                except RuntimeError as e:
+                    if "free blocks" not in str(e):
+                        raise
+                    self._give_back_prompt()
             return []
         for s in self._lb_ids:               # members of the last call that sit this one out keep their logits
             if s not in self.last_logits and s in self._lb_pos and s in self.active and s not in batch:
@@ -379,12 +459,14 @@ class BatchScheduler:
         keep = None
         while True:
             try:
-                new_logits = self.decoder.decode(batch, tokens, use_graph=self.use_graph) \
-                    if self.use_graph else self.decoder.decode(batch, tokens)
+                new_logits = self._advance(batch, tokens, portions)
                 break
             except RuntimeError as e:                                           # :110-115
                 if "free blocks" not in str(e):
                     raise
+                if portions and len(portions) + len(batch) > 1:      # unfinished prompts wait before a running sequence is preempted
+                    portions = []
+                    continue
                 # the reference picks the youngest sequence other than the one being processed; with a
                 # batch in flight, prefer a victim outside the batch, else the youngest member
                 outside = [s for s in self.active if s not in batch]
@@ -438,7 +520,7 @@ class BatchScheduler:
         return batch
 
     def pending(self) -> bool:
-        return bool(self.active or self.swapped or self.waiting)
+        return bool(self.active or self.swapped or self.waiting or self.prefilling)
 
     def run(self, max_steps: Optional[int] = None) -> int:
         """Step until no sequence is running, swapped out or queued (scheduler.py:55-115); returns the number of steps."""
