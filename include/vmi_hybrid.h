@@ -72,6 +72,10 @@ VMI_HY_API int vmi_hy_add_norm(float* x, const void* add, int64_t ld_add, const 
 VMI_HY_API int vmi_hy_glu(const void* in, int64_t ld_in, void* out, int64_t ld_out, int32_t T, int32_t n, float limit, int32_t dtype,
                           int32_t device, void* stream);
 
+/* out [T, 2 n] = (x | x2) in the element type, x and x2 float32 [T, n] */
+VMI_HY_API int vmi_hy_concat(const float* x, const float* x2, void* out, int32_t T, int32_t n, int32_t dtype, int32_t device,
+                             void* stream);
+
 /* index of the largest of each row's first V values (first maximum on ties) */
 VMI_HY_API int vmi_hy_argmax(const float* logits, int64_t ld, int32_t rows, int32_t V, int64_t* out, int32_t device, void* stream);
 

@@ -125,7 +125,7 @@ def test_builder_refuses_missing_and_misshapen_tensors():
     with pytest.raises(ValueError, match="head"):
         build_model(cfg, {**w, "head": w["head"][:-1]}, torch.float32, "cpu")
     m = build_model(cfg, w, torch.float32, "cpu")
-    assert len(m.runs) == 3 and m.head.N % 32 == 0
+    assert len(m.runs) == 3 and m.head.w.N % 32 == 0
 
 
 def test_padded_layouts_keep_the_products():

@@ -73,19 +73,20 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
   const T* cache = static_cast<const T*>(p.cache);
   const int* tab = s.table + (int64_t)e * s.table_ld;
   const int kj = tid / TPK, kcol = (tid % TPK) * 8;   // this thread's key of a tile, first column
-  auto page_of = [&](int kt) -> int64_t {              // cache row of the thread's key, -1 past the end
-    const int pos = kt * KT + kj;
-    return pos < kv_end ? (int64_t)tab[pos / s.page_size] * s.page_size + pos % s.page_size : -1;
+  auto page_of = [&](int kt) -> int64_t {   // cache row of the thread's key; past the end the last one (it is masked)
+    const int pos = min(kt * KT + kj, kv_end - 1);
+    return (int64_t)tab[pos / s.page_size] * s.page_size + pos % s.page_size;
   };
   V8<T> kr[U];
-  auto load_tile = [&](int64_t row) {
-    const T* src = cache + row * D + kcol;
+  const int nu = (D + TPK * 8 - 1) / (TPK * 8);
+  auto load_tile = [&](int64_t row) {   // (no lane-wise condition around a load: all of them are in flight together)
+    const T* src = cache + row * D;
 #pragma unroll
     for (int i = 0; i < U; ++i)
-      kr[i] = row >= 0 && kcol + i * TPK * 8 < D ? load8(src + i * TPK * 8) : zero8<T>();
+      if (i < nu) kr[i] = load8(src + min(kcol + i * TPK * 8, D - 8));
   };
   load_tile(page_of(kt0));
-  int64_t next_row = kt0 + 1 < kt1 ? page_of(kt0 + 1) : -1;
+  int64_t next_row = page_of(min(kt0 + 1, kt1 - 1));
 
   for (int u = tid; u < R * (D >> 3); u += 256) {   // the query rows
     const int m = u / (D >> 3), k = (u - m * (D >> 3)) * 8;
@@ -110,11 +111,11 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
 
   for (int kt = kt0; kt < kt1; ++kt) {
 #pragma unroll
-    for (int i = 0; i < U; ++i)
-      if (kcol + i * TPK * 8 < D) *reinterpret_cast<V8<T>*>(ks + kj * LDK + kcol + i * TPK * 8) = kr[i];
+    for (int i = 0; i < U; ++i)   // (a clamped column is written twice with the same values)
+      if (i < nu) *reinterpret_cast<V8<T>*>(ks + kj * LDK + min(kcol + i * TPK * 8, D - 8)) = kr[i];
     if (kt + 1 < kt1) {
       load_tile(next_row);
-      next_row = kt + 2 < kt1 ? page_of(kt + 2) : -1;
+      next_row = page_of(min(kt + 2, kt1 - 1));
     }
     __syncthreads();
     f32x4 sc[RT];
@@ -242,22 +243,37 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const vmi_hy_latent
   const int64_t row = blockIdx.x, n = (int64_t)s.T * p.heads;
   if (s.tok_seq[row / p.heads] < 0) return;
   const int ld = p.rank + 2;
-  float m = -1e30f;
-  for (int i = 0; i < p.splits; ++i) m = fmaxf(m, p.partial[(i * n + row) * ld + p.rank]);
-  float l = 0.f;
-  for (int i = 0; i < p.splits; ++i) {
-    const float* q = p.partial + (i * n + row) * ld + p.rank;
-    l += exp2_hw(q[0] - m) * q[1];
+  __shared__ float wt[128];   // weight of every part (at most 128 of them)
+  const float* first = p.partial + row * ld;
+  if (threadIdx.x < 64) {
+    float m[2], l[2], top = -1e30f, sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int i = threadIdx.x + 64 * j;
+      m[j] = i < p.splits ? first[i * n * ld + p.rank] : -1e30f;
+      l[j] = i < p.splits ? first[i * n * ld + p.rank + 1] : 0.f;
+      top = fmaxf(top, m[j]);
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) top = fmaxf(top, __shfl_xor(top, o, 64));
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      m[j] = l[j] > 0.f ? exp2_hw(m[j] - top) : 0.f;   // (a part without keys holds no values)
+      sum += m[j] * l[j];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < 2; ++j) wt[threadIdx.x + 64 * j] = m[j] / sum;
   }
-  const float inv = 1.f / l;
+  __syncthreads();
   for (int k = threadIdx.x; k < p.rank; k += blockDim.x) {
     float a = 0.f;
-#pragma unroll 4
+#pragma unroll 8
     for (int i = 0; i < p.splits; ++i) {
-      const float* q = p.partial + (i * n + row) * ld;
-      if (q[p.rank + 1] > 0.f) a = fmaf(exp2_hw(q[p.rank] - m), q[k], a);   // (a part without keys holds no values)
+      const float w = wt[i];
+      if (w != 0.f) a = fmaf(w, first[i * n * ld + k], a);
     }
-    static_cast<T*>(p.out)[row * p.rank + k] = (T)(a * inv);
+    static_cast<T*>(p.out)[row * p.rank + k] = (T)a;
   }
 }
 
@@ -267,19 +283,22 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_pr
   extern __shared__ float cs[];   // [rot_n / 2][2]
   __shared__ float part[4];
   const int t = blockIdx.x, tid = threadIdx.x, half = p.rot_n >> 1, hd = p.dim + p.rot, D = p.rank + p.rot;
-  if (s.tok_seq[t] < 0) return;
+  const int seq = s.tok_seq[t];
+  const int64_t slot = s.tok_slot[t];
   const double pos = (double)s.tok_pos[t];
+  const T* row = static_cast<const T*>(p.proj) + (int64_t)t * p.ldp;
+  const T* lat = row + p.heads * hd;
+  f32x8 v0 = to_f32<T>(load8(lat + min(tid * 8, p.rank - 8))), w0 = load8(p.norm_w + min(tid * 8, p.rank - 8));
+  if (seq < 0) return;
   for (int i = tid; i < half; i += 256) {   // the angle reduced in fp64: exact to fp32 at any position
     const double a = pos * p.freq[i];
     const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
     cs[2 * i] = cosf(r);
     cs[2 * i + 1] = sinf(r);
   }
-  const T* row = static_cast<const T*>(p.proj) + (int64_t)t * p.ldp;
-  const T* lat = row + p.heads * hd;
   float ss = 0.f;
   for (int k = tid * 8; k < p.rank; k += 2048) {
-    const f32x8 v = to_f32<T>(load8(lat + k));
+    const f32x8 v = k < 2048 ? v0 : to_f32<T>(load8(lat + k));
 #pragma unroll
     for (int e = 0; e < 8; ++e) ss = fmaf(v[e], v[e], ss);
   }
@@ -287,12 +306,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_pr
   if ((tid & 63) == 0) part[tid >> 6] = ss;
   __syncthreads();
   const float rms = 1.f / sqrtf((part[0] + part[1] + part[2] + part[3]) / (float)p.rank_n + p.eps);
-  const int64_t slot = s.tok_slot[t];
   T* crow = slot >= 0 ? static_cast<T*>(p.cache) + slot * D : nullptr;
   if (crow) {
     for (int k = tid * 8; k < p.rank; k += 2048) {
-      f32x8 v = to_f32<T>(load8(lat + k));
-      const f32x8 w = load8(p.norm_w + k);
+      f32x8 v = k < 2048 ? v0 : to_f32<T>(load8(lat + k));
+      const f32x8 w = k < 2048 ? w0 : load8(p.norm_w + k);
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] = v[e] * rms * w[e];
       *reinterpret_cast<V8<T>*>(crow + k) = from_f32<T>(v);
@@ -391,7 +409,7 @@ int vmi_hy_latent_attention(const vmi_hy_latent_attention_args* a, const vmi_hy_
   static const char* who = "vmi_hy_latent_attention";
   if (!a || !s || !a->q || !a->cache || !a->out || !a->tiles || !s->tok_seq || !s->q_start || !s->q_len || !s->ctx || !s->table ||
       s->T <= 0 || s->table_ld <= 0 || s->page_size <= 0 || a->heads <= 0 || a->rank <= 0 || a->rot <= 0 || a->n_tiles <= 0 ||
-      a->splits <= 0 || a->splits > 65535 || (a->splits > 1 && !a->partial))
+      a->splits <= 0 || a->splits > 128 || (a->splits > 1 && !a->partial))
     return fail(VMI_HY_E_ARG, who, "null pointer or a size out of range");
   if ((a->rank & 31) || (a->rot & 31)) return fail(VMI_HY_E_SHAPE, who, "needs sizes that are multiples of 32");
   DeviceScope dev(a->device);

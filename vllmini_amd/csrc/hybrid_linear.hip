@@ -1,7 +1,7 @@
 // The linear layers and the elementwise ends of a step (include/vmi_hybrid.h).
 //
 // y = epilogue(prologue(x) . W^T), written for steps of few rows, where the weights are what has to be read: every wave owns 16
-// output columns and streams its weight tiles (one contiguous KiB per k-step of 32) straight into registers one chunk ahead; the
+// output columns and streams its weight tiles (one contiguous KiB per k-step of 32) straight into registers one or two chunks ahead; the
 // BM rows of x go through LDS in chunks of K, double-buffered, normalised / concatenated / rounded to the element type on their
 // way in, so no normalised copy of the residual stream is ever written.  KS > 1: the k-steps of a chunk are dealt over KS waves
 // whose partial tiles meet in LDS in a fixed order.  D[row = column n][col = row m]: a lane ends with 4 consecutive columns of
@@ -24,10 +24,12 @@ int launched(const char* who) {
   return e == hipSuccess ? VMI_HY_OK : fail(VMI_HY_E_HIP, who, hipGetErrorString(e));
 }
 
-template <int BM, int KS>
+template <typename T, int BM, int KS>
 struct Chunk {
-  static constexpr int CS = BM == 16 ? (KS == 1 ? 8 : 4) : 4;   // k-steps a wave takes from a chunk
-  static constexpr int KC = 32 * CS * KS;                        // columns of x in a chunk
+  static constexpr bool DEEP = BM == 16 && sizeof(T) == 2;   // few rows: bytes in flight are what counts
+  static constexpr int CS = DEEP ? 8 : 4;                     // k-steps a wave takes from a chunk
+  static constexpr int NB = DEEP ? 3 : 2;                     // chunks of weights in registers, NB - 1 of them ahead
+  static constexpr int KC = 32 * CS * KS;                     // columns of x in a chunk
 };
 
 // 8 consecutive elements of row m at column k, as they go into LDS
@@ -68,7 +70,8 @@ struct XUnit<T, VMI_HY_X_CONCAT> {
 
 template <typename T, int BM, int NW, int KS, int XK, int EPI>
 __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear_args p) {
-  constexpr int TH = NW * KS * 64, MT = BM / 16, CS = Chunk<BM, KS>::CS, KC = Chunk<BM, KS>::KC;
+  using CK = Chunk<T, BM, KS>;
+  constexpr int TH = NW * KS * 64, MT = BM / 16, CS = CK::CS, KC = CK::KC, NB_W = CK::NB;
   constexpr int LD = KC + 16 / (int)sizeof(T), UPR = KC / 8, UPT = BM * UPR / TH;
   static_assert(BM * UPR % TH == 0, "a chunk's units divide over the threads");
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -88,7 +91,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
 
   const T* wp = static_cast<const T*>(p.w) + (((int64_t)grp * (p.N >> 4) + (nvalid ? n0 >> 4 : 0)) * nks * 64 + lane) * 8;
   const int nchunk = (p.K + KC - 1) / KC;
-  V8<T> wb[2][CS];
+  V8<T> wb[NB_W][CS];
   auto load_w = [&](V8<T>(&dst)[CS], int c) {
 #pragma unroll
     for (int j = 0; j < CS; ++j) {
@@ -96,9 +99,10 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       dst[j] = k < nks && nvalid ? load8(wp + (int64_t)k * 512) : zero8<T>();
     }
   };
-  load_w(wb[0], 0);
+#pragma unroll
+  for (int b = 0; b < NB_W - 1; ++b) load_w(wb[b], b);
 
-  auto source_row = [&](int m) -> int64_t {   // rows past M read row M - 1 and are never stored
+  auto source_row = [&](int m) -> int64_t {
     const int mm = m0 + m < p.M ? m0 + m : p.M - 1;
     if constexpr (XK == VMI_HY_X_NORM) return p.rows ? p.rows[mm] : mm;
     return mm;
@@ -106,12 +110,13 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
 
   if constexpr (XK == VMI_HY_X_NORM) {   // row statistics, one pass around the row's first element: no cancellation to speak of
     constexpr int NWV = TH / 64;
-    for (int mbase = wave; mbase < BM; mbase += 4 * NWV) {
+    const int mrows = min(BM, p.M - m0);
+    for (int mbase = wave; mbase < mrows; mbase += 4 * NWV) {
       const float* row[4];
       float sh[4], s[4], q[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int m = mbase + i * NWV < BM ? mbase + i * NWV : mbase;
+        const int m = mbase + i * NWV < mrows ? mbase + i * NWV : mbase;
         row[i] = static_cast<const float*>(p.x) + source_row(m) * p.ldx;
         sh[i] = row[i][0];
         s[i] = q[i] = 0.f;
@@ -132,7 +137,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       for (int i = 0; i < 4; ++i) {
         const float ms = wave_sum(s[i]) / (float)p.norm_n, mq = wave_sum(q[i]) / (float)p.norm_n;
         const int m = mbase + i * NWV;
-        if (lane == 0 && m < BM) {
+        if (lane == 0 && m < mrows) {
           stats[2 * m] = sh[i] + ms;
           stats[2 * m + 1] = 1.f / sqrtf(fmaxf(mq - ms * ms, 0.f) + p.eps);
         }
@@ -143,6 +148,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
 
   int64_t srow[UPT];
   int xm[UPT], xk[UPT];
+  bool xin[UPT];
   float mean[UPT], rstd[UPT];
 #pragma unroll
   for (int i = 0; i < UPT; ++i) {
@@ -150,8 +156,12 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
     xm[i] = u / UPR;
     xk[i] = (u % UPR) * 8;
     srow[i] = source_row(xm[i]);
+    xin[i] = m0 + xm[i] < p.M;
     mean[i] = rstd[i] = 0.f;
-    if constexpr (XK == VMI_HY_X_NORM) {
+    if (!xin[i]) {   // rows past M: zeros in both buffers, once
+      *reinterpret_cast<V8<T>*>(xs + xm[i] * LD + xk[i]) = zero8<T>();
+      *reinterpret_cast<V8<T>*>(xs + (BM + xm[i]) * LD + xk[i]) = zero8<T>();
+    } else if constexpr (XK == VMI_HY_X_NORM) {
       mean[i] = stats[2 * xm[i]];
       rstd[i] = stats[2 * xm[i] + 1];
     }
@@ -160,7 +170,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   auto load_x = [&](int c) {
 #pragma unroll
     for (int i = 0; i < UPT; ++i)
-      if (c * KC + xk[i] < p.K) xu[i].load(p, srow[i], goff, c * KC + xk[i]);
+      if (xin[i] && c * KC + xk[i] < p.K) xu[i].load(p, srow[i], goff, c * KC + xk[i]);
   };
   load_x(0);
 
@@ -171,12 +181,10 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
     T* dst = xs + (size_t)(c & 1) * BM * LD;
 #pragma unroll
     for (int i = 0; i < UPT; ++i)
-      if (c * KC + xk[i] < p.K)
+      if (xin[i] && c * KC + xk[i] < p.K)
         *reinterpret_cast<V8<T>*>(dst + xm[i] * LD + xk[i]) = xu[i].finish(p, c * KC + xk[i], mean[i], rstd[i]);
-    if (c + 1 < nchunk) {
-      load_w(nxt, c + 1);
-      load_x(c + 1);
-    }
+    if (c + 1 < nchunk) load_x(c + 1);
+    if (c + NB_W - 1 < nchunk) load_w(nxt, c + NB_W - 1);
     __syncthreads();   // (two buffers: the writes of chunk c + 1 go where chunk c - 1 was read, which every wave has left behind)
     const int kn = min(nks - c * (CS * KS), CS * KS) - ks * CS;   // k-steps of this chunk that are this wave's
 #pragma unroll
@@ -188,9 +196,10 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       }
     }
   };
-  for (int c = 0; c < nchunk; c += 2) {
-    step(c, wb[0], wb[1]);
-    if (c + 1 < nchunk) step(c + 1, wb[1], wb[0]);
+  for (int c = 0; c < nchunk; c += NB_W) {   // chunk c sits in wb[c % NB_W]; the one behind it has been used up
+#pragma unroll
+    for (int b = 0; b < NB_W; ++b)
+      if (c + b < nchunk) step(c + b, wb[b], wb[(b + NB_W - 1) % NB_W]);
   }
 
   if constexpr (KS > 1) {
@@ -251,7 +260,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
 
 template <typename T, int BM, int NW, int KS, int XK, int EPI>
 static int launch_linear(const vmi_hy_linear_args& p, hipStream_t st) {
-  constexpr int KC = Chunk<BM, KS>::KC, LD = KC + 16 / (int)sizeof(T);
+  constexpr int KC = Chunk<T, BM, KS>::KC, LD = KC + 16 / (int)sizeof(T);
   const size_t lds = (size_t)2 * BM * LD * sizeof(T) + 2 * BM * 4 + (size_t)(KS - 1) * NW * (BM / 16) * 64 * 16;
   auto* fn = linear_kernel<T, BM, NW, KS, XK, EPI>;
   if (int rc = allow_lds(fn, lds, "vmi_hy_linear")) return rc;
@@ -268,7 +277,8 @@ static int linear_shape(const vmi_hy_linear_args& p, hipStream_t st) {
     const int64_t wgs = slabs * ((p.M + 15) / 16);
     if (wgs >= 2048) return launch_linear<T, 16, 4, 1, XK, EPI>(p, st);
     if (wgs >= 512 || p.K < 256) return launch_linear<T, 16, 2, 2, XK, EPI>(p, st);
-    return launch_linear<T, 16, 1, 4, XK, EPI>(p, st);
+    if (wgs >= 192 || p.K < 1024) return launch_linear<T, 16, 1, 4, XK, EPI>(p, st);
+    return launch_linear<T, 16, 1, 8, XK, EPI>(p, st);
   }
   if (p.M <= 96 || slabs / 4 * ((p.M + 63) / 64) < 256) return launch_linear<T, 32, 4, 1, XK, EPI>(p, st);
   return launch_linear<T, 64, 4, 1, XK, EPI>(p, st);
@@ -366,6 +376,14 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* x, const T* add, i
     if (k < ld) put(v[i], k);
   }
   for (int k = (tid + MAXV * 256) * 4; k < ld; k += 1024) put(*reinterpret_cast<const f32x4*>(row + k), k);
+}
+
+// out [T, 2 n] = (x | x2) in the element type
+template <typename T>
+__global__ __launch_bounds__(256) void concat_kernel(const float* __restrict__ x, const float* __restrict__ x2, T* __restrict__ out, int n) {
+  const int t = blockIdx.y, j = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (j >= 2 * n) return;
+  *reinterpret_cast<V8<T>*>(out + (int64_t)t * 2 * n + j) = from_f32<T>(load8((j < n ? x + j : x2 + j - n) + (int64_t)t * n));
 }
 
 template <typename T>
@@ -471,6 +489,20 @@ int vmi_hy_glu(const void* in, int64_t ld_in, void* out, int64_t ld_out, int32_t
     hipLaunchKernelGGL(glu_kernel<b16>, grid, dim3(256), 0, st, static_cast<const b16*>(in), ld_in, static_cast<b16*>(out), ld_out, n, limit);
   else
     hipLaunchKernelGGL(glu_kernel<float>, grid, dim3(256), 0, st, static_cast<const float*>(in), ld_in, static_cast<float*>(out), ld_out, n, limit);
+  return launched(who);
+}
+
+int vmi_hy_concat(const float* x, const float* x2, void* out, int32_t T, int32_t n, int32_t dtype, int32_t device, void* stream) {
+  static const char* who = "vmi_hy_concat";
+  if (!x || !x2 || !out || T <= 0 || T > 65535 || n <= 0 || (n & 7)) return fail(VMI_HY_E_ARG, who, "bad argument");
+  DeviceScope dev(device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  const dim3 grid((2 * n / 8 + 255) / 256, T);
+  if (dtype == VMI_HY_BF16)
+    hipLaunchKernelGGL(concat_kernel<b16>, grid, dim3(256), 0, st, x, x2, static_cast<b16*>(out), n);
+  else
+    hipLaunchKernelGGL(concat_kernel<float>, grid, dim3(256), 0, st, x, x2, static_cast<float*>(out), n);
   return launched(who);
 }
 

@@ -31,28 +31,35 @@ struct Lds {
   T u[BM * LDU];
   float a[BM * LDA];
   float b[BM * LDA];
+  float end[2][4][CT];
   RowMeta meta[BM];
 };
 
-// convolution of 8 channels for the token of row m
-template <typename T>
+// convolution of 8 channels for the token of row m.  TAPS = 0: any number of taps; else exactly that many, every load issued
+// without a condition around it (taps before the start read a valid row and count zero), so that all of them are in flight
+template <typename T, int TAPS>
 __device__ __forceinline__ f32x8 conv8(const vmi_hy_rglru_args& p, const RowMeta& r, int t, int c) {
   f32x8 acc = load8(p.conv_b + c);
   const T* in = static_cast<const T*>(p.yx) + p.width + c;
-  const int pos = r.ctx + t - r.qs;
-  for (int j = 0; j < p.taps; ++j) {
-    const int back = p.taps - 1 - j;
-    if (pos < back) continue;               // zeros before the start
-    V8<T> v;
-    if (t - back >= r.qs) {
-      v = load8(in + (int64_t)(t - back) * p.ldx);
-    } else {
-      const int e = pos - back - (r.ctx - (p.taps - 1));   // tail entries: positions ctx - (taps - 1) .. ctx - 1
-      v = load8(static_cast<const T*>(p.tail) + (((int64_t)r.slot * 2 + r.flip) * (p.taps - 1) + e) * p.width + c);
-    }
+  const int taps = TAPS ? TAPS : p.taps, pos = r.ctx + t - r.qs;
+  // tail entries: positions ctx - (taps - 1) .. ctx - 1
+  const T* tail = static_cast<const T*>(p.tail) + ((int64_t)r.slot * 2 + r.flip) * (taps - 1) * p.width + c;
+  auto tap = [&](int j) {
+    const int back = taps - 1 - j;
+    const T* src = t - back >= r.qs ? in + (int64_t)(t - back) * p.ldx
+                   : pos >= back    ? tail + (int64_t)(pos - back - (r.ctx - (taps - 1))) * p.width
+                                    : in + (int64_t)t * p.ldx;
+    const V8<T> v = load8(src);
     const f32x8 w = load8(p.conv_w + (int64_t)j * p.width + c);
+    const bool on = pos >= back;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[e], (float)v[e], acc[e]);
+    for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[e], on ? (float)v[e] : 0.f, acc[e]);
+  };
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) tap(j);
+  } else {
+    for (int j = 0; j < taps; ++j) tap(j);
   }
   return acc;
 }
@@ -66,7 +73,7 @@ __device__ __forceinline__ void store_out8(const vmi_hy_rglru_args& p, int t, in
   *reinterpret_cast<V8<T>*>(static_cast<T*>(p.out) + (int64_t)t * p.ldo + c) = from_f32<T>(o);
 }
 
-template <typename T, int BM>
+template <typename T, int BM, int TAPS>
 __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args p, const vmi_hy_step s) {
   constexpr int MT = BM / 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -102,16 +109,14 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
   const T* wr = static_cast<const T*>(p.gates) + blk * gsz + ((int64_t)((cin >> 4) + wave) * nks * 64 + lane) * 8;
   const T* wi = wr + p.blocks * gsz;
   for (int k0 = 0; k0 < bw; k0 += KCH) {
-    const int kn = min(KCH, bw - k0), upr = kn >> 3;
+    const int kn = min(KCH, bw - k0);
     __syncthreads();   // meta is there; the previous chunk has been read
-    for (int u = tid; u < BM * upr; u += 256) {
-      const int m = u / upr, k = (u - m * upr) * 8;
+#pragma unroll 2
+    for (int u = tid; u < BM * (KCH / 8); u += 256) {   // (a row of LDS is KCH channels, the last chunk may have fewer)
+      const int m = u / (KCH / 8), k = (u % (KCH / 8)) * 8;
       const RowMeta& r = L.meta[m];
-      f32x8 v;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] = 0.f;
-      if (r.seq >= 0) v = conv8<T>(p, r, t0 + m, blk * bw + k0 + k);
-      *reinterpret_cast<V8<T>*>(L.u + m * LDU + k) = from_f32<T>(v);
+      if (r.seq >= 0 && k < kn) *reinterpret_cast<V8<T>*>(L.u + m * LDU + k) = from_f32<T>(conv8<T, TAPS>(p, r, t0 + m, blk * bw + k0 + k));
+      else if (k < kn) *reinterpret_cast<V8<T>*>(L.u + m * LDU + k) = zero8<T>();
     }
     __syncthreads();
     if (wvalid) {
@@ -127,14 +132,17 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
       }
     }
   }
-  // the workgroup's own channels of u, again (they may have left LDS): into b
+  // the workgroup's own channels of u: into b, from LDS or (a block of several chunks) computed again
+  const bool held = bw <= KCH;
+  if (held) __syncthreads();
   for (int u = tid; u < BM * (CT / 8); u += 256) {
     const int m = u / (CT / 8), k = (u % (CT / 8)) * 8;
     const RowMeta& r = L.meta[m];
     f32x8 v;
 #pragma unroll
     for (int e = 0; e < 8; ++e) v[e] = 0.f;
-    if (r.seq >= 0 && k < nch) v = to_f32<T>(from_f32<T>(conv8<T>(p, r, t0 + m, c0 + k)));   // rounded as the gates saw it
+    if (held && k < nch) v = to_f32<T>(load8(L.u + m * LDU + cin + k));
+    else if (r.seq >= 0 && k < nch) v = to_f32<T>(from_f32<T>(conv8<T, TAPS>(p, r, t0 + m, c0 + k)));   // rounded as the gates saw it
     *reinterpret_cast<f32x8*>(L.b + m * LDA + k) = v;
   }
   __syncthreads();
@@ -167,17 +175,35 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
   }
   __syncthreads();
   const bool lead0 = L.meta[0].seq >= 0 && !L.meta[0].first;   // the tile opens inside a portion
-  if (!p.single && tid < nch) {   // the walk: one thread per channel, in place (b becomes S, a becomes P)
-    float S = 0.f, P = lead0 ? 1.f : 0.f;
-    float* pa = L.a + tid;
-    float* pb = L.b + tid;
+  if (!p.single) {   // the walk, in place (b becomes S, a becomes P): a wave takes a quarter of the rows, a lane a channel
+    constexpr int RW = BM / 4;
+    float* pa = L.a + wave * RW * LDA + lane;
+    float* pb = L.b + wave * RW * LDA + lane;
+    if (lane < nch) {
+      float S = 0.f, P = wave == 0 ? (lead0 ? 1.f : 0.f) : 1.f;
 #pragma unroll 8
-    for (int m = 0; m < BM; ++m) {
-      const float a = pa[m * LDA], b = pb[m * LDA];
-      S = fmaf(a, S, b);
-      P *= a;
-      pb[m * LDA] = S;
-      pa[m * LDA] = P;
+      for (int m = 0; m < RW; ++m) {
+        const float a = pa[m * LDA], b = pb[m * LDA];
+        S = fmaf(a, S, b);
+        P *= a;
+        pb[m * LDA] = S;
+        pa[m * LDA] = P;
+      }
+      L.end[0][wave][lane] = S;
+      L.end[1][wave][lane] = P;
+    }
+    __syncthreads();
+    if (lane < nch && wave > 0) {   // what the quarters before this one hand over
+      float S = L.end[0][0][lane], P = L.end[1][0][lane];
+      for (int w = 1; w < wave; ++w) {
+        S = fmaf(L.end[1][w][lane], S, L.end[0][w][lane]);
+        P *= L.end[1][w][lane];
+      }
+#pragma unroll 8
+      for (int m = 0; m < RW; ++m) {
+        pb[m * LDA] = fmaf(pa[m * LDA], S, pb[m * LDA]);
+        pa[m * LDA] *= P;
+      }
     }
   }
   __syncthreads();
@@ -202,23 +228,18 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
     if (r.last) *reinterpret_cast<f32x8*>(p.state + (int64_t)r.slot * p.width + c) = S;
   }
   // the convolution tail of entries that end in this tile, into its other half
-  if (p.taps > 1) {
-    for (int m = 0; m < rows; ++m) {
-      const RowMeta& r = L.meta[m];
-      if (r.seq < 0 || !r.last) continue;   // uniform
-      const int nt = p.taps - 1;
-      const T* from = static_cast<const T*>(p.tail) + ((int64_t)r.slot * 2 + r.flip) * nt * p.width;
-      T* to = static_cast<T*>(p.tail) + ((int64_t)r.slot * 2 + (r.flip ^ 1)) * nt * p.width;
-      for (int u = tid; u < nt * (CT / 8); u += 256) {
-        const int e = u / (CT / 8), k = (u % (CT / 8)) * 8, c = c0 + k;
-        if (k >= nch) continue;
-        const int pos = r.ctx + r.len - nt + e;   // the position this entry stands for
-        V8<T> v = zero8<T>();
-        if (pos >= r.ctx) v = load8(static_cast<const T*>(p.yx) + (int64_t)(r.qs + pos - r.ctx) * p.ldx + p.width + c);
-        else if (pos >= 0) v = load8(from + (int64_t)(pos - (r.ctx - nt)) * p.width + c);
-        *reinterpret_cast<V8<T>*>(to + (int64_t)e * p.width + c) = v;
-      }
-    }
+  const int nt = p.taps - 1;
+  for (int u = tid; u < rows * nt * (CT / 8); u += 256) {
+    const int k = (u % (CT / 8)) * 8, e = u / (CT / 8) % nt, m = u / (CT / 8) / nt, c = c0 + k;
+    const RowMeta& r = L.meta[m];
+    if (k >= nch || r.seq < 0 || !r.last) continue;
+    const T* from = static_cast<const T*>(p.tail) + ((int64_t)r.slot * 2 + r.flip) * nt * p.width;
+    T* to = static_cast<T*>(p.tail) + ((int64_t)r.slot * 2 + (r.flip ^ 1)) * nt * p.width;
+    const int pos = r.ctx + r.len - nt + e;   // the position this entry stands for
+    V8<T> v = zero8<T>();
+    if (pos >= r.ctx) v = load8(static_cast<const T*>(p.yx) + (int64_t)(r.qs + pos - r.ctx) * p.ldx + p.width + c);
+    else if (pos >= 0) v = load8(from + (int64_t)(pos - (r.ctx - nt)) * p.width + c);
+    *reinterpret_cast<V8<T>*>(to + (int64_t)e * p.width + c) = v;
   }
 }
 
@@ -270,9 +291,9 @@ __global__ __launch_bounds__(256) void rglru_finish_kernel(const vmi_hy_rglru_ar
   store_out8<T>(p, t, c, o);
 }
 
-template <typename T, int BM>
+template <typename T, int BM, int TAPS>
 static int launch_tile(const vmi_hy_rglru_args& p, const vmi_hy_step& s, hipStream_t st) {
-  auto* fn = rglru_tile_kernel<T, BM>;
+  auto* fn = rglru_tile_kernel<T, BM, TAPS>;
   if (int rc = allow_lds(fn, sizeof(Lds<T, BM>), "vmi_hy_rglru")) return rc;
   const int bw = p.width / p.blocks;
   hipLaunchKernelGGL(fn, dim3(p.blocks * ((bw + CT - 1) / CT), (s.T + BM - 1) / BM), dim3(256), sizeof(Lds<T, BM>), st, p, s);
@@ -281,8 +302,8 @@ static int launch_tile(const vmi_hy_rglru_args& p, const vmi_hy_step& s, hipStre
 
 template <typename T>
 static int run_rglru(const vmi_hy_rglru_args& p, const vmi_hy_step& s, hipStream_t st) {
-  if (p.single) return launch_tile<T, 16>(p, s, st);
-  if (int rc = launch_tile<T, 64>(p, s, st)) return rc;
+  if (p.single) return p.taps == 4 ? launch_tile<T, 16, 4>(p, s, st) : launch_tile<T, 16, 0>(p, s, st);
+  if (int rc = p.taps == 4 ? launch_tile<T, 64, 4>(p, s, st) : launch_tile<T, 64, 0>(p, s, st)) return rc;
   if (!p.spans) return VMI_HY_OK;
   hipLaunchKernelGGL(rglru_carry_kernel, dim3((p.width + 63) / 64, s.B), dim3(64), 0, st, p, s);
   hipLaunchKernelGGL(rglru_finish_kernel<T>, dim3((p.width / 8 + 255) / 256, s.T), dim3(256), 0, st, p, s);

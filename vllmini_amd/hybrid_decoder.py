@@ -17,7 +17,7 @@ import numpy as np
 import torch
 
 from . import hybrid_ops as ops
-from .hybrid_layers import ClampedGLU, ConcatProjection, LatentAttention, Norm, Residual, RGLRU
+from .hybrid_layers import ClampedGLU, ConcatProjection, Head, LatentAttention, Residual, RGLRU
 from .kv_pool import PagedKVPool
 
 
@@ -38,9 +38,7 @@ class HybridModel:
     embed: torch.Tensor            # bfloat16 [vocab, width padded to 32]
     embed_scale: float
     runs: List[LayerRun]
-    final_norm: Norm
-    head: ops.MatrixTiles
-    logit_scale: float
+    head: Head
     eos_token_id: int = -1         # (a design without one: generation ends at its length)
 
     def make_pool(self, max_tokens: int, max_seqs: int, page_size: int = 64, max_length: Optional[int] = None, **kw) -> PagedKVPool:
@@ -190,7 +188,7 @@ class HybridDecoder:
                 self.tap.append(res.settle()[:, : m.width].clone())
         if rows is None:
             return None
-        return ops.linear(res.settle(), m.head, norm=m.final_norm.args, rows=rows, float_out=(m.vocab_size, m.logit_scale))
+        return m.head.run(res.settle(), rows)
 
     def _ids(self, tokens: Sequence) -> torch.Tensor:
         """The step's token ids on the device; host ids are range-checked here."""

@@ -20,7 +20,12 @@ import torch.nn.functional as F
 from . import hybrid_ops as ops
 from .hybrid_ops import MatrixTiles, StepLayout, pad32
 
-DENSE_MIN_TOKENS = 512
+DENSE_MIN_TOKENS = 48
+
+
+def float_product(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x W^T as float32, whatever the operands' type."""
+    return torch.mm(x, w.t()) if x.dtype == torch.float32 else torch.mm(x, w.t(), out_dtype=torch.float32)
 
 
 class Norm:
@@ -34,6 +39,21 @@ class Norm:
     @property
     def args(self) -> Tuple[torch.Tensor, int, float]:
         return self.weight, self.n, self.eps
+
+
+class Head:
+    """Final norm and vocabulary projection, logits float32 times a scale (folded into the norm's weight on the dense path)."""
+
+    def __init__(self, norm: Norm, weight: torch.Tensor, ld: int, scale: float, dtype: torch.dtype):
+        self.norm, self.vocab, self.scale, self.dtype = norm, weight.shape[0], float(scale), dtype
+        self.w = MatrixTiles(spread(weight, 1, torch.arange(weight.shape[1]), ld), dtype, dense=True)
+        self.scaled = (norm.weight * self.scale, norm.n, norm.eps)
+
+    def run(self, x: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
+        if rows.numel() >= DENSE_MIN_TOKENS:
+            h = ops.add_norm(x.index_select(0, rows), None, self.scaled, self.dtype)
+            return float_product(h, self.w.dense)[:, : self.vocab]
+        return ops.linear(x, self.w, norm=self.norm.args, rows=rows, float_out=(self.vocab, self.scale))
 
 
 class Residual:
@@ -202,8 +222,11 @@ class ConcatProjection:
     def __init__(self, *, width: int, weight: torch.Tensor, dtype: torch.dtype):
         E = pad32(width)
         cols = torch.cat([torch.arange(width), E + torch.arange(width)])
-        self.w = MatrixTiles(spread(spread(weight, 1, cols, 2 * E), 0, torch.arange(width), E), dtype)
+        self.w = MatrixTiles(spread(spread(weight, 1, cols, 2 * E), 0, torch.arange(width), E), dtype, dense=True)
 
     def run(self, res: Residual, x0: torch.Tensor) -> None:
         x = res.settle()
-        res.x = ops.linear(x, self.w, x2=x0, float_out=(x.shape[1], 1.0))      # (the stream stays float32)
+        if x.shape[0] >= DENSE_MIN_TOKENS:
+            res.x = float_product(ops.concat(x, x0, res.dtype), self.w.dense)      # (the stream stays float32)
+        else:
+            res.x = ops.linear(x, self.w, x2=x0, float_out=(x.shape[1], 1.0))

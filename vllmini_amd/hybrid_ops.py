@@ -52,6 +52,7 @@ SIGNATURES = {
     "vmi_hy_embed": (ctypes.c_int, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
     "vmi_hy_add_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32, _vp]),
     "vmi_hy_glu": (ctypes.c_int, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_concat": (ctypes.c_int, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _vp]),
     "vmi_hy_argmax": (ctypes.c_int, [_vp, _i64, _i32, _i32, _vp, _i32, _vp]),
     "vmi_hy_rglru": (ctypes.c_int, [ctypes.POINTER(RglruArgs), ctypes.POINTER(StepArgs), _vp]),
     "vmi_hy_latent_prep": (ctypes.c_int, [ctypes.POINTER(PrepArgs), ctypes.POINTER(StepArgs), _vp]),
@@ -217,6 +218,17 @@ def glu(x: torch.Tensor, limit: float) -> torch.Tensor:
     for t in range(0, T, 65535):      # (a launch's grid holds that many rows)
         m = min(65535, T - t)
         _check(load().vmi_hy_glu(x[t:].data_ptr(), x.stride(0), out[t:].data_ptr(), n, m, n, float(limit), DTYPES[x.dtype], device, stream))
+    return out
+
+
+def concat(x: torch.Tensor, x2: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """(x | x2) of two float32 [T, n] tensors, in `dtype`."""
+    device, stream = _on(x)
+    _need(x.shape == x2.shape and x.is_contiguous() and x2.is_contiguous() and x.dtype == x2.dtype == torch.float32
+          and x2.device == x.device, "hybrid_ops.concat: two contiguous float32 tensors of one shape")
+    T, n = x.shape
+    out = torch.empty((T, 2 * n), dtype=dtype, device=x.device)
+    _check(load().vmi_hy_concat(x.data_ptr(), x2.data_ptr(), out.data_ptr(), T, n, DTYPES[dtype], device, stream))
     return out
 
 

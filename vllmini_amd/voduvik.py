@@ -12,8 +12,8 @@ from typing import Dict, List, Optional, Tuple
 import torch
 
 from .hybrid_decoder import HybridModel, LayerRun
-from .hybrid_layers import ClampedGLU, ConcatProjection, LatentAttention, Norm, RGLRU, spread
-from .hybrid_ops import MatrixTiles, pad32
+from .hybrid_layers import ClampedGLU, ConcatProjection, Head, LatentAttention, Norm, RGLRU, spread
+from .hybrid_ops import pad32
 
 
 @dataclasses.dataclass(frozen=True)
@@ -127,5 +127,4 @@ def build_model(cfg: VoduvikConfig, tensors: Dict[str, torch.Tensor], dtype: tor
     return HybridModel(vocab_size=cfg.vocab, width=E, dtype=dtype, device=device,
                        embed=spread(w["embed"].to(torch.bfloat16), 1, torch.arange(E), ld).contiguous(), embed_scale=cfg.embedding_scale,
                        runs=[LayerRun(mixers[i], mlps[i], enter if first else None) for i, first in cfg.order()],
-                       final_norm=norm("final.norm"),
-                       head=MatrixTiles(spread(w["head"], 1, torch.arange(E), ld), dtype), logit_scale=cfg.logit_scale)
+                       head=Head(norm("final.norm"), w["head"], ld, cfg.logit_scale, dtype))
