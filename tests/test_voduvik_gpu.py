@@ -464,7 +464,13 @@ def test_long_decoding_from_one_token(dtype):
     logits_close(got, want, dtype, tol32=5e-4)
 
 
-def test_graph_replay_equals_eager_steps():
+@pytest.mark.parametrize("vendor", [False, True], ids=["streaming", "vendor"])
+def test_graph_replay_equals_eager_steps(vendor, monkeypatch):
+    """Both ways a layer's products may run, captured; eager steps run between the replays."""
+    from vllmini_amd import hybrid_layers
+
+    if vendor:
+        monkeypatch.setattr(hybrid_layers, "DENSE_MIN_TOKENS", 1)
     name = "mixed"
     c = cases.CONFIGS[name]
     a, b = decoder(name, torch.bfloat16, pad_batch_to=4), decoder(name, torch.bfloat16)

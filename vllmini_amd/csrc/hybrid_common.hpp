@@ -73,9 +73,17 @@ __device__ __forceinline__ V8<T> from_f32(const f32x8& v) {
   return r;
 }
 
-__device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+// exponential, reciprocal and root on the vector unit's own instructions (about 1 ulp each, all of it fp32)
+__device__ __forceinline__ float exp_hw(float z) { return __builtin_amdgcn_exp2f(z * 1.4426950408889634f); }
+__device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.f + exp_hw(-z)); }
+// 0.5 (1 + tanh w) is sigmoid(2 w)
 __device__ __forceinline__ float gelu_tanh(float z) {
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  return z * sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
+}
+// 1 - exp(-x), x >= 0, given e = exp(-x): a series where the difference would cancel
+__device__ __forceinline__ float one_minus_exp(float x, float e) {
+  const float s = x * fmaf(-x, fmaf(-x, fmaf(-x, fmaf(-x, fmaf(-x, 1.f / 720.f, 1.f / 120.f), 1.f / 24.f), 1.f / 6.f), 0.5f), 1.f);
+  return x < 0.25f ? s : 1.f - e;
 }
 // the clamped gated unit: gate g (already a product), up-projection u
 __device__ __forceinline__ float glu(float g, float u, float limit) {

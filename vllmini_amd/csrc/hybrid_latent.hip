@@ -28,6 +28,24 @@ __device__ __forceinline__ f32x8 column8(const float* tile, int ld, int row0, in
   return r;
 }
 
+// maximum / sum over the 16 lanes that share kc, on the cross-lane paths of the vector unit (no LDS round trip)
+template <int CTRL>
+__device__ __forceinline__ float dpp(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float max16(float v) {
+  v = fmaxf(v, dpp<0xB1>(v));    // quad_perm [1,0,3,2]
+  v = fmaxf(v, dpp<0x4E>(v));    // quad_perm [2,3,0,1]
+  v = fmaxf(v, dpp<0x141>(v));   // row_half_mirror
+  return fmaxf(v, dpp<0x140>(v));   // row_mirror
+}
+__device__ __forceinline__ float sum16(float v) {
+  v += dpp<0xB1>(v);
+  v += dpp<0x4E>(v);
+  v += dpp<0x141>(v);
+  return v + dpp<0x140>(v);
+}
+
 __device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
 
 template <typename T>
@@ -41,14 +59,17 @@ inline size_t attention_lds(int D) {
 }
 
 // RT row tiles, NT value tiles (of 16 columns) per wave, U 16-byte-element units of a cache row per thread
-template <typename T, int KT, int RT, int NT, int U>
-__global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_latent_attention_args p, const vmi_hy_step s) {
+// EXACT: a row has exactly that many (its length is known to the compiler: loops over it unroll, and with one row tile the query
+// stays in registers, which leaves LDS for a second workgroup)
+template <typename T, int KT, int RT, int NT, int U, bool EXACT>
+__global__ __launch_bounds__(256, EXACT && RT == 1 ? 2 : 1) void latent_attention_kernel(const vmi_hy_latent_attention_args p, const vmi_hy_step s) {
   constexpr int R = 16 * RT, TPK = 256 / KT, PAD = pad_of<T>(), LDP = KT + PAD, SW = KT / 16;   // SW waves score
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-  const int D = p.rank + p.rot, LDK = D + PAD;
+  constexpr bool QREG = EXACT && RT == 1 && sizeof(T) == 2;
+  const int D = EXACT ? U * TPK * 8 : p.rank + p.rot, LDK = D + PAD;
   T* ks = reinterpret_cast<T*>(smem);              // [KT][LDK]
   T* qs = ks + (size_t)KT * LDK;                   // [R][LDK]
-  T* ps = qs + (size_t)R * LDK;                    // [R][LDP]
+  T* ps = qs + (QREG ? 0 : (size_t)R * LDK);       // [R][LDP]
   float* sx = reinterpret_cast<float*>(ps + (size_t)R * LDP);   // [4][R]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), kc = lane >> 4, r16 = lane & 15;
   const int e = p.tiles[2 * blockIdx.x], r0 = p.tiles[2 * blockIdx.x + 1], split = blockIdx.y;
@@ -73,24 +94,29 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
   const T* cache = static_cast<const T*>(p.cache);
   const int* tab = s.table + (int64_t)e * s.table_ld;
   const int kj = tid / TPK, kcol = (tid % TPK) * 8;   // this thread's key of a tile, first column
-  auto page_of = [&](int kt) -> int64_t {   // cache row of the thread's key; past the end the last one (it is masked)
-    const int pos = min(kt * KT + kj, kv_end - 1);
-    return (int64_t)tab[pos / s.page_size] * s.page_size + pos % s.page_size;
-  };
+  // The page number of a tile is read one tile before the tile itself, and not touched before that tile is requested: loads
+  // complete in order, so an earlier use would wait for everything requested in between.  Keys past the end read the last one's
+  // row and columns past the row its last ones: nothing lane-wise stands around a load, all of a tile's are in flight together.
+  auto key_of = [&](int kt) { return min(kt * KT + kj, kv_end - 1); };
   V8<T> kr[U];
-  const int nu = (D + TPK * 8 - 1) / (TPK * 8);
-  auto load_tile = [&](int64_t row) {   // (no lane-wise condition around a load: all of them are in flight together)
-    const T* src = cache + row * D;
+  auto load_tile = [&](int page, int kt) {
+    const T* src = cache + ((int64_t)page * s.page_size + key_of(kt) % s.page_size) * D;
 #pragma unroll
-    for (int i = 0; i < U; ++i)
-      if (i < nu) kr[i] = load8(src + min(kcol + i * TPK * 8, D - 8));
+    for (int i = 0; i < U; ++i) kr[i] = load8(src + min(kcol + i * TPK * 8, D - 8));
   };
-  load_tile(page_of(kt0));
-  int64_t next_row = page_of(min(kt0 + 1, kt1 - 1));
+  load_tile(tab[key_of(kt0) / s.page_size], kt0);
+  int next_page = tab[key_of(min(kt0 + 1, kt1 - 1)) / s.page_size];
 
-  for (int u = tid; u < R * (D >> 3); u += 256) {   // the query rows
-    const int m = u / (D >> 3), k = (u - m * (D >> 3)) * 8;
-    *reinterpret_cast<V8<T>*>(qs + m * LDK + k) = m < nrows ? load8(static_cast<const T*>(p.q) + (grow0 + m) * D + k) : zero8<T>();
+  constexpr int QK = QREG ? U * TPK / 4 : 1;   // k-steps of a row
+  V8<T> qr[QK];
+  if constexpr (QREG) {   // (rows past the last one repeat it and are not stored)
+#pragma unroll
+    for (int k = 0; k < QK; ++k) qr[k] = load8(static_cast<const T*>(p.q) + (grow0 + min(r16, nrows - 1)) * D + k * 32 + 8 * kc);
+  } else {
+    for (int u = tid; u < R * (D >> 3); u += 256) {
+      const int m = u / (D >> 3), k = (u - m * (D >> 3)) * 8;
+      *reinterpret_cast<V8<T>*>(qs + m * LDK + k) = m < nrows ? load8(static_cast<const T*>(p.q) + (grow0 + m) * D + k) : zero8<T>();
+    }
   }
 
   f32x4 o[RT][NT];
@@ -111,24 +137,38 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
 
   for (int kt = kt0; kt < kt1; ++kt) {
 #pragma unroll
-    for (int i = 0; i < U; ++i)   // (a clamped column is written twice with the same values)
-      if (i < nu) *reinterpret_cast<V8<T>*>(ks + kj * LDK + min(kcol + i * TPK * 8, D - 8)) = kr[i];
+    for (int i = 0; i < U; ++i)   // (a clamped column is written again with the same values)
+      *reinterpret_cast<V8<T>*>(ks + kj * LDK + min(kcol + i * TPK * 8, D - 8)) = kr[i];
     if (kt + 1 < kt1) {
-      load_tile(next_row);
-      next_row = page_of(min(kt + 2, kt1 - 1));
+      load_tile(next_page, kt + 1);
+      next_page = tab[key_of(min(kt + 2, kt1 - 1)) / s.page_size];
     }
     __syncthreads();
     f32x4 sc[RT];
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) sc[rt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (wave < SW) {
+    if (SW == 4 || wave < SW) {
       const T* krow = ks + (wave * 16 + r16) * LDK + 8 * kc;
       const T* qrow = qs + r16 * LDK + 8 * kc;
-#pragma unroll 4
-      for (int k = 0; k < D; k += 32) {
-        const V8<T> kf = load8(krow + k);
+      if constexpr (QREG) {
+        f32x4 odd = f32x4{0.f, 0.f, 0.f, 0.f};   // (two chains of sums)
 #pragma unroll
-        for (int rt = 0; rt < RT; ++rt) mma(sc[rt], load8(qrow + rt * 16 * LDK + k), kf);
+        for (int k = 0; k < QK; ++k) mma(k & 1 ? odd : sc[0], qr[k], load8(krow + k * 32));
+        sc[0] += odd;
+      } else if constexpr (EXACT) {
+#pragma unroll
+        for (int k = 0; k < U * TPK * 8; k += 32) {
+          const V8<T> kf = load8(krow + k);
+#pragma unroll
+          for (int rt = 0; rt < RT; ++rt) mma(sc[rt], load8(qrow + rt * 16 * LDK + k), kf);
+        }
+      } else {
+#pragma unroll 2
+        for (int k = 0; k < D; k += 32) {
+          const V8<T> kf = load8(krow + k);
+#pragma unroll
+          for (int rt = 0; rt < RT; ++rt) mma(sc[rt], load8(qrow + rt * 16 * LDK + k), kf);
+        }
       }
       const int key = kt * KT + wave * 16 + r16;
 #pragma unroll
@@ -136,15 +176,12 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           sc[rt][r] = key <= lim[rt][r] ? sc[rt][r] * sc2 : -INFINITY;   // (keys past kv_end are past every row's limit)
-          float v = sc[rt][r];
-#pragma unroll
-          for (int x = 1; x < 16; x <<= 1) v = fmaxf(v, __shfl_xor(v, x, 64));
+          const float v = max16(sc[rt][r]);
           if (r16 == 0) sx[wave * R + rt * 16 + 4 * kc + r] = v;
         }
       }
     }
     __syncthreads();
-    bool moved = false;
     float alpha[RT][4];
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
@@ -159,23 +196,20 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
       for (int r = 0; r < 4; ++r) {
         const float mn = fmaxf(mrun[rt][r], mx[r]);
         alpha[rt][r] = exp2_hw(mrun[rt][r] - mn);
-        moved |= mn != mrun[rt][r];
         mrun[rt][r] = mn;
-        if (wave < SW) {
+        if (SW == 4 || wave < SW) {
           const T pr = (T)exp2_hw(sc[rt][r] - mn);
           lrun[rt][r] = fmaf(lrun[rt][r], alpha[rt][r], (float)pr);   // (what is summed is what multiplies the values)
           ps[(rt * 16 + 4 * kc + r) * LDP + wave * 16 + r16] = pr;
         }
       }
     }
-    if (__ballot(moved)) {
 #pragma unroll
-      for (int rt = 0; rt < RT; ++rt)
+    for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
-        for (int nt = 0; nt < NT; ++nt)
+      for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) o[rt][nt][r] *= alpha[rt][r];
-    }
+        for (int r = 0; r < 4; ++r) o[rt][nt][r] *= alpha[rt][r];
     __syncthreads();
 #pragma unroll
     for (int k = 0; k < KT; k += 32) {
@@ -184,12 +218,10 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
       for (int rt = 0; rt < RT; ++rt) pf[rt] = load8(ps + (rt * 16 + r16) * LDP + k + 8 * kc);
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt) {
-        const int dt = d0 + wave + 4 * nt;
-        if (dt < n16) {
-          const V8<T> vf = column8(ks, LDK, k + 8 * kc, dt * 16, r16);
+        const int dt = min(d0 + wave + 4 * nt, n16 - 1);   // (past the last one: computed, not stored)
+        const V8<T> vf = column8(ks, LDK, k + 8 * kc, dt * 16, r16);
 #pragma unroll
-          for (int rt = 0; rt < RT; ++rt) mma(o[rt][nt], pf[rt], vf);
-        }
+        for (int rt = 0; rt < RT; ++rt) mma(o[rt][nt], pf[rt], vf);
       }
     }
     __syncthreads();
@@ -200,9 +232,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const vmi_hy_late
   for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      float v = lrun[rt][r];
-#pragma unroll
-      for (int x = 1; x < 16; x <<= 1) v += __shfl_xor(v, x, 64);
+      const float v = sum16(lrun[rt][r]);
       if (r16 == 0) sx[wave * R + rt * 16 + 4 * kc + r] = v;
     }
   __syncthreads();
@@ -270,8 +300,8 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const vmi_hy_latent
     float a = 0.f;
 #pragma unroll 8
     for (int i = 0; i < p.splits; ++i) {
-      const float w = wt[i];
-      if (w != 0.f) a = fmaf(w, first[i * n * ld + k], a);
+      const float w = wt[i], v = first[i * n * ld + k];
+      a = fmaf(w, w != 0.f ? v : 0.f, a);   // (a part without keys holds whatever was there)
     }
     static_cast<T*>(p.out)[row * p.rank + k] = (T)a;
   }
@@ -316,6 +346,28 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_pr
       *reinterpret_cast<V8<T>*>(crow + k) = from_f32<T>(v);
     }
   }
+  if ((half & 7) == 0) {   // eight pairs at a time
+    const int per = half >> 3;
+    for (int u = tid; u < (p.heads + 1) * per; u += 256) {
+      const int h = u / per, i = (u - h * per) * 8;
+      const T* src = h < p.heads ? row + h * hd + p.dim : lat + p.rank;
+      T* dst = h < p.heads ? static_cast<T*>(p.q) + ((int64_t)t * p.heads + h) * D + p.rank : (crow ? crow + p.rank : nullptr);
+      if (!dst) continue;
+      const f32x8 a = to_f32<T>(load8(src + i)), b = to_f32<T>(load8(src + i + half));
+      f32x8 x, y;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float c = cs[2 * (i + e)], sn = cs[2 * (i + e) + 1];
+        x[e] = a[e] * c - b[e] * sn;
+        y[e] = b[e] * c + a[e] * sn;
+      }
+      *reinterpret_cast<V8<T>*>(dst + i) = from_f32<T>(x);
+      *reinterpret_cast<V8<T>*>(dst + i + half) = from_f32<T>(y);
+      if (i == 0)
+        for (int k = p.rot_n; k < p.rot; k += 8) *reinterpret_cast<V8<T>*>(dst + k) = load8(src + k);   // passes unrotated
+    }
+    return;
+  }
   // heads 0 .. heads - 1: the query's rotated part; "head" `heads`: the shared key
   T* qrow = static_cast<T*>(p.q) + (int64_t)t * p.heads * D;
   for (int u = tid; u < (p.heads + 1) * p.rot; u += 256) {
@@ -334,10 +386,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_pr
   }
 }
 
-template <typename T, int KT, int RT, int NT, int U>
+template <typename T, int KT, int RT, int NT, int U, bool EXACT = false>
 static int launch_attention(const vmi_hy_latent_attention_args& p, const vmi_hy_step& s, hipStream_t st) {
-  auto* fn = latent_attention_kernel<T, KT, RT, NT, U>;
-  const size_t lds = attention_lds<T, KT, RT>(p.rank + p.rot);
+  auto* fn = latent_attention_kernel<T, KT, RT, NT, U, EXACT>;
+  const int D = p.rank + p.rot;
+  const size_t lds = attention_lds<T, KT, RT>(D) - (EXACT && RT == 1 && sizeof(T) == 2 ? (size_t)16 * (D + pad_of<T>()) * sizeof(T) : 0);
   if (int rc = allow_lds(fn, lds, "vmi_hy_latent_attention")) return rc;
   const int zb = ((p.rank >> 4) + 4 * NT - 1) / (4 * NT);
   hipLaunchKernelGGL(fn, dim3(p.n_tiles, p.splits, zb), dim3(256), lds, st, p, s);
@@ -351,6 +404,8 @@ static int attention_width(const vmi_hy_latent_attention_args& p, const vmi_hy_s
   const int units = (p.rank + p.rot + 2048 / KT - 1) / (2048 / KT);   // of 8 elements of a cache row, per thread
   if (p.rank <= 128 && units <= 8) return launch_attention<T, KT, RT, 2, 8>(p, s, st);
   if (p.rank <= 256 && units <= 12) return launch_attention<T, KT, RT, 4, 12>(p, s, st);
+  if constexpr (sizeof(T) == 2 && KT == 64)
+    if (p.rank + p.rot == 576) return launch_attention<T, KT, RT, 8, 18, true>(p, s, st);
   if (units <= 20) return launch_attention<T, KT, RT, 8, 20>(p, s, st);
   if constexpr (RT == 1)
     if (units <= 32) return launch_attention<T, KT, RT, 8, 32>(p, s, st);

@@ -27,7 +27,7 @@ int launched(const char* who) {
 template <typename T, int BM, int KS>
 struct Chunk {
   static constexpr bool DEEP = BM == 16 && sizeof(T) == 2;   // few rows: bytes in flight are what counts
-  static constexpr int CS = DEEP ? 8 : 4;                     // k-steps a wave takes from a chunk
+  static constexpr int CS = DEEP && KS < 8 ? 8 : 4;                    // k-steps a wave takes from a chunk
   static constexpr int NB = DEEP ? 3 : 2;                     // chunks of weights in registers, NB - 1 of them ahead
   static constexpr int KC = 32 * CS * KS;                     // columns of x in a chunk
 };
@@ -37,20 +37,20 @@ template <typename T, int XK>
 struct XUnit;
 template <typename T>
 struct XUnit<T, VMI_HY_X_ROWS> {
-  V8<T> v;
+  V8<T> v = zero8<T>();
   __device__ __forceinline__ void load(const vmi_hy_linear_args& p, int64_t row, int64_t goff, int k) {
     v = load8(static_cast<const T*>(p.x) + goff + row * p.ldx + k);
   }
-  __device__ __forceinline__ V8<T> finish(const vmi_hy_linear_args&, int, float, float) const { return v; }
+  __device__ __forceinline__ V8<T> finish(const float*, int, float, float) const { return v; }
 };
 template <typename T>
 struct XUnit<T, VMI_HY_X_NORM> {
-  f32x8 v;
+  f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   __device__ __forceinline__ void load(const vmi_hy_linear_args& p, int64_t row, int64_t, int k) {
     v = load8(static_cast<const float*>(p.x) + row * p.ldx + k);
   }
-  __device__ __forceinline__ V8<T> finish(const vmi_hy_linear_args& p, int k, float mean, float rstd) const {
-    const f32x8 w = load8(p.norm_w + k);   // (zero past norm_n: padding columns come out as zeros)
+  __device__ __forceinline__ V8<T> finish(const float* nw, int k, float mean, float rstd) const {
+    const f32x8 w = load8(nw + k);   // (zero past norm_n: padding columns come out as zeros)
     f32x8 r;
 #pragma unroll
     for (int e = 0; e < 8; ++e) r[e] = (v[e] - mean) * rstd * w[e];
@@ -59,13 +59,13 @@ struct XUnit<T, VMI_HY_X_NORM> {
 };
 template <typename T>
 struct XUnit<T, VMI_HY_X_CONCAT> {
-  f32x8 v;
+  f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   __device__ __forceinline__ void load(const vmi_hy_linear_args& p, int64_t row, int64_t, int k) {
     const int half = p.K >> 1;
     const float* src = static_cast<const float*>(k < half ? p.x : p.x2);
     v = load8(src + row * p.ldx + (k < half ? k : k - half));
   }
-  __device__ __forceinline__ V8<T> finish(const vmi_hy_linear_args&, int, float, float) const { return from_f32<T>(v); }
+  __device__ __forceinline__ V8<T> finish(const float*, int, float, float) const { return from_f32<T>(v); }
 };
 
 template <typename T, int BM, int NW, int KS, int XK, int EPI>
@@ -78,12 +78,17 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   T* xs = reinterpret_cast<T*>(smem);                                   // [2][BM][LD]
   float* stats = reinterpret_cast<float*>(xs + (size_t)2 * BM * LD);    // [BM][2]
   float* red = stats + 2 * BM;                                          // [KS - 1][NW][MT][64][4]
+  // the norm's weight, in LDS: read from memory between the weight tiles it would wait for all of them
+  float* nwl = red + (KS - 1) * NW * MT * 256;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), nw = wave % NW, ks = wave / NW;
   const int kc = lane >> 4, r16 = lane & 15;
   // column blocks are dealt so that all row blocks of one stay on one XCD (workgroups go round-robin over the 8 of them): its
   // weights are read from HBM once
   const int MB = (p.M + BM - 1) / BM, NB = (p.N + 16 * NW - 1) / (16 * NW);
-  const int nb = (int)(blockIdx.x / (8 * MB)) * 8 + (int)(blockIdx.x & 7), mb = (int)(blockIdx.x >> 3) % MB, grp = blockIdx.y;
+  // (fewer than 8 of them: a plain order, or most XCDs would stay idle)
+  const int grp = blockIdx.y;
+  const int nb = NB < 8 ? (int)blockIdx.x % NB : (int)(blockIdx.x / (8 * MB)) * 8 + (int)(blockIdx.x & 7);
+  const int mb = NB < 8 ? (int)blockIdx.x / NB : (int)(blockIdx.x >> 3) % MB;
   if (nb >= NB) return;
   const int m0 = mb * BM, n0 = (nb * NW + nw) * 16, nks = p.K >> 5;
   const bool nvalid = n0 < p.N;
@@ -95,8 +100,10 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   auto load_w = [&](V8<T>(&dst)[CS], int c) {
 #pragma unroll
     for (int j = 0; j < CS; ++j) {
-      const int k = c * (CS * KS) + ks * CS + j;
-      dst[j] = k < nks && nvalid ? load8(wp + (int64_t)k * 512) : zero8<T>();
+      // (no lane-wise condition around a load, here or for x: all of a chunk's are in flight together.  A k-step past the last
+      //  one reads that one again and meets zeros of x)
+      const int k = min(c * (CS * KS) + ks * CS + j, nks - 1);
+      dst[j] = load8(wp + (int64_t)k * 512);
     }
   };
 #pragma unroll
@@ -111,6 +118,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   if constexpr (XK == VMI_HY_X_NORM) {   // row statistics, one pass around the row's first element: no cancellation to speak of
     constexpr int NWV = TH / 64;
     const int mrows = min(BM, p.M - m0);
+    for (int k = tid * 4; k < p.K; k += TH * 4) *reinterpret_cast<f32x4*>(nwl + k) = *reinterpret_cast<const f32x4*>(p.norm_w + k);
     for (int mbase = wave; mbase < mrows; mbase += 4 * NWV) {
       const float* row[4];
       float sh[4], s[4], q[4];
@@ -158,10 +166,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
     srow[i] = source_row(xm[i]);
     xin[i] = m0 + xm[i] < p.M;
     mean[i] = rstd[i] = 0.f;
-    if (!xin[i]) {   // rows past M: zeros in both buffers, once
-      *reinterpret_cast<V8<T>*>(xs + xm[i] * LD + xk[i]) = zero8<T>();
-      *reinterpret_cast<V8<T>*>(xs + (BM + xm[i]) * LD + xk[i]) = zero8<T>();
-    } else if constexpr (XK == VMI_HY_X_NORM) {
+    if (XK == VMI_HY_X_NORM && xin[i]) {
       mean[i] = stats[2 * xm[i]];
       rstd[i] = stats[2 * xm[i] + 1];
     }
@@ -169,8 +174,8 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   XUnit<T, XK> xu[UPT];
   auto load_x = [&](int c) {
 #pragma unroll
-    for (int i = 0; i < UPT; ++i)
-      if (xin[i] && c * KC + xk[i] < p.K) xu[i].load(p, srow[i], goff, c * KC + xk[i]);
+    for (int i = 0; i < UPT; ++i)   // (a wave whose rows all lie past M reads none: a scalar condition)
+      if ((wave * 64 + i * TH) / UPR < p.M - m0) xu[i].load(p, srow[i], goff, min(c * KC + xk[i], p.K - 8));
   };
   load_x(0);
 
@@ -180,21 +185,20 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
   auto step = [&](int c, V8<T>(&cur)[CS], V8<T>(&nxt)[CS]) {
     T* dst = xs + (size_t)(c & 1) * BM * LD;
 #pragma unroll
-    for (int i = 0; i < UPT; ++i)
-      if (xin[i] && c * KC + xk[i] < p.K)
-        *reinterpret_cast<V8<T>*>(dst + xm[i] * LD + xk[i]) = xu[i].finish(p, c * KC + xk[i], mean[i], rstd[i]);
-    if (c + 1 < nchunk) load_x(c + 1);
-    if (c + NB_W - 1 < nchunk) load_w(nxt, c + NB_W - 1);
-    __syncthreads();   // (two buffers: the writes of chunk c + 1 go where chunk c - 1 was read, which every wave has left behind)
-    const int kn = min(nks - c * (CS * KS), CS * KS) - ks * CS;   // k-steps of this chunk that are this wave's
-#pragma unroll
-    for (int j = 0; j < CS; ++j) {
-      if (j < kn) {
-#pragma unroll
-        for (int mi = 0; mi < MT; ++mi)
-          mma(acc[mi], cur[j], load8(dst + (mi * 16 + r16) * LD + (ks * CS + j) * 32 + 8 * kc));
-      }
+    for (int u = 0; u < UPT; ++u) {
+      const int k = c * KC + xk[u];
+      const V8<T> v = xu[u].finish(nwl, min(k, p.K - 8), mean[u], rstd[u]);
+      *reinterpret_cast<V8<T>*>(dst + xm[u] * LD + xk[u]) = xin[u] && k < p.K ? v : zero8<T>();
     }
+    // x first, and the weights whatever is left (past the end: one tile again, a cache hit): a wait for x then always knows how
+    // many younger loads it may leave in flight
+    if (c + 1 < nchunk) load_x(c + 1);
+    load_w(nxt, c + NB_W - 1);
+    __syncthreads();   // (two buffers: the writes of chunk c + 1 go where chunk c - 1 was read, which every wave has left behind)
+#pragma unroll
+    for (int j = 0; j < CS; ++j)
+#pragma unroll
+      for (int mi = 0; mi < MT; ++mi) mma(acc[mi], cur[j], load8(dst + (mi * 16 + r16) * LD + (ks * CS + j) * 32 + 8 * kc));
   };
   for (int c = 0; c < nchunk; c += NB_W) {   // chunk c sits in wb[c % NB_W]; the one behind it has been used up
 #pragma unroll
@@ -261,11 +265,12 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
 template <typename T, int BM, int NW, int KS, int XK, int EPI>
 static int launch_linear(const vmi_hy_linear_args& p, hipStream_t st) {
   constexpr int KC = Chunk<T, BM, KS>::KC, LD = KC + 16 / (int)sizeof(T);
-  const size_t lds = (size_t)2 * BM * LD * sizeof(T) + 2 * BM * 4 + (size_t)(KS - 1) * NW * (BM / 16) * 64 * 16;
+  const size_t lds = (size_t)2 * BM * LD * sizeof(T) + 2 * BM * 4 + (size_t)(KS - 1) * NW * (BM / 16) * 64 * 16 +
+                     (XK == VMI_HY_X_NORM ? (size_t)p.K * 4 : 0);
   auto* fn = linear_kernel<T, BM, NW, KS, XK, EPI>;
   if (int rc = allow_lds(fn, lds, "vmi_hy_linear")) return rc;
   const int MB = (p.M + BM - 1) / BM, NB = (p.N + 16 * NW - 1) / (16 * NW);
-  hipLaunchKernelGGL(fn, dim3((NB + 7) / 8 * 8 * MB, p.groups), dim3(NW * KS * 64), lds, st, p);
+  hipLaunchKernelGGL(fn, dim3((NB < 8 ? NB : (NB + 7) / 8 * 8) * MB, p.groups), dim3(NW * KS * 64), lds, st, p);
   return launched("vmi_hy_linear");
 }
 
@@ -276,9 +281,10 @@ static int linear_shape(const vmi_hy_linear_args& p, hipStream_t st) {
   if (p.M <= 32) {
     const int64_t wgs = slabs * ((p.M + 15) / 16);
     if (wgs >= 2048) return launch_linear<T, 16, 4, 1, XK, EPI>(p, st);
-    if (wgs >= 512 || p.K < 256) return launch_linear<T, 16, 2, 2, XK, EPI>(p, st);
-    if (wgs >= 192 || p.K < 1024) return launch_linear<T, 16, 1, 4, XK, EPI>(p, st);
-    return launch_linear<T, 16, 1, 8, XK, EPI>(p, st);
+    if (wgs >= 400 || p.K < 256) return launch_linear<T, 16, 2, 2, XK, EPI>(p, st);
+    if constexpr (sizeof(T) == 2)
+      if (wgs < 192 && p.K >= 1024) return launch_linear<T, 16, 1, 8, XK, EPI>(p, st);
+    return launch_linear<T, 16, 1, 4, XK, EPI>(p, st);
   }
   if (p.M <= 96 || slabs / 4 * ((p.M + 63) / 64) < 256) return launch_linear<T, 32, 4, 1, XK, EPI>(p, st);
   return launch_linear<T, 64, 4, 1, XK, EPI>(p, st);

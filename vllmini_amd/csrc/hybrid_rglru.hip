@@ -65,8 +65,7 @@ __device__ __forceinline__ f32x8 conv8(const vmi_hy_rglru_args& p, const RowMeta
 }
 
 template <typename T>
-__device__ __forceinline__ void store_out8(const vmi_hy_rglru_args& p, int t, int c, const f32x8& s) {
-  const f32x8 y = to_f32<T>(load8(static_cast<const T*>(p.yx) + (int64_t)t * p.ldx + c));
+__device__ __forceinline__ void store_out8(const vmi_hy_rglru_args& p, int t, int c, const f32x8& s, const f32x8& y) {
   f32x8 o;
 #pragma unroll
   for (int e = 0; e < 8; ++e) o[e] = s[e] * gelu_tanh(y[e]);
@@ -74,7 +73,7 @@ __device__ __forceinline__ void store_out8(const vmi_hy_rglru_args& p, int t, in
 }
 
 template <typename T, int BM, int TAPS>
-__global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args p, const vmi_hy_step s) {
+__global__ __launch_bounds__(256, 2) void rglru_tile_kernel(const vmi_hy_rglru_args p, const vmi_hy_step s) {
   constexpr int MT = BM / 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   auto& L = *reinterpret_cast<Lds<T, BM>*>(smem);
@@ -108,27 +107,95 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
   const int64_t gsz = (int64_t)bw * bw, nks = bw >> 5;
   const T* wr = static_cast<const T*>(p.gates) + blk * gsz + ((int64_t)((cin >> 4) + wave) * nks * 64 + lane) * 8;
   const T* wi = wr + p.blocks * gsz;
+  // requested now, used behind the products
+  const int cl = wave * 16 + 4 * kc;
+  f32x4 br, bi, dec, S0[MT];
+  if (wvalid) {
+    br = *reinterpret_cast<const f32x4*>(p.gate_b + c0 + cl);
+    bi = *reinterpret_cast<const f32x4*>(p.gate_b + p.width + c0 + cl);
+    dec = *reinterpret_cast<const f32x4*>(p.decay + c0 + cl);
+  }
+  __syncthreads();   // meta is there
+#pragma unroll
+  for (int mi = 0; mi < MT; ++mi) {
+    const RowMeta& r = L.meta[mi * 16 + r16];
+    S0[mi] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (wvalid && r.seq >= 0 && r.first && r.ctx > 0) S0[mi] = *reinterpret_cast<const f32x4*>(p.state + (int64_t)r.slot * p.width + c0 + cl);
+  }
+  constexpr int YU = (BM * (CT / 8) + 255) / 256;   // this thread's units of the output: y
+  V8<T> yv[YU];
+#pragma unroll
+  for (int i = 0; i < YU; ++i) {
+    const int m = (tid + i * 256) / (CT / 8), k = ((tid + i * 256) % (CT / 8)) * 8;
+    yv[i] = load8(static_cast<const T*>(p.yx) + (int64_t)(t0 + min(m, rows - 1)) * p.ldx + c0 + min(k, nch - 8));
+  }
   for (int k0 = 0; k0 < bw; k0 += KCH) {
     const int kn = min(KCH, bw - k0);
-    __syncthreads();   // meta is there; the previous chunk has been read
-#pragma unroll 2
-    for (int u = tid; u < BM * (KCH / 8); u += 256) {   // (a row of LDS is KCH channels, the last chunk may have fewer)
-      const int m = u / (KCH / 8), k = (u % (KCH / 8)) * 8;
+    // few rows: the chunk's gate tiles are in flight while u is computed (many rows: those registers are worth a second workgroup)
+    constexpr bool AHEAD = BM == 16;
+    V8<T> fr[AHEAD ? KCH / 32 : 1], fi[AHEAD ? KCH / 32 : 1];
+    if constexpr (AHEAD) {
+#pragma unroll
+      for (int k = 0; k < KCH / 32; ++k) {
+        const int64_t at = (int64_t)((k0 >> 5) + min(k, (kn >> 5) - 1)) * 512;
+        if (wvalid) fr[k] = load8(wr + at), fi[k] = load8(wi + at);
+      }
+    }
+    if (k0 > 0) __syncthreads();   // the previous chunk has been read
+    auto conv_row = [&](int m, int k) {
       const RowMeta& r = L.meta[m];
       if (r.seq >= 0 && k < kn) *reinterpret_cast<V8<T>*>(L.u + m * LDU + k) = from_f32<T>(conv8<T, TAPS>(p, r, t0 + m, blk * bw + k0 + k));
       else if (k < kn) *reinterpret_cast<V8<T>*>(L.u + m * LDU + k) = zero8<T>();
+    };
+    if constexpr (BM == 64 && TAPS > 0) {
+      // eight channels of eight consecutive rows: inside one portion, past its first taps, the rows share their inputs
+      const int k = (tid % (KCH / 8)) * 8, m0 = (tid / (KCH / 8)) * 8;
+      const RowMeta &ra = L.meta[m0], &rb = L.meta[m0 + 7];
+      if (k < kn && ra.seq >= 0 && ra.seq == rb.seq && t0 + m0 - (TAPS - 1) >= ra.qs) {
+        const int c = blk * bw + k0 + k;
+        const T* in = static_cast<const T*>(p.yx) + (int64_t)(t0 + m0 - (TAPS - 1)) * p.ldx + p.width + c;
+        V8<T> v[TAPS + 7];
+        f32x8 w[TAPS];
+#pragma unroll
+        for (int j = 0; j < TAPS + 7; ++j) v[j] = load8(in + (int64_t)j * p.ldx);
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[j] = load8(p.conv_w + (int64_t)j * p.width + c);
+        const f32x8 b = load8(p.conv_b + c);
+#pragma unroll
+        for (int m = 0; m < 8; ++m) {
+          f32x8 acc = b;
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[j][e], (float)v[m + j][e], acc[e]);
+          *reinterpret_cast<V8<T>*>(L.u + (m0 + m) * LDU + k) = from_f32<T>(acc);
+        }
+      } else {
+#pragma unroll 1
+        for (int m = 0; m < 8; ++m) conv_row(m0 + m, k);
+      }
+    } else {
+#pragma unroll 2
+      for (int u = tid; u < BM * (KCH / 8); u += 256) conv_row(u / (KCH / 8), (u % (KCH / 8)) * 8);
     }
     __syncthreads();
     if (wvalid) {
-#pragma unroll 2
-      for (int k = 0; k < kn >> 5; ++k) {
-        const V8<T> fr = load8(wr + (int64_t)((k0 >> 5) + k) * 512), fi = load8(wi + (int64_t)((k0 >> 5) + k) * 512);
+      auto product = [&](int k, const V8<T>& a, const V8<T>& b) {
 #pragma unroll
         for (int mi = 0; mi < MT; ++mi) {
           const V8<T> fu = load8(L.u + (mi * 16 + r16) * LDU + k * 32 + 8 * kc);
-          mma(ar[mi], fr, fu);
-          mma(ai[mi], fi, fu);
+          mma(ar[mi], a, fu);
+          mma(ai[mi], b, fu);
         }
+      };
+      if constexpr (AHEAD) {
+#pragma unroll
+        for (int k = 0; k < KCH / 32; ++k)
+          if (k < kn >> 5) product(k, fr[k], fi[k]);
+      } else {
+#pragma unroll 2
+        for (int k = 0; k < kn >> 5; ++k)
+          product(k, load8(wr + (int64_t)((k0 >> 5) + k) * 512), load8(wi + (int64_t)((k0 >> 5) + k) * 512));
       }
     }
   }
@@ -147,25 +214,20 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
   }
   __syncthreads();
   if (wvalid) {
-    const int cl = wave * 16 + 4 * kc, c = c0 + cl;
-    const f32x4 br = *reinterpret_cast<const f32x4*>(p.gate_b + c), bi = *reinterpret_cast<const f32x4*>(p.gate_b + p.width + c);
-    const f32x4 dec = *reinterpret_cast<const f32x4*>(p.decay + c);
 #pragma unroll
     for (int mi = 0; mi < MT; ++mi) {
       const int m = mi * 16 + r16;
       const RowMeta& r = L.meta[m];
       const f32x4 u = *reinterpret_cast<const f32x4*>(L.b + m * LDA + cl);
-      f32x4 S0 = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (r.seq >= 0 && r.first && r.ctx > 0) S0 = *reinterpret_cast<const f32x4*>(p.state + (int64_t)r.slot * p.width + c);
       f32x4 a, b;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float la = dec[e] * sigmoid(ar[mi][e] + br[e]);
-        a[e] = expf(la);
-        b[e] = sqrtf(-expm1f(2.f * la)) * sigmoid(ai[mi][e] + bi[e]) * u[e];
+        a[e] = exp_hw(la);
+        b[e] = __builtin_amdgcn_sqrtf(one_minus_exp(-2.f * la, a[e] * a[e])) * sigmoid(ai[mi][e] + bi[e]) * u[e];
         if (r.seq < 0) a[e] = 1.f, b[e] = 0.f;
         if (r.first) {
-          b[e] = fmaf(a[e], S0[e], b[e]);
+          b[e] = fmaf(a[e], S0[mi][e], b[e]);
           a[e] = 0.f;
         }
       }
@@ -208,9 +270,10 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
   }
   __syncthreads();
   const int lead_end = lead0 ? min(rows, L.meta[0].qs + L.meta[0].len - t0) : 0;   // rows of the leading segment
-  for (int u = tid; u < rows * (CT / 8); u += 256) {
-    const int m = u / (CT / 8), k = (u % (CT / 8)) * 8;
-    if (k >= nch) continue;
+#pragma unroll
+  for (int i = 0; i < YU; ++i) {
+    const int u = tid + i * 256, m = u / (CT / 8), k = (u % (CT / 8)) * 8;
+    if (m >= rows || k >= nch) continue;
     const RowMeta& r = L.meta[m];
     const f32x8 S = *reinterpret_cast<const f32x8*>(L.b + m * LDA + k);
     const int t = t0 + m, c = c0 + k;
@@ -224,7 +287,7 @@ __global__ __launch_bounds__(256) void rglru_tile_kernel(const vmi_hy_rglru_args
       *reinterpret_cast<f32x8*>(p.scratch + ((int64_t)s.T + t) * p.width + c) = *reinterpret_cast<const f32x8*>(L.a + m * LDA + k);
     }
     if (lead) continue;
-    store_out8<T>(p, t, c, S);
+    store_out8<T>(p, t, c, S, to_f32<T>(yv[i]));
     if (r.last) *reinterpret_cast<f32x8*>(p.state + (int64_t)r.slot * p.width + c) = S;
   }
   // the convolution tail of entries that end in this tile, into its other half
@@ -288,7 +351,7 @@ __global__ __launch_bounds__(256) void rglru_finish_kernel(const vmi_hy_rglru_ar
   f32x8 o;
 #pragma unroll
   for (int e = 0; e < 8; ++e) o[e] = fmaf(P[e], k[e], S[e]);
-  store_out8<T>(p, t, c, o);
+  store_out8<T>(p, t, c, o, to_f32<T>(load8(static_cast<const T*>(p.yx) + (int64_t)t * p.ldx + c)));
 }
 
 template <typename T, int BM, int TAPS>

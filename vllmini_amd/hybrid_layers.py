@@ -6,9 +6,10 @@ once (heads, blocks and ranks zero-padded to multiples of 32, so no kernel has a
     ClampedGLU        the feed-forward with a clamped gated unit
     ConcatProjection  x <- W [x ; x0]
 
-The residual stream is float32 (`Residual`).  Up to DENSE_MIN_TOKENS tokens a layer runs on the streaming kernels with everything
-fused around the products (norm in front, gated unit / head gate / residual add behind); above it the big products go to the
-vendor library (F.linear, as the prefill of the GPT-2 decoder does) with one elementwise kernel between two of them.
+The residual stream is float32 (`Residual`).  Steps of few tokens run on the streaming kernels with everything fused around the
+products (norm in front, gated unit / head gate / residual add behind); from DENSE_MIN_TOKENS tokens on (from DENSE_MIN_TOKENS_LARGE
+for matrices of DENSE_LARGE elements) the products go to the vendor library (F.linear, as the prefill of the GPT-2 decoder does)
+with one elementwise kernel between two of them.
 """
 from __future__ import annotations
 
@@ -21,6 +22,11 @@ from . import hybrid_ops as ops
 from .hybrid_ops import MatrixTiles, StepLayout, pad32
 
 DENSE_MIN_TOKENS = 48
+DENSE_MIN_TOKENS_LARGE, DENSE_LARGE = 17, 32 << 20
+
+
+def dense(tokens: int, w: MatrixTiles) -> bool:
+    return tokens >= DENSE_MIN_TOKENS or (tokens >= DENSE_MIN_TOKENS_LARGE and w.N * w.K >= DENSE_LARGE)
 
 
 def float_product(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -50,7 +56,7 @@ class Head:
         self.scaled = (norm.weight * self.scale, norm.n, norm.eps)
 
     def run(self, x: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
-        if rows.numel() >= DENSE_MIN_TOKENS:
+        if dense(rows.numel(), self.w):
             h = ops.add_norm(x.index_select(0, rows), None, self.scaled, self.dtype)
             return float_product(h, self.w.dense)[:, : self.vocab]
         return ops.linear(x, self.w, norm=self.norm.args, rows=rows, float_out=(self.vocab, self.scale))
@@ -75,22 +81,19 @@ class Residual:
         self.pending = None
         return h
 
-    def dense(self, step: StepLayout) -> bool:
-        return step.T >= DENSE_MIN_TOKENS
-
     def branch_in(self, norm: Norm, w: MatrixTiles, step: StepLayout, bias: Optional[torch.Tensor] = None,
                   dense_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
         """norm(x) W^T (+ bias) in the element type."""
-        if self.dense(step):
+        if dense(step.T, w):
             return F.linear(self.normed(norm), w.dense, dense_bias)
         return ops.linear(self.settle(), w, norm=norm.args, bias=bias)
 
     def branch_out(self, o: torch.Tensor, w: MatrixTiles, step: StepLayout) -> None:
         """x += o W^T."""
-        if self.dense(step):
+        if dense(step.T, w):
             self.pending = F.linear(o, w.dense)
         else:
-            ops.linear(o, w, residual=True, out=self.x)
+            ops.linear(o, w, residual=True, out=self.settle())
 
 
 def spread(t: torch.Tensor, dim: int, index: torch.Tensor, size: int) -> torch.Tensor:
@@ -209,7 +212,7 @@ class ClampedGLU:
         self.w_out = MatrixTiles(spread(spread(down, 1, torch.arange(ff), fp), 0, torch.arange(width), E), dtype, dense=True)
 
     def run(self, res: Residual, step: StepLayout) -> None:
-        if res.dense(step):
+        if dense(step.T, self.w_in):
             h = ops.glu(F.linear(res.normed(self.norm), self.w_in.dense), self.limit)
         else:
             h = ops.linear(res.settle(), self.w_in, norm=self.norm.args, glu_limit=self.limit)
@@ -226,7 +229,7 @@ class ConcatProjection:
 
     def run(self, res: Residual, x0: torch.Tensor) -> None:
         x = res.settle()
-        if x.shape[0] >= DENSE_MIN_TOKENS:
+        if dense(x.shape[0], self.w):
             res.x = float_product(ops.concat(x, x0, res.dtype), self.w.dense)      # (the stream stays float32)
         else:
             res.x = ops.linear(x, self.w, x2=x0, float_out=(x.shape[1], 1.0))
