@@ -62,7 +62,8 @@ class AttentionPlan:
 
 class HybridDecoder:
     MAX_STEP_TOKENS = 16384        # longer prompts run in several portions
-    FILL_WORKGROUPS = 512          # a step with fewer query tiles splits the keys of each over several workgroups
+    FILL_WORKGROUPS = {1: 512, 2: 256, 4: 256}     # by row tiles, what the chip holds at once: a step with fewer query tiles splits
+                                                   # the keys of each over several workgroups
     KEY_TILE = 64
 
     def __init__(self, model: HybridModel, pool: PagedKVPool, pad_batch_to: int = 0):
@@ -84,10 +85,10 @@ class HybridDecoder:
         self._sets: Dict[tuple, dict] = {}             # captured decode steps
 
     # ---- the step's layout -----------------------------------------------------------------------------------------------
-    def _split_of(self, n_tiles: int, heads: int, row: int, max_keys: int, T: int) -> int:
-        if n_tiles >= self.FILL_WORKGROUPS // 2:
+    def _split_of(self, n_tiles: int, row_tiles: int, heads: int, row: int, max_keys: int, T: int) -> int:
+        if n_tiles > 128:
             return 1
-        want = min(self.FILL_WORKGROUPS // max(n_tiles, 1), -(-max_keys // (2 * self.KEY_TILE)))
+        want = min(self.FILL_WORKGROUPS[row_tiles] // max(n_tiles, 1), -(-max_keys // self.KEY_TILE))
         fit = (256 << 20) // max(1, T * heads * (row + 2) * 4)             # (bytes of the partial results)
         n = 1
         while 2 * n <= min(want, fit, 128):
@@ -133,7 +134,7 @@ class HybridDecoder:
             t = np.full((nt, 2), -1, dtype=np.int32)
             t[: len(ent), 0], t[: len(ent), 1] = ent, first
             sec[f"tiles{len(plans)}"] = t.reshape(-1)
-            plans.append((rt, self._split_of(nt, heads, row, max_keys, T), nt))
+            plans.append((rt, self._split_of(nt, rt, heads, row, max_keys, T), nt))
         offs, total = {}, 0
         for name, v in sec.items():
             offs[name] = (total, len(v))
