@@ -9,8 +9,8 @@
 #                   does not change
 #   make layer      libvmi_gpt2_layer.so (include/vmi_gpt2_layer.h): the decode harness's own library — the GPT-2 block's
 #                   linear layers; one unit, part of `make` / `all`
-#   make hybrid     libvmi_hybrid.so (include/vmi_hybrid.h): the layers of decoders with recurrent blocks and latent
-#                   attention; three units, part of `make` / `all`
+#   make hybrid     libvmi_hybrid.so (include/vmi_hybrid.h): the layers of decoders that mix recurrences, linear and
+#                   softmax attention; part of `make` / `all`
 HIPCC  ?= hipcc
 ARCH   ?= gfx950
 # -ffp-contract=off: the fp16 p*v products are rounded before the fp16 adds (the reference's rounding points)
@@ -35,14 +35,14 @@ DEPS   := $(wildcard $(CSRC)/*.hpp) $(wildcard $(CSRC)/*.inc) include/vmi_paged_
 LAYER_LIB := $(OUTDIR)/libvmi_gpt2_layer.so
 
 HYBRID_LIB := $(OUTDIR)/libvmi_hybrid.so
-HYBRID_UNITS := hybrid_linear hybrid_rglru hybrid_latent
+HYBRID_UNITS := hybrid_linear hybrid_rglru hybrid_latent hybrid_state hybrid_attention
 HYBRID_SRCS := $(HYBRID_UNITS:%=$(CSRC)/%.hip)
 
 all: $(LIB) $(LAYER_LIB) $(HYBRID_LIB) oracle
 
 hybrid: $(HYBRID_LIB)
 
-$(HYBRID_LIB): $(HYBRID_SRCS) $(CSRC)/hybrid_common.hpp include/vmi_hybrid.h
+$(HYBRID_LIB): $(HYBRID_SRCS) $(CSRC)/hybrid_common.hpp $(CSRC)/hybrid_softmax.hpp include/vmi_hybrid.h
 	mkdir -p $(OUTDIR)
 	$(HIPCC) $(filter-out -ffp-contract=off,$(FLAGS)) -shared $(HYBRID_SRCS) -o $@
 

@@ -83,7 +83,7 @@ def test_linear_kinds(dtype, M, N, K):
     close(ops.linear(xf, t, norm=(nw, n, 1e-5), rows=rows, float_out=(cols, 0.3)), (h @ W.T)[rows.long(), :cols] * 0.3, dtype, tol32=1e-4)
     y = h @ W.T
     gate, up = y[:, 0::2].clamp(max=0.8), y[:, 1::2].clamp(-0.8, 0.8)
-    close(ops.linear(xf, t, norm=(nw, n, 1e-5), glu_limit=0.8), gate * torch.sigmoid(1.702 * gate) * (up + 1), dtype, tol32=1e-4, tol16=3e-2)
+    close(ops.linear(xf, t, norm=(nw, n, 1e-5), glu=ops.GatedUnit.clamped(0.8)), gate * torch.sigmoid(1.702 * gate) * (up + 1), dtype, tol32=1e-4, tol16=3e-2)
     if K % 64 == 0:
         a, b = rnd(M, K // 2).to(dev()), rnd(M, K // 2).to(dev())
         close(ops.linear(a, t, x2=b, float_out=(N, 1.0)), torch.cat([a, b], 1).double() @ W.T, dtype)
@@ -126,7 +126,7 @@ def test_elementwise_ends(dtype, n):
     assert not h[:, n:].any()
     v = (torch.randn(7, 2 * ld, generator=g) * 2).to(dtype).to(dev())
     gate, up = v[:, 0::2].double().clamp(max=1.25), v[:, 1::2].double().clamp(-1.25, 1.25)
-    close(ops.glu(v, 1.25), gate * torch.sigmoid(1.702 * gate) * (up + 1), dtype)
+    close(ops.glu(v, ops.GatedUnit.clamped(1.25)), gate * torch.sigmoid(1.702 * gate) * (up + 1), dtype)
     table = torch.zeros(40, ld, dtype=torch.bfloat16, device=dev())
     table[:, :n] = torch.randn(40, n, generator=g).to(dev())
     ids = torch.tensor([0, 39, 7], device=dev())

@@ -84,8 +84,9 @@ EXTRAS_LIB_PATH = os.path.join(OUT_DIR, "libvmi_paged_attention_extras.so")
 SRC_LAYER = os.path.join(CSRC, "gpt2_layer.hip")
 LAYER_LIB_PATH = os.path.join(OUT_DIR, "libvmi_gpt2_layer.so")
 
-# the layers of decoders with recurrent blocks and latent attention (include/vmi_hybrid.h): three units, loaded by hybrid_ops.py only
-SRC_HYBRID = [os.path.join(CSRC, f"hybrid_{t}.hip") for t in ("linear", "rglru", "latent")]
+# the layers of decoders that mix recurrences, linear and softmax attention (include/vmi_hybrid.h), loaded by hybrid_ops.py only
+SRC_HYBRID = [os.path.join(CSRC, f"hybrid_{t}.hip") for t in ("linear", "rglru", "latent", "state", "attention")]
+HDRS_HYBRID = [os.path.join(CSRC, f"hybrid_{t}.hpp") for t in ("common", "softmax")]
 HYBRID_LIB_PATH = os.path.join(OUT_DIR, "libvmi_hybrid.so")
 
 ARCH = "gfx950"
@@ -228,7 +229,7 @@ def hybrid_is_stale() -> bool:
     if not os.path.exists(HYBRID_LIB_PATH):
         return True
     t = os.path.getmtime(HYBRID_LIB_PATH)
-    deps = [*SRC_HYBRID, os.path.join(CSRC, "hybrid_common.hpp"), os.path.join(INCLUDE, "vmi_hybrid.h")]
+    deps = [*SRC_HYBRID, *HDRS_HYBRID, os.path.join(INCLUDE, "vmi_hybrid.h")]
     return any(os.path.getmtime(d) > t for d in deps)
 
 

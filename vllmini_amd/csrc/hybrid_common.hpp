@@ -85,12 +85,13 @@ __device__ __forceinline__ float one_minus_exp(float x, float e) {
   const float s = x * fmaf(-x, fmaf(-x, fmaf(-x, fmaf(-x, fmaf(-x, 1.f / 720.f, 1.f / 120.f), 1.f / 24.f), 1.f / 6.f), 0.5f), 1.f);
   return x < 0.25f ? s : 1.f - e;
 }
-// the clamped gated unit: gate g (already a product), up-projection u
-__device__ __forceinline__ float glu(float g, float u, float limit) {
+// the gated unit: gate g (already a product), up-projection u.  limit infinite, alpha 1, up 0: silu(g) u
+__device__ __forceinline__ float glu(float g, float u, float limit, float alpha, float up) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g * sigmoid(1.702f * g) * (u + 1.f);
+  return g * sigmoid(alpha * g) * (u + up);
 }
+__device__ __forceinline__ float silu(float z) { return z * sigmoid(z); }
 
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

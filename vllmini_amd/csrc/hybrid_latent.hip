@@ -7,51 +7,9 @@
 // statistics meet in LDS; then wave w adds the value columns w, w + 4, ... (tiles of 16) of all rows, the value operand read
 // column-wise from the same LDS rows (ds_read_b64_tr_b16).  Scores, softmax and accumulators are fp32.  A sequence whose rows do
 // not fill the chip has its keys dealt to `splits` workgroups, whose unnormalised parts a second kernel adds up.
-#include "hybrid_common.hpp"
+#include "hybrid_softmax.hpp"
 
 namespace vmi_hybrid {
-
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-
-// 8 consecutive rows (keys) of one column of an LDS tile, as a matrix operand's fragment: lane = (kc, column r16)
-__device__ __forceinline__ b16x8 column8(const b16* tile, int ld, int row0, int col0, int r16) {
-  const b16* a = tile + (row0 + (r16 >> 2)) * ld + col0 + 4 * (r16 & 3);
-  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a);
-  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a + 4 * ld));
-  // (whole vectors are cast: a bit_cast of one vector element takes element 0 on this compiler)
-  return __builtin_shufflevector(__builtin_bit_cast(b16x4, lo), __builtin_bit_cast(b16x4, hi), 0, 1, 2, 3, 4, 5, 6, 7);
-}
-__device__ __forceinline__ f32x8 column8(const float* tile, int ld, int row0, int col0, int r16) {
-  f32x8 r;
-#pragma unroll
-  for (int e = 0; e < 8; ++e) r[e] = tile[(row0 + e) * ld + col0 + r16];
-  return r;
-}
-
-// maximum / sum over the 16 lanes that share kc, on the cross-lane paths of the vector unit (no LDS round trip)
-template <int CTRL>
-__device__ __forceinline__ float dpp(float v) {
-  return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
-}
-__device__ __forceinline__ float max16(float v) {
-  v = fmaxf(v, dpp<0xB1>(v));    // quad_perm [1,0,3,2]
-  v = fmaxf(v, dpp<0x4E>(v));    // quad_perm [2,3,0,1]
-  v = fmaxf(v, dpp<0x141>(v));   // row_half_mirror
-  return fmaxf(v, dpp<0x140>(v));   // row_mirror
-}
-__device__ __forceinline__ float sum16(float v) {
-  v += dpp<0xB1>(v);
-  v += dpp<0x4E>(v);
-  v += dpp<0x141>(v);
-  return v + dpp<0x140>(v);
-}
-
-__device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
-
-template <typename T>
-constexpr int pad_of() {
-  return 16 / (int)sizeof(T);
-}
 
 template <typename T, int KT, int RT>
 inline size_t attention_lds(int D) {
@@ -267,46 +225,6 @@ __global__ __launch_bounds__(256, EXACT && RT == 1 ? 2 : 1) void latent_attentio
   }
 }
 
-// out[row] = sum over splits of 2^(m_s - m) part_s / sum of 2^(m_s - m) l_s; one workgroup per (token, head)
-template <typename T>
-__global__ __launch_bounds__(256) void latent_combine_kernel(const vmi_hy_latent_attention_args p, const vmi_hy_step s) {
-  const int64_t row = blockIdx.x, n = (int64_t)s.T * p.heads;
-  if (s.tok_seq[row / p.heads] < 0) return;
-  const int ld = p.rank + 2;
-  __shared__ float wt[128];   // weight of every part (at most 128 of them)
-  const float* first = p.partial + row * ld;
-  if (threadIdx.x < 64) {
-    float m[2], l[2], top = -1e30f, sum = 0.f;
-#pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      const int i = threadIdx.x + 64 * j;
-      m[j] = i < p.splits ? first[i * n * ld + p.rank] : -1e30f;
-      l[j] = i < p.splits ? first[i * n * ld + p.rank + 1] : 0.f;
-      top = fmaxf(top, m[j]);
-    }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) top = fmaxf(top, __shfl_xor(top, o, 64));
-#pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      m[j] = l[j] > 0.f ? exp2_hw(m[j] - top) : 0.f;   // (a part without keys holds no values)
-      sum += m[j] * l[j];
-    }
-    sum = wave_sum(sum);
-#pragma unroll
-    for (int j = 0; j < 2; ++j) wt[threadIdx.x + 64 * j] = m[j] / sum;
-  }
-  __syncthreads();
-  for (int k = threadIdx.x; k < p.rank; k += blockDim.x) {
-    float a = 0.f;
-#pragma unroll 8
-    for (int i = 0; i < p.splits; ++i) {
-      const float w = wt[i], v = first[i * n * ld + k];
-      a = fmaf(w, w != 0.f ? v : 0.f, a);   // (a part without keys holds whatever was there)
-    }
-    static_cast<T*>(p.out)[row * p.rank + k] = (T)a;
-  }
-}
-
 // RMS norm of the latent, rotation of the shared key and of the query parts; one workgroup per token
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const vmi_hy_latent_prep_args p, const vmi_hy_step s) {
@@ -395,7 +313,7 @@ static int launch_attention(const vmi_hy_latent_attention_args& p, const vmi_hy_
   const int zb = ((p.rank >> 4) + 4 * NT - 1) / (4 * NT);
   hipLaunchKernelGGL(fn, dim3(p.n_tiles, p.splits, zb), dim3(256), lds, st, p, s);
   if (p.splits > 1)
-    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3((int64_t)s.T * p.heads), dim3(p.rank > 128 ? 256 : 128), 0, st, p, s);
+    launch_combine<T>(Combine{p.partial, p.out, nullptr, s.tok_seq, (int64_t)p.heads * p.rank, 0, s.T, p.heads, p.rank, p.splits}, st);
   return launched("vmi_hy_latent_attention");
 }
 

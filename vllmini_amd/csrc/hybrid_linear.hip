@@ -126,7 +126,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       for (int i = 0; i < 4; ++i) {
         const int m = mbase + i * NWV < mrows ? mbase + i * NWV : mbase;
         row[i] = static_cast<const float*>(p.x) + source_row(m) * p.ldx;
-        sh[i] = row[i][0];
+        sh[i] = p.rms ? 0.f : row[i][0];
         s[i] = q[i] = 0.f;
       }
       for (int k = lane * 4; k < p.K; k += 256) {
@@ -143,7 +143,7 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float ms = wave_sum(s[i]) / (float)p.norm_n, mq = wave_sum(q[i]) / (float)p.norm_n;
+        const float ms = p.rms ? 0.f : wave_sum(s[i]) / (float)p.norm_n, mq = wave_sum(q[i]) / (float)p.norm_n;
         const int m = mbase + i * NWV;
         if (lane == 0 && m < mrows) {
           stats[2 * m] = sh[i] + ms;
@@ -249,9 +249,21 @@ __global__ __launch_bounds__(NW* KS * 64) void linear_kernel(const vmi_hy_linear
       }
     } else if constexpr (EPI == VMI_HY_E_GLU) {
       typename Elem<T>::v2 o;
-      o[0] = (T)glu(acc[mi][0], acc[mi][1], p.scale);
-      o[1] = (T)glu(acc[mi][2], acc[mi][3], p.scale);
+      o[0] = (T)glu(acc[mi][0], acc[mi][1], p.scale, p.glu_alpha, p.glu_up);
+      o[1] = (T)glu(acc[mi][2], acc[mi][3], p.scale, p.glu_alpha, p.glu_up);
       *reinterpret_cast<typename Elem<T>::v2*>(static_cast<T*>(p.y) + yoff + (n >> 1)) = o;
+    } else if constexpr (EPI == VMI_HY_E_STORE_GLU) {
+      if (n0 < p.n_split) {
+        V4<T> o;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = (T)acc[mi][r];
+        *reinterpret_cast<V4<T>*>(static_cast<T*>(p.y) + yoff + n) = o;
+      } else {
+        typename Elem<T>::v2 o;
+        o[0] = (T)glu(acc[mi][0], acc[mi][1], p.scale, p.glu_alpha, p.glu_up);
+        o[1] = (T)glu(acc[mi][2], acc[mi][3], p.scale, p.glu_alpha, p.glu_up);
+        *reinterpret_cast<typename Elem<T>::v2*>(static_cast<T*>(p.y2) + (int64_t)m * p.ldy2 + ((n - p.n_split) >> 1)) = o;
+      }
     } else {   // VMI_HY_E_GATED
       const float g = sigmoid((float)static_cast<const T*>(p.gate)[(int64_t)m * p.ldg + grp]);
       V4<T> o;
@@ -299,6 +311,7 @@ static int linear_kind(const vmi_hy_linear_args& p, hipStream_t st) {
     case VMI_HY_X_NORM * 8 + VMI_HY_E_STORE: return linear_shape<T, VMI_HY_X_NORM, VMI_HY_E_STORE>(p, st);
     case VMI_HY_X_NORM * 8 + VMI_HY_E_FLOAT: return linear_shape<T, VMI_HY_X_NORM, VMI_HY_E_FLOAT>(p, st);
     case VMI_HY_X_NORM * 8 + VMI_HY_E_GLU: return linear_shape<T, VMI_HY_X_NORM, VMI_HY_E_GLU>(p, st);
+    case VMI_HY_X_NORM * 8 + VMI_HY_E_STORE_GLU: return linear_shape<T, VMI_HY_X_NORM, VMI_HY_E_STORE_GLU>(p, st);
     case VMI_HY_X_CONCAT * 8 + VMI_HY_E_FLOAT: return linear_shape<T, VMI_HY_X_CONCAT, VMI_HY_E_FLOAT>(p, st);
     default: return fail(VMI_HY_E_ARG, "vmi_hy_linear", "this combination of input and epilogue is not built");
   }
@@ -321,7 +334,7 @@ __global__ __launch_bounds__(256) void embed_kernel(const int64_t* __restrict__ 
 // one workgroup per row; a row of up to 4 * 4096 columns stays in registers between the three passes
 template <typename T>
 __global__ __launch_bounds__(256) void add_norm_kernel(float* x, const T* add, int64_t ld_add, const float* norm_w, T* out, int n,
-                                                       int ld, float eps) {
+                                                       int ld, float eps, int rms) {
   __shared__ float part[2][4];
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   float* row = x + (int64_t)t * ld;
@@ -350,10 +363,13 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* x, const T* add, i
     s += a[0] + a[1] + a[2] + a[3];
   }
   if (!out) return;
-  s = wave_sum(s);
-  if (lane == 0) part[0][wave] = s;
-  __syncthreads();
-  const float mean = (part[0][0] + part[0][1] + part[0][2] + part[0][3]) / (float)n;
+  float mean = 0.f;
+  if (!rms) {
+    s = wave_sum(s);
+    if (lane == 0) part[0][wave] = s;
+    __syncthreads();
+    mean = (part[0][0] + part[0][1] + part[0][2] + part[0][3]) / (float)n;
+  }
   float q = 0.f;
   auto dev2 = [&](const f32x4& a, int k) {
 #pragma unroll
@@ -384,6 +400,82 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* x, const T* add, i
   for (int k = (tid + MAXV * 256) * 4; k < ld; k += 1024) put(*reinterpret_cast<const f32x4*>(row + k), k);
 }
 
+// x += scale (rms norm of a + rms norm of b) + add; one workgroup per row
+template <typename T>
+__global__ __launch_bounds__(256) void merge_kernel(float* x, const T* a, int64_t ld_a, const T* b, int64_t ld_b, const T* add,
+                                                    int64_t ld_add, const float* wa, const float* wb, int n, int ld, float eps,
+                                                    float scale) {
+  __shared__ float part[2][4];
+  const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  a += (int64_t)t * ld_a;
+  b += (int64_t)t * ld_b;
+  float sa = 0.f, sb = 0.f;
+  for (int k = tid * 4; k < ld; k += 1024) {   // (padding columns are zeros)
+    const V4<T> va = *reinterpret_cast<const V4<T>*>(a + k), vb = *reinterpret_cast<const V4<T>*>(b + k);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      sa = fmaf((float)va[e], (float)va[e], sa);
+      sb = fmaf((float)vb[e], (float)vb[e], sb);
+    }
+  }
+  sa = wave_sum(sa);
+  sb = wave_sum(sb);
+  if (lane == 0) part[0][wave] = sa, part[1][wave] = sb;
+  __syncthreads();
+  const float ra = scale / sqrtf((part[0][0] + part[0][1] + part[0][2] + part[0][3]) / (float)n + eps);
+  const float rb = scale / sqrtf((part[1][0] + part[1][1] + part[1][2] + part[1][3]) / (float)n + eps);
+  float* row = x + (int64_t)t * ld;
+  for (int k = tid * 4; k < ld; k += 1024) {
+    const V4<T> va = *reinterpret_cast<const V4<T>*>(a + k), vb = *reinterpret_cast<const V4<T>*>(b + k);
+    const f32x4 w0 = *reinterpret_cast<const f32x4*>(wa + k), w1 = *reinterpret_cast<const f32x4*>(wb + k);
+    f32x4 v = *reinterpret_cast<const f32x4*>(row + k);
+    if (add) {
+      const V4<T> d = *reinterpret_cast<const V4<T>*>(add + (int64_t)t * ld_add + k);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += (float)d[e];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] += (float)va[e] * ra * w0[e] + (float)vb[e] * rb * w1[e];
+    *reinterpret_cast<f32x4*>(row + k) = v;
+  }
+}
+
+// every head's o over its root mean square, times a weight and the activated gate; 16 lanes per (token, head)
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate, int64_t ldg,
+                                                             const float* __restrict__ norm_w, T* __restrict__ out, int64_t ldo,
+                                                             int64_t rows, int heads, int vdim, int vdim_n, float eps, int act) {
+  const int64_t row = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  if (row >= rows) return;
+  const int64_t t = row / heads;
+  const int h = (int)(row - t * heads), l = threadIdx.x & 15;
+  o += row * vdim;
+  gate += t * ldg + (int64_t)h * vdim;
+  out += t * ldo + (int64_t)h * vdim;
+  float ss = 0.f;
+  for (int k = l * 4; k < vdim; k += 64) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+#pragma unroll
+  for (int m = 8; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  const float r = 1.f / sqrtf(ss / (float)vdim_n + eps);
+  for (int k = l * 4; k < vdim; k += 64) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
+    const V4<T> g = *reinterpret_cast<const V4<T>*>(gate + k);
+    f32x4 w = f32x4{1.f, 1.f, 1.f, 1.f};
+    if (norm_w) w = *reinterpret_cast<const f32x4*>(norm_w + k);
+    V4<T> y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float z = (float)g[e];
+      y[e] = (T)(v[e] * r * w[e] * (act == VMI_HY_ACT_SILU ? silu(z) : sigmoid(z)));
+    }
+    *reinterpret_cast<V4<T>*>(out + k) = y;
+  }
+}
+
 // out [T, 2 n] = (x | x2) in the element type
 template <typename T>
 __global__ __launch_bounds__(256) void concat_kernel(const float* __restrict__ x, const float* __restrict__ x2, T* __restrict__ out, int n) {
@@ -394,13 +486,13 @@ __global__ __launch_bounds__(256) void concat_kernel(const float* __restrict__ x
 
 template <typename T>
 __global__ __launch_bounds__(256) void glu_kernel(const T* __restrict__ in, int64_t ld_in, T* __restrict__ out, int64_t ld_out, int n,
-                                                  float limit) {
+                                                  float limit, float alpha, float up) {
   const int t = blockIdx.y, j = (blockIdx.x * 256 + threadIdx.x) * 4;
   if (j >= n) return;
   const V8<T> v = load8(in + (int64_t)t * ld_in + 2 * j);
   V4<T> o;
 #pragma unroll
-  for (int e = 0; e < 4; ++e) o[e] = (T)glu((float)v[2 * e], (float)v[2 * e + 1], limit);
+  for (int e = 0; e < 4; ++e) o[e] = (T)glu((float)v[2 * e], (float)v[2 * e + 1], limit, alpha, up);
   *reinterpret_cast<V4<T>*>(out + (int64_t)t * ld_out + j) = o;
 }
 
@@ -444,11 +536,13 @@ int vmi_hy_linear(const vmi_hy_linear_args* a, void* stream) {
   static const char* who = "vmi_hy_linear";
   if (!a || !a->x || !a->w || !a->y || a->M <= 0 || a->N <= 0 || a->K <= 0 || a->groups <= 0 || a->dtype < 0 || a->dtype > 1 ||
       (a->x_kind == VMI_HY_X_NORM && (!a->norm_w || a->norm_n <= 0 || a->norm_n > a->K)) || (a->x_kind == VMI_HY_X_CONCAT && !a->x2) ||
-      (a->epilogue == VMI_HY_E_GATED && !a->gate))
+      (a->epilogue == VMI_HY_E_GATED && !a->gate) || (a->epilogue == VMI_HY_E_STORE_GLU && !a->y2))
     return fail(VMI_HY_E_ARG, who, "null pointer, non-positive size or unknown element type");
   if ((a->K & 31) || (a->N & 15) || (a->x_kind == VMI_HY_X_CONCAT && (a->K & 63)) || (a->ldx & 7) || (a->x_gstride & 7) ||
       (a->epilogue != VMI_HY_E_FLOAT && ((a->ldy & 3) || (a->y_gstride & 3))) || ((uintptr_t)a->x & 15) || ((uintptr_t)a->w & 15) ||
-      ((uintptr_t)a->y & 15) || (a->epilogue == VMI_HY_E_FLOAT && (a->n_out <= 0 || a->n_out > a->N || a->groups != 1)))
+      ((uintptr_t)a->y & 15) || (a->epilogue == VMI_HY_E_FLOAT && (a->n_out <= 0 || a->n_out > a->N || a->groups != 1)) ||
+      (a->epilogue == VMI_HY_E_STORE_GLU && (a->n_split < 0 || a->n_split > a->N || (a->n_split & 15) || (a->ldy2 & 1) ||
+                                             ((uintptr_t)a->y2 & 7) || a->groups != 1)))
     return fail(VMI_HY_E_SHAPE, who, "needs K % 32 == 0, N % 16 == 0 and 16-byte aligned rows");
   DeviceScope dev(a->device);
   if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
@@ -468,7 +562,7 @@ int vmi_hy_embed(const int64_t* ids, const void* table, float* x, int32_t T, int
 }
 
 int vmi_hy_add_norm(float* x, const void* add, int64_t ld_add, const float* norm_w, void* out, int32_t T, int32_t n, int32_t ld,
-                    float eps, int32_t dtype, int32_t device, void* stream) {
+                    float eps, int32_t rms, int32_t dtype, int32_t device, void* stream) {
   static const char* who = "vmi_hy_add_norm";
   if (!x || T <= 0 || n <= 0 || ld < n || (ld & 3) || (add && (ld_add & 3)) || (out && !norm_w)) return fail(VMI_HY_E_ARG, who, "bad argument");
   DeviceScope dev(device);
@@ -476,15 +570,15 @@ int vmi_hy_add_norm(float* x, const void* add, int64_t ld_add, const float* norm
   hipStream_t st = static_cast<hipStream_t>(stream);
   if (dtype == VMI_HY_BF16)
     hipLaunchKernelGGL(add_norm_kernel<b16>, dim3(T), dim3(256), 0, st, x, static_cast<const b16*>(add), ld_add, norm_w,
-                       static_cast<b16*>(out), n, ld, eps);
+                       static_cast<b16*>(out), n, ld, eps, rms);
   else
     hipLaunchKernelGGL(add_norm_kernel<float>, dim3(T), dim3(256), 0, st, x, static_cast<const float*>(add), ld_add, norm_w,
-                       static_cast<float*>(out), n, ld, eps);
+                       static_cast<float*>(out), n, ld, eps, rms);
   return launched(who);
 }
 
-int vmi_hy_glu(const void* in, int64_t ld_in, void* out, int64_t ld_out, int32_t T, int32_t n, float limit, int32_t dtype,
-               int32_t device, void* stream) {
+int vmi_hy_glu(const void* in, int64_t ld_in, void* out, int64_t ld_out, int32_t T, int32_t n, float limit, float alpha,
+               float up, int32_t dtype, int32_t device, void* stream) {
   static const char* who = "vmi_hy_glu";
   if (!in || !out || T <= 0 || T > 65535 || n <= 0 || (n & 3) || (ld_in & 7) || (ld_out & 3)) return fail(VMI_HY_E_ARG, who, "bad argument");
   DeviceScope dev(device);
@@ -492,9 +586,49 @@ int vmi_hy_glu(const void* in, int64_t ld_in, void* out, int64_t ld_out, int32_t
   hipStream_t st = static_cast<hipStream_t>(stream);
   const dim3 grid((n / 4 + 255) / 256, T);
   if (dtype == VMI_HY_BF16)
-    hipLaunchKernelGGL(glu_kernel<b16>, grid, dim3(256), 0, st, static_cast<const b16*>(in), ld_in, static_cast<b16*>(out), ld_out, n, limit);
+    hipLaunchKernelGGL(glu_kernel<b16>, grid, dim3(256), 0, st, static_cast<const b16*>(in), ld_in, static_cast<b16*>(out), ld_out, n,
+                       limit, alpha, up);
   else
-    hipLaunchKernelGGL(glu_kernel<float>, grid, dim3(256), 0, st, static_cast<const float*>(in), ld_in, static_cast<float*>(out), ld_out, n, limit);
+    hipLaunchKernelGGL(glu_kernel<float>, grid, dim3(256), 0, st, static_cast<const float*>(in), ld_in, static_cast<float*>(out), ld_out, n,
+                       limit, alpha, up);
+  return launched(who);
+}
+
+int vmi_hy_merge(float* x, const void* a, int64_t ld_a, const void* b, int64_t ld_b, const void* add, int64_t ld_add, const float* wa,
+                 const float* wb, int32_t T, int32_t n, int32_t ld, float eps, float scale, int32_t dtype, int32_t device,
+                 void* stream) {
+  static const char* who = "vmi_hy_merge";
+  if (!x || !a || !b || !wa || !wb || T <= 0 || n <= 0 || ld < n || (ld & 3) || (ld_a & 3) || (ld_b & 3) || (add && (ld_add & 3)))
+    return fail(VMI_HY_E_ARG, who, "bad argument");
+  DeviceScope dev(device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  if (dtype == VMI_HY_BF16)
+    hipLaunchKernelGGL(merge_kernel<b16>, dim3(T), dim3(256), 0, st, x, static_cast<const b16*>(a), ld_a, static_cast<const b16*>(b), ld_b,
+                       static_cast<const b16*>(add), ld_add, wa, wb, n, ld, eps, scale);
+  else
+    hipLaunchKernelGGL(merge_kernel<float>, dim3(T), dim3(256), 0, st, x, static_cast<const float*>(a), ld_a, static_cast<const float*>(b),
+                       ld_b, static_cast<const float*>(add), ld_add, wa, wb, n, ld, eps, scale);
+  return launched(who);
+}
+
+int vmi_hy_head_norm_gate(const float* o, const void* gate, int64_t ldg, const float* norm_w, void* out, int64_t ldo, int32_t T,
+                          int32_t heads, int32_t vdim, int32_t vdim_n, float eps, int32_t act, int32_t dtype, int32_t device,
+                          void* stream) {
+  static const char* who = "vmi_hy_head_norm_gate";
+  if (!o || !gate || !out || T <= 0 || heads <= 0 || vdim <= 0 || (vdim & 3) || (ldg & 3) || (ldo & 3) || vdim_n <= 0 || vdim_n > vdim)
+    return fail(VMI_HY_E_ARG, who, "bad argument");
+  DeviceScope dev(device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  const int64_t rows = (int64_t)T * heads;
+  const dim3 grid((rows + 15) / 16);
+  if (dtype == VMI_HY_BF16)
+    hipLaunchKernelGGL(head_norm_gate_kernel<b16>, grid, dim3(256), 0, st, o, static_cast<const b16*>(gate), ldg, norm_w,
+                       static_cast<b16*>(out), ldo, rows, heads, vdim, vdim_n, eps, act);
+  else
+    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, st, o, static_cast<const float*>(gate), ldg, norm_w,
+                       static_cast<float*>(out), ldo, rows, heads, vdim, vdim_n, eps, act);
   return launched(who);
 }
 

@@ -1,0 +1,591 @@
+// Linear attention with a matrix state per head (include/vmi_hybrid.h): retention (fixed decay per head, rotated q and k) and the
+// gated delta rule (decay per head and key channel, short convolutions, unit q and k).  All of it is fp32 from the projections on.
+//
+// Portions: cut into chunks of 16 rows.  With G_i the decay accumulated from the chunk's start through row i (log), the rows obey
+//     u_i + beta_i sum_{j<i} A_ij u_j = beta_i (v_i - S^T k_i e^{G_i}),    A_ij = sum_c k_ic k_jc e^{G_ic - G_jc}
+//     o_i = S^T (q_i e^{G_i}) + sum_{j<=i} B_ij u_j,                       B_ij = sum_c q_ic k_jc e^{G_ic - G_jc}
+//     S  <- e^{G_15} S + sum_j (k_j e^{G_15 - G_j}) u_j^T
+// (retention: u = v, no A).  state_prep_kernel makes, for every (chunk, head) independently, the triangular system's solutions
+// W = (I + beta A)^-1 beta (k e^G) and U0 = (I + beta A)^-1 beta v, q e^G, k e^{G_15 - G} and B; exponents are always of differences
+// i >= j, so nothing can overflow.  state_scan_kernel then walks a state's chunks: u = U0 - W S, o = q e^G S + B u, S update, on
+// v_mfma_f32_16x16x4_f32.  A wave owns 16 value columns of one head's state for the whole walk, in the matrix core's result layout
+// (lane (kc, r16): rows 4 kc + r of column r16), which is at the same time the operand layout of the next product: no LDS, no
+// barrier, and rows past a portion's end are zeros in every operand.
+//
+// Steps of single tokens: state_step_kernel reads each state once, keeps it in registers between the correction and the read-out,
+// and writes it back; convolution, gates, norm and output gate ride along.
+#include "hybrid_common.hpp"
+
+namespace vmi_hybrid {
+
+constexpr int CH = 16;        // rows of a chunk
+constexpr int MAX_TAPS = 16;
+
+__device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+struct Portion {
+  int qs, len, ctx, slot, flip;
+};
+__device__ __forceinline__ Portion portion(const vmi_hy_step& s, int e) {
+  return Portion{s.q_start[e], s.q_len[e], s.ctx[e], s.state_slot[e], s.flip[e]};
+}
+
+// 8 channels from channel c of the token in packed row t, through the convolution and silu.  TAPS = 0: any number of taps
+template <typename T, int TAPS>
+__device__ __forceinline__ f32x8 conv_silu8(const vmi_hy_state_args& p, const Portion& r, int C, int t, int c) {
+  f32x8 acc = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  const T* in = static_cast<const T*>(p.proj) + c;
+  const int taps = TAPS ? TAPS : p.taps, pos = r.ctx + t - r.qs;
+  const T* tail = static_cast<const T*>(p.tail) + ((int64_t)r.slot * 2 + r.flip) * (taps - 1) * C + c;   // positions ctx - (taps - 1) ..
+  auto tap = [&](int j) {
+    const int back = taps - 1 - j;
+    const T* src = t - back >= r.qs ? in + (int64_t)(t - back) * p.ldp
+                   : pos >= back    ? tail + (int64_t)(pos - back - (r.ctx - (taps - 1))) * C
+                                    : in + (int64_t)t * p.ldp;
+    const V8<T> v = load8(src);
+    const f32x8 w = load8(p.conv_w + (int64_t)j * C + c);
+    const bool on = pos >= back;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[e], on ? (float)v[e] : 0.f, acc[e]);
+  };
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) tap(j);
+  } else {
+    for (int j = 0; j < taps; ++j) tap(j);
+  }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) acc[e] = silu(acc[e]);
+  return acc;
+}
+
+// the last taps - 1 inputs of an entry, channels [c0, c0 + n), into the half of the tail this step does not read
+template <typename T>
+__device__ __forceinline__ void write_tail(const vmi_hy_state_args& p, const Portion& r, int C, int c0, int n, int tid, int threads) {
+  const int nt = p.taps - 1, per = n >> 3;
+  const T* from = static_cast<const T*>(p.tail) + ((int64_t)r.slot * 2 + r.flip) * nt * C;
+  T* to = static_cast<T*>(p.tail) + ((int64_t)r.slot * 2 + (r.flip ^ 1)) * nt * C;
+  for (int u = tid; u < nt * per; u += threads) {
+    const int e = u / per, c = c0 + (u - e * per) * 8, pos = r.ctx + r.len - nt + e;   // the position this row stands for
+    V8<T> v = zero8<T>();
+    if (pos >= r.ctx) v = load8(static_cast<const T*>(p.proj) + (int64_t)(r.qs + pos - r.ctx) * p.ldp + c);
+    else if (pos >= 0) v = load8(from + (int64_t)(pos - (r.ctx - nt)) * C + c);
+    *reinterpret_cast<V8<T>*>(to + (int64_t)e * C + c) = v;
+  }
+}
+
+// cos, sin of position * frequency, the angle reduced in fp64: exact to fp32 at any position
+__device__ __forceinline__ f32x2 turn(double pos, double f) {
+  const double a = pos * f;
+  const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
+  return f32x2{cosf(r), sinf(r)};
+}
+
+// q and k of one head, `rows` of them from packed row t0, rotated, k / sqrt(dim_n), into LDS
+template <typename T>
+__device__ __forceinline__ void rotated_rows(const vmi_hy_state_args& p, int t0, int pos0, int rows, int n, int h, int hk, float* ql,
+                                             float* kl, int ld, int tid) {
+  const int half = p.rot_n >> 1;
+  const float ks = 1.f / sqrtf((float)p.dim_n);
+  for (int u = tid; u < rows * p.dim; u += 256) {
+    const int m = u / p.dim, i = u - m * p.dim;
+    float q = 0.f, k = 0.f;
+    if (m < n && i < p.rot_n) {
+      if (i >= half) continue;
+      const T* qr = static_cast<const T*>(p.proj) + (int64_t)(t0 + m) * p.ldp + (int64_t)hk * p.dim;
+      const T* kr = qr + (int64_t)p.kv_heads * p.dim;
+      const f32x2 cs = turn((double)(pos0 + m), p.freq[i]);
+      const float qa = (float)qr[i], qb = (float)qr[i + half], ka = (float)kr[i], kb = (float)kr[i + half];
+      ql[m * ld + i] = qa * cs[0] - qb * cs[1];
+      ql[m * ld + i + half] = qb * cs[0] + qa * cs[1];
+      kl[m * ld + i] = (ka * cs[0] - kb * cs[1]) * ks;
+      kl[m * ld + i + half] = (kb * cs[0] + ka * cs[1]) * ks;
+      continue;
+    }
+    if (m < n) {
+      const T* qr = static_cast<const T*>(p.proj) + (int64_t)(t0 + m) * p.ldp + (int64_t)hk * p.dim;
+      q = (float)qr[i];
+      k = (float)qr[(int64_t)p.kv_heads * p.dim + i] * ks;
+    }
+    ql[m * ld + i] = q;
+    kl[m * ld + i] = k;
+  }
+}
+
+// what one (chunk, head) hands to the walk, in floats
+struct Scratch {
+  int q, w, k, u, b, d, size;
+  __host__ __device__ Scratch(int kind, int dim, int vdim) {
+    q = 0;                                                // [16][dim]   q e^G
+    w = q + CH * dim;                                     // [16][dim]   W (delta only)
+    k = w + (kind == VMI_HY_DELTA ? CH * dim : 0);        // [dim][16]   k e^{G_15 - G}
+    u = k + CH * dim;                                     // [vdim][16]  U0
+    b = u + CH * vdim;                                    // [16][16]    B
+    d = b + CH * CH;                                      // [dim]       e^{G_15}
+    size = d + dim;
+  }
+};
+
+inline size_t prep_lds(int kind, int dim, int vdim) {
+  return ((size_t)CH * (dim + 4) * (kind == VMI_HY_DELTA ? 3 : 2) + (size_t)CH * (vdim + 4) + 2 * CH * 20 + CH) * sizeof(float);
+}
+
+template <typename T, int KIND, int TAPS>
+__global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int dim = p.dim, vdim = p.vdim, LD = dim + 4, LDV = vdim + 4;
+  float* ql = lds;                                             // [16][LD]
+  float* kl = ql + CH * LD;                                    // [16][LD]
+  float* gl = kl + CH * LD;                                    // [16][LD] (delta)
+  float* vl = gl + (KIND == VMI_HY_DELTA ? CH * LD : 0);       // [16][LDV]
+  float* Al = vl + CH * LDV;                                   // [16][20] beta_i A_ij
+  float* Bl = Al + CH * 20;                                    // [16][20]
+  float* be = Bl + CH * 20;                                    // [16]
+  const int tid = threadIdx.x, h = blockIdx.y, hk = h / (p.heads / p.kv_heads);
+  const int e = s.chunks[2 * blockIdx.x], first = s.chunks[2 * blockIdx.x + 1];
+  const Portion r = portion(s, e);
+  const int t0 = r.qs + first, n = min(CH, r.len - first), C = 2 * p.kv_heads * dim + p.heads * vdim;
+  const int cq = hk * dim, ck = (p.kv_heads + hk) * dim, cv = 2 * p.kv_heads * dim + h * vdim;
+  const Scratch sc(KIND, dim, vdim);
+  float* out = p.scratch + ((int64_t)blockIdx.x * p.heads + h) * sc.size;
+
+  if constexpr (KIND == VMI_HY_DELTA) {
+    const int ud = dim >> 3, uv = vdim >> 3;
+    for (int u = tid; u < CH * (2 * ud + uv); u += 256) {
+      const int m = u / (2 * ud + uv);
+      int c = u - m * (2 * ud + uv);
+      float* dst;
+      int ch;
+      if (c < ud) dst = ql + m * LD + c * 8, ch = cq + c * 8;
+      else if (c < 2 * ud) c -= ud, dst = kl + m * LD + c * 8, ch = ck + c * 8;
+      else c -= 2 * ud, dst = vl + m * LDV + c * 8, ch = cv + c * 8;
+      f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (m < n) v = conv_silu8<T, TAPS>(p, r, C, t0 + m, ch);
+      *reinterpret_cast<f32x4*>(dst) = f32x4{v[0], v[1], v[2], v[3]};
+      *reinterpret_cast<f32x4*>(dst + 4) = f32x4{v[4], v[5], v[6], v[7]};
+    }
+    if (tid < CH) be[tid] = tid < n ? sigmoid((float)static_cast<const T*>(p.beta)[(int64_t)(t0 + tid) * p.ldp + h]) : 0.f;
+    const float rate = p.rate[h];
+    for (int c = tid; c < dim; c += 256) {
+      const float bias = p.dt_bias[(int64_t)h * dim + c];
+      float G = 0.f;
+#pragma unroll 4
+      for (int m = 0; m < CH; ++m) {
+        const float z = (float)static_cast<const T*>(p.z)[(int64_t)(t0 + min(m, n - 1)) * p.ldz + (int64_t)h * dim + c] + bias;
+        if (m < n) G -= rate * softplus(z);
+        gl[m * LD + c] = G;
+      }
+    }
+    __syncthreads();
+    {   // unit lengths: 16 lanes a row
+      const int m = tid >> 4, l = tid & 15;
+      float a = 0.f, b = 0.f;
+      for (int c = l; c < dim; c += 16) {
+        a = fmaf(ql[m * LD + c], ql[m * LD + c], a);
+        b = fmaf(kl[m * LD + c], kl[m * LD + c], b);
+      }
+#pragma unroll
+      for (int o = 8; o > 0; o >>= 1) a += __shfl_xor(a, o, 64), b += __shfl_xor(b, o, 64);
+      a = 1.f / sqrtf((a + 1e-6f) * (float)p.dim_n);
+      b = 1.f / sqrtf(b + 1e-6f);
+      for (int c = l; c < dim; c += 16) {
+        ql[m * LD + c] *= a;
+        kl[m * LD + c] *= b;
+      }
+    }
+    __syncthreads();
+    {
+      const int i = tid >> 4, j = tid & 15;
+      float a = 0.f, b = 0.f;
+      if (j <= i) {
+        for (int c = 0; c < dim; c += 4) {
+          const f32x4 qi = *reinterpret_cast<const f32x4*>(ql + i * LD + c), ki = *reinterpret_cast<const f32x4*>(kl + i * LD + c);
+          const f32x4 kj = *reinterpret_cast<const f32x4*>(kl + j * LD + c), gi = *reinterpret_cast<const f32x4*>(gl + i * LD + c);
+          const f32x4 gj = *reinterpret_cast<const f32x4*>(gl + j * LD + c);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            const float w = kj[x] * exp_hw(gi[x] - gj[x]);
+            a = fmaf(ki[x], w, a);
+            b = fmaf(qi[x], w, b);
+          }
+        }
+      }
+      Al[i * 20 + j] = j < i ? a * be[i] : 0.f;
+      out[sc.b + i * CH + j] = j <= i ? b : 0.f;
+    }
+    __syncthreads();
+    // forward substitution, a column a thread: of W (dim of them), of U0 (vdim)
+    for (int col = tid; col < dim + vdim; col += 256) {
+      const bool isw = col < dim;
+      const int c = isw ? col : col - dim;
+      float x[CH];
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        float v = isw ? kl[i * LD + c] * exp_hw(gl[i * LD + c]) : vl[i * LDV + c];
+        v *= be[i];
+#pragma unroll
+        for (int j = 0; j < i; ++j) v = fmaf(-Al[i * 20 + j], x[j], v);
+        x[i] = v;
+      }
+      if (isw) {
+        const float G = gl[(CH - 1) * LD + c];
+        out[sc.d + c] = exp_hw(G);
+#pragma unroll
+        for (int i = 0; i < CH; ++i) {
+          out[sc.w + i * dim + c] = x[i];
+          out[sc.q + i * dim + c] = ql[i * LD + c] * exp_hw(gl[i * LD + c]);
+        }
+#pragma unroll
+        for (int i = 0; i < CH; i += 4) {
+          f32x4 k;
+#pragma unroll
+          for (int y = 0; y < 4; ++y) k[y] = kl[(i + y) * LD + c] * exp_hw(G - gl[(i + y) * LD + c]);
+          *reinterpret_cast<f32x4*>(out + sc.k + c * CH + i) = k;
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < CH; i += 4) *reinterpret_cast<f32x4*>(out + sc.u + c * CH + i) = f32x4{x[i], x[i + 1], x[i + 2], x[i + 3]};
+      }
+    }
+    if (first + CH >= r.len && p.taps > 1) {   // the chunk that ends the portion
+      write_tail<T>(p, r, C, cv, vdim, tid, 256);
+      if (h == hk * (p.heads / p.kv_heads)) {
+        write_tail<T>(p, r, C, cq, dim, tid, 256);
+        write_tail<T>(p, r, C, ck, dim, tid, 256);
+      }
+    }
+  } else {
+    rotated_rows<T>(p, t0, r.ctx + first, CH, n, h, hk, ql, kl, LD, tid);
+    for (int u = tid; u < CH * vdim; u += 256) {
+      const int m = u / vdim, c = u - m * vdim;
+      vl[m * LDV + c] = m < n ? (float)static_cast<const T*>(p.proj)[(int64_t)(t0 + m) * p.ldp + cv + c] : 0.f;
+    }
+    __syncthreads();
+    const float ld = p.log2_decay[h];
+    {
+      const int i = tid >> 4, j = tid & 15;
+      float b = 0.f;
+      if (j <= i && i < n) {
+        for (int c = 0; c < dim; c += 4) {
+          const f32x4 qi = *reinterpret_cast<const f32x4*>(ql + i * LD + c), kj = *reinterpret_cast<const f32x4*>(kl + j * LD + c);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) b = fmaf(qi[x], kj[x], b);
+        }
+        b *= exp2f(ld * (float)(i - j));
+      }
+      out[sc.b + i * CH + j] = b;
+    }
+    for (int u = tid; u < CH * dim; u += 256) {
+      const int i = u / dim, c = u - i * dim;
+      out[sc.q + u] = ql[i * LD + c] * exp2f(ld * (float)(i + 1));
+      const int ck2 = u / CH, ik = u % CH;
+      out[sc.k + u] = kl[ik * LD + ck2] * exp2f(ld * (float)max(n - 1 - ik, 0));
+    }
+    for (int u = tid; u < CH * vdim; u += 256) out[sc.u + u] = vl[(u % CH) * LDV + u / CH];
+    for (int c = tid; c < dim; c += 256) out[sc.d + c] = exp2f(ld * (float)n);
+  }
+}
+
+__device__ __forceinline__ void mma4(f32x4& acc, const f32x4& a, const f32x4& b) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], acc, 0, 0, 0);
+}
+
+// NT: 16-row tiles of the state.  One wave: 16 value columns of one (entry, head)
+template <int KIND, int NT>
+__global__ __launch_bounds__(256, 1) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), kc = lane >> 4, r16 = lane & 15;
+  const int waves = blockDim.x >> 6, per = (p.vdim / 16 + waves - 1) / waves;
+  const int h = blockIdx.x / per, col0 = ((int)(blockIdx.x % per) * waves + wave) * 16, e = blockIdx.y;
+  if (col0 >= p.vdim) return;
+  const Portion r = portion(s, e);
+  if (r.len <= 0) return;
+  constexpr int dim = NT * 16;
+  const Scratch sc(KIND, dim, p.vdim);
+  const int nch = (r.len + CH - 1) / CH;
+  const int64_t step = (int64_t)p.heads * sc.size;
+  const float* in = p.scratch + ((int64_t)s.chunk_start[e] * p.heads + h) * sc.size;
+  float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim) * p.vdim + col0 + r16;
+  f32x4 S[NT], w[KIND == VMI_HY_DELTA ? NT : 1], q[NT], k[NT];
+#pragma unroll
+  for (int ct = 0; ct < NT; ++ct)
+#pragma unroll
+    for (int x = 0; x < 4; ++x) S[ct][x] = r.ctx > 0 ? st[(int64_t)(16 * ct + 4 * kc + x) * p.vdim] : 0.f;
+
+  const int row = r16 * dim + 4 * kc, col = r16 * CH + 4 * kc;
+  auto load_w = [&](const float* c) {
+    if constexpr (KIND == VMI_HY_DELTA) {
+#pragma unroll
+      for (int ct = 0; ct < NT; ++ct) w[ct] = *reinterpret_cast<const f32x4*>(c + sc.w + row + 16 * ct);
+    }
+  };
+  auto load_q = [&](const float* c) {
+#pragma unroll
+    for (int ct = 0; ct < NT; ++ct) q[ct] = *reinterpret_cast<const f32x4*>(c + sc.q + row + 16 * ct);
+  };
+  auto load_k = [&](const float* c) {
+#pragma unroll
+    for (int ct = 0; ct < NT; ++ct) k[ct] = *reinterpret_cast<const f32x4*>(c + sc.k + 16 * ct * CH + col);
+  };
+  f32x4 u0, b;
+  auto load_u = [&](const float* c) {
+    u0 = *reinterpret_cast<const f32x4*>(c + sc.u + col0 * CH + col);
+    b = *reinterpret_cast<const f32x4*>(c + sc.b + col);
+  };
+  load_u(in);
+  load_w(in);
+  load_q(in);
+  load_k(in);
+  float* o = p.o + (int64_t)r.qs * p.heads * p.vdim + (int64_t)h * p.vdim + col0 + r16;
+  for (int c = 0; c < nch; ++c) {
+    // every operand is asked for again, from the next chunk, as soon as its last use has been issued (the last chunk: from itself)
+    const float* next = c + 1 < nch ? in + step : in;
+    f32x4 u = u0, a0 = f32x4{0.f, 0.f, 0.f, 0.f}, a1 = a0;
+    const f32x4 bb = b;
+    load_u(next);
+    if constexpr (KIND == VMI_HY_DELTA) {
+#pragma unroll
+      for (int ct = 0; ct < NT; ++ct) mma4(ct & 1 ? a1 : a0, w[ct], S[ct]);
+      u -= a0 + a1;
+      load_w(next);
+    }
+    f32x4 o0 = f32x4{0.f, 0.f, 0.f, 0.f}, o1 = o0;
+#pragma unroll
+    for (int ct = 0; ct < NT; ++ct) mma4(ct & 1 ? o1 : o0, q[ct], S[ct]);
+    load_q(next);
+    mma4(o0, bb, u);
+#pragma unroll
+    for (int ct = 0; ct < NT; ++ct) {
+      const f32x4 d = *reinterpret_cast<const f32x4*>(in + sc.d + 16 * ct + 4 * kc);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) S[ct][x] *= d[x];
+      mma4(S[ct], k[ct], u);
+    }
+    load_k(next);
+    o0 += o1;
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const int m = c * CH + 4 * kc + x;
+      if (m < r.len) o[(int64_t)m * p.heads * p.vdim] = o0[x];
+    }
+    in = next;
+  }
+#pragma unroll
+  for (int ct = 0; ct < NT; ++ct)
+#pragma unroll
+    for (int x = 0; x < 4; ++x) st[(int64_t)(16 * ct + 4 * kc + x) * p.vdim] = S[ct][x];
+}
+
+// the columns of a state that one workgroup of the single-token step takes, and the rows a thread then holds
+inline int step_slice(int dim, int vdim) {
+  const int most = dim <= 128 ? 128 : dim <= 256 ? 64 : 32;
+  return vdim <= most ? vdim : most;
+}
+inline int step_rows(int dim, int slice) {
+  const int groups = 256 / (slice / 4);
+  return (dim + groups - 1) / groups;
+}
+
+// one token of one (entry, head), a slice of the value columns.  RPT: state rows a thread holds (at most)
+template <typename T, int KIND, int RPT>
+__global__ __launch_bounds__(256) void state_step_kernel(const vmi_hy_state_args p, const vmi_hy_step s, const int slice) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int dim = p.dim, tid = threadIdx.x, h = blockIdx.x, e = blockIdx.y, c0 = (int)blockIdx.z * slice;
+  const int width = min(slice, p.vdim - c0), quads = slice >> 2, groups = 256 / quads;
+  float* ql = lds;               // [dim]
+  float* kl = ql + dim;          // [dim]
+  float* gl = kl + dim;          // [dim]
+  float* vl = gl + dim;          // [slice]
+  float* ul = vl + slice;        // [slice]
+  float* red = ul + slice;       // [groups][slice]
+  float* sums = red + 1024;      // [8]
+  const Portion r = portion(s, e);
+  if (r.len <= 0) return;
+  const int t = r.qs, hk = h / (p.heads / p.kv_heads), C = 2 * p.kv_heads * dim + p.heads * p.vdim;
+  const int cq = hk * dim, ck = (p.kv_heads + hk) * dim, cv = 2 * p.kv_heads * dim + h * p.vdim + c0;
+  const int quad = tid % quads, grp = tid / quads;
+  const bool mine = grp < groups && quad * 4 < width;
+  float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim) * p.vdim + c0 + quad * 4;
+  f32x4 S[RPT];
+  const bool have = r.ctx > 0;
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int row = grp + i * groups;
+    S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (have && mine && row < dim) S[i] = *reinterpret_cast<const f32x4*>(st + (int64_t)row * p.vdim);
+  }
+  float beta = 1.f;
+  if constexpr (KIND == VMI_HY_DELTA) {
+    const int ud = dim >> 3, uv = width >> 3;
+    for (int u = tid; u < 2 * ud + uv; u += 256) {
+      float* dst;
+      int ch;
+      if (u < ud) dst = ql + u * 8, ch = cq + u * 8;
+      else if (u < 2 * ud) dst = kl + (u - ud) * 8, ch = ck + (u - ud) * 8;
+      else dst = vl + (u - 2 * ud) * 8, ch = cv + (u - 2 * ud) * 8;
+      const f32x8 v = p.taps == 4 ? conv_silu8<T, 4>(p, r, C, t, ch) : conv_silu8<T, 0>(p, r, C, t, ch);
+      *reinterpret_cast<f32x4*>(dst) = f32x4{v[0], v[1], v[2], v[3]};
+      *reinterpret_cast<f32x4*>(dst + 4) = f32x4{v[4], v[5], v[6], v[7]};
+    }
+    const float rate = p.rate[h];
+    for (int c = tid; c < dim; c += 256)
+      gl[c] = exp_hw(-rate * softplus((float)static_cast<const T*>(p.z)[(int64_t)t * p.ldz + (int64_t)h * dim + c] + p.dt_bias[(int64_t)h * dim + c]));
+    beta = sigmoid((float)static_cast<const T*>(p.beta)[(int64_t)t * p.ldp + h]);
+    if (p.taps > 1) {
+      write_tail<T>(p, r, C, cv, width, tid, 256);
+      if (blockIdx.z == 0 && h == hk * (p.heads / p.kv_heads)) {
+        write_tail<T>(p, r, C, cq, dim, tid, 256);
+        write_tail<T>(p, r, C, ck, dim, tid, 256);
+      }
+    }
+    __syncthreads();
+    if (tid < 128) {   // wave 0: q, wave 1: k
+      float* x = tid < 64 ? ql : kl;
+      float a = 0.f;
+      for (int c = tid & 63; c < dim; c += 64) a = fmaf(x[c], x[c], a);
+      a = wave_sum(a) + 1e-6f;
+      a = 1.f / sqrtf(tid < 64 ? a * (float)p.dim_n : a);
+      for (int c = tid & 63; c < dim; c += 64) x[c] *= a;
+    }
+  } else {
+    rotated_rows<T>(p, t, r.ctx, 1, 1, h, hk, ql, kl, dim, tid);
+    for (int c = tid; c < width; c += 256) vl[c] = (float)static_cast<const T*>(p.proj)[(int64_t)t * p.ldp + cv + c];
+    beta = p.decay[h];   // (the one decay of the head)
+  }
+  __syncthreads();
+  auto gather = [&](const f32x4& part) {   // sums over the row groups, into red[0]'s place of every column; returns column tid's
+    if (mine) *reinterpret_cast<f32x4*>(red + grp * slice + quad * 4) = part;
+    __syncthreads();
+    float v = 0.f;
+    if (tid < width)
+      for (int g = 0; g < groups; ++g) v += red[g * slice + tid];
+    return v;
+  };
+  f32x4 part = f32x4{0.f, 0.f, 0.f, 0.f}, u;
+  if constexpr (KIND == VMI_HY_DELTA) {
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+      const int row = grp + i * groups;
+      if (mine && row < dim) {
+        S[i] = S[i] * gl[row];
+        const float k = kl[row];
+#pragma unroll
+        for (int x = 0; x < 4; ++x) part[x] = fmaf(S[i][x], k, part[x]);
+      }
+    }
+    const float held = gather(part);
+    if (tid < width) ul[tid] = beta * (vl[tid] - held);
+    __syncthreads();
+    if (mine) u = *reinterpret_cast<const f32x4*>(ul + quad * 4);
+  } else {
+    if (mine) u = *reinterpret_cast<const f32x4*>(vl + quad * 4);
+  }
+  part = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int row = grp + i * groups;
+    if (mine && row < dim) {
+      const float k = kl[row], q = ql[row];
+      if constexpr (KIND == VMI_HY_RETENTION) S[i] = S[i] * beta;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        S[i][x] = fmaf(k, u[x], S[i][x]);
+        part[x] = fmaf(S[i][x], q, part[x]);
+      }
+      *reinterpret_cast<f32x4*>(st + (int64_t)row * p.vdim) = S[i];
+    }
+  }
+  const float o = gather(part);
+  if (!p.out) {
+    if (tid < width) p.o[((int64_t)t * p.heads + h) * p.vdim + c0 + tid] = o;
+    return;
+  }
+  const float ss = wave_sum(tid < width ? o * o : 0.f);   // (this workgroup holds the whole head, at most 128 columns of it)
+  if ((tid & 63) == 0) sums[tid >> 6] = ss;
+  __syncthreads();
+  if (tid < width) {
+    const float z = (float)static_cast<const T*>(p.gate)[(int64_t)t * p.ldg + (int64_t)h * p.vdim + tid];
+    const float y = o / sqrtf((sums[0] + sums[1] + sums[2] + sums[3]) / (float)p.vdim_n + p.eps) * (p.norm_w ? p.norm_w[tid] : 1.f);
+    static_cast<T*>(p.out)[(int64_t)t * p.ldo + (int64_t)h * p.vdim + tid] = (T)(y * (p.act == VMI_HY_ACT_SILU ? silu(z) : sigmoid(z)));
+  }
+}
+
+template <typename T, int KIND>
+static int run_step(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
+  const int slice = step_slice(p.dim, p.vdim), rows = step_rows(p.dim, slice);
+  const dim3 grid(p.heads, s.B, (p.vdim + slice - 1) / slice);
+  const size_t lds = (size_t)(3 * p.dim + 2 * slice + 1024 + 8) * sizeof(float);
+  if (rows <= 4) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 4>), grid, dim3(256), lds, st, p, s, slice);
+  else if (rows <= 8) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 8>), grid, dim3(256), lds, st, p, s, slice);
+  else if (rows <= 16) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 16>), grid, dim3(256), lds, st, p, s, slice);
+  else if (rows <= 32) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 32>), grid, dim3(256), lds, st, p, s, slice);
+  else return fail(VMI_HY_E_SHAPE, "vmi_hy_state", "heads this large are not built");
+  return launched("vmi_hy_state");
+}
+
+template <int KIND, int NT>
+static void launch_scan(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
+  const int waves = p.vdim >= 64 ? 4 : p.vdim / 16;
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT>), dim3(p.heads * ((p.vdim / 16 + waves - 1) / waves), s.B), dim3(64 * waves),
+                     0, st, p, s);
+}
+
+template <typename T, int KIND>
+static int run_chunks(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
+  auto* fn = KIND == VMI_HY_DELTA && p.taps == 4 ? state_prep_kernel<T, KIND, 4> : state_prep_kernel<T, KIND, 0>;
+  const size_t lds = prep_lds(KIND, p.dim, p.vdim);
+  if (int rc = allow_lds(fn, lds, "vmi_hy_state")) return rc;
+  hipLaunchKernelGGL(fn, dim3(s.n_chunks, p.heads), dim3(256), lds, st, p, s);
+  switch (p.dim) {
+    case 32: launch_scan<KIND, 2>(p, s, st); break;
+    case 64: launch_scan<KIND, 4>(p, s, st); break;
+    case 96: launch_scan<KIND, 6>(p, s, st); break;
+    case 128: launch_scan<KIND, 8>(p, s, st); break;
+    case 192: launch_scan<KIND, 12>(p, s, st); break;
+    case 256: launch_scan<KIND, 16>(p, s, st); break;
+    case 512: launch_scan<KIND, 32>(p, s, st); break;
+    default: return fail(VMI_HY_E_SHAPE, "vmi_hy_state", "key dimensions of 32, 64, 96, 128, 192, 256 and 512 are built");
+  }
+  return launched("vmi_hy_state");
+}
+
+template <typename T>
+static int run_state(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
+  if (p.kind == VMI_HY_DELTA) return p.single ? run_step<T, VMI_HY_DELTA>(p, s, st) : run_chunks<T, VMI_HY_DELTA>(p, s, st);
+  return p.single ? run_step<T, VMI_HY_RETENTION>(p, s, st) : run_chunks<T, VMI_HY_RETENTION>(p, s, st);
+}
+
+}  // namespace vmi_hybrid
+
+using namespace vmi_hybrid;
+
+extern "C" {
+
+int64_t vmi_hy_state_scratch(int32_t kind, int32_t dim, int32_t vdim) { return Scratch(kind, dim, vdim).size; }
+
+int32_t vmi_hy_state_fuses(int32_t dim, int32_t vdim) { return step_slice(dim, vdim) == vdim; }
+
+int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream) {
+  static const char* who = "vmi_hy_state";
+  if (!a || !s || !a->proj || !a->state || (!a->o && !a->out) || !s->q_start || !s->q_len || !s->ctx || !s->state_slot || !s->flip ||
+      s->T <= 0 || s->B <= 0 || a->heads <= 0 || a->kv_heads <= 0 || a->dim <= 0 || a->vdim <= 0 || a->dim_n <= 0 || a->dim_n > a->dim ||
+      a->vdim_n <= 0 || a->vdim_n > a->vdim || a->heads % a->kv_heads || a->kind < 0 || a->kind > 1 || a->dtype < 0 || a->dtype > 1)
+    return fail(VMI_HY_E_ARG, who, "null pointer or a size out of range");
+  if (a->kind == VMI_HY_DELTA && (!a->beta || !a->z || !a->conv_w || !a->rate || !a->dt_bias || a->taps < 1 || a->taps > MAX_TAPS ||
+                                  (a->taps > 1 && !a->tail)))
+    return fail(VMI_HY_E_ARG, who, "the delta rule needs its gates and a convolution of 1 to 16 taps");
+  if (a->kind == VMI_HY_RETENTION && (!a->freq || !a->decay || !a->log2_decay || a->rot_n < 0 || a->rot_n > a->dim || (a->rot_n & 1)))
+    return fail(VMI_HY_E_ARG, who, "retention needs decays and an even number of rotated dimensions");
+  if (!a->single && (!a->scratch || !a->o || !s->chunks || !s->chunk_start || s->n_chunks <= 0))
+    return fail(VMI_HY_E_ARG, who, "portions need chunks and scratch");
+  if (a->out && (!a->single || !a->gate || !vmi_hy_state_fuses(a->dim, a->vdim)))
+    return fail(VMI_HY_E_ARG, who, "only a step of single tokens with whole heads writes finished rows");
+  if ((a->dim & 31) || (a->vdim & 31) || (a->ldp & 7) || ((uintptr_t)a->proj & 15) || a->dim > 512 || s->B > 65535 || a->heads > 65535)
+    return fail(VMI_HY_E_SHAPE, who, "needs sizes that are multiples of 32, key dimensions up to 512 and aligned rows");
+  DeviceScope dev(a->device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipStream_t st = static_cast<hipStream_t>(stream);
+  return a->dtype == VMI_HY_BF16 ? run_state<b16>(*a, *s, st) : run_state<float>(*a, *s, st);
+}
+
+}  // extern "C"

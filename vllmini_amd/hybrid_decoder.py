@@ -1,4 +1,4 @@
-"""A decoder over hybrid_layers: recurrent blocks and latent attention, in any order, some of them run several times.
+"""A decoder over hybrid_layers: recurrences, linear and softmax attention, in any order, some of them run several times.
 
 The counterpart of GPT2PagedDecoder for models that are described by a list of layer runs (`HybridModel`): same pool
 (kv_pool.PagedKVPool with row pages and state slots), same scheduler (prefill / prefill_batch / decode / greedy), one forward
@@ -11,21 +11,22 @@ Every layer RUN has its own cache / state: a layer inside a loop keeps one per p
 from __future__ import annotations
 
 import dataclasses
-from typing import Dict, List, Optional, Sequence, Tuple, Union
+from typing import Dict, List, Optional, Sequence, Union
 
 import numpy as np
 import torch
 
 from . import hybrid_ops as ops
-from .hybrid_layers import ClampedGLU, ConcatProjection, Head, LatentAttention, Residual, RGLRU
+from .hybrid_layers import AttentionPlan, ClampedGLU, ConcatProjection, Head, LatentAttention, ParallelBlock, QueryTiling, Residual, RGLRU
 from .kv_pool import PagedKVPool
 
 
 @dataclasses.dataclass
 class LayerRun:
-    """One pass through one layer: an input projection in front of it (or None), its mixer, its feed-forward (or None)."""
-    mixer: Union[LatentAttention, RGLRU]
-    mlp: Optional[ClampedGLU]
+    """One pass through one layer: an input projection in front of it (or None), its mixer, its feed-forward (or None; a
+    ParallelBlock brings its own)."""
+    mixer: Union[LatentAttention, RGLRU, ParallelBlock]
+    mlp: Optional[ClampedGLU] = None
     enter: Optional[ConcatProjection] = None
 
 
@@ -46,18 +47,10 @@ class HybridModel:
         the longest a sequence may get (default: it may take the whole pool)."""
         blocks = max(1, max_tokens // page_size)
         per_seq = blocks if max_length is None else -(-max_length // page_size)
-        rows = [r.mixer.page_row() for r in self.runs if isinstance(r.mixer, LatentAttention)]
-        state = [s for r in self.runs if isinstance(r.mixer, RGLRU) for s in r.mixer.state_shapes()]
+        rows = [n for r in self.runs for n in r.mixer.page_rows()]
+        state = [s for r in self.runs for s in r.mixer.state_shapes()]
         return PagedKVPool(blocks, 1, max(rows, default=1), page_size, per_seq + 1, 1, device=self.device, max_seqs=max_seqs,
                            page_rows=rows, page_dtype=self.dtype, state=state, state_slots=max_seqs, **kw)
-
-
-@dataclasses.dataclass
-class AttentionPlan:
-    """How the query rows of a step are dealt to workgroups, for layers of one (heads, row length)."""
-    tiles: torch.Tensor
-    row_tiles: int
-    splits: int
 
 
 class HybridDecoder:
@@ -73,23 +66,25 @@ class HybridDecoder:
         ops.load()
         self.pad_batch_to = int(pad_batch_to)
         self.paged_prefill = True                      # (prefill_batch is the one prefill there is)
-        self._slots: List[tuple] = []                  # per run: its cache tensor | its (state, tail)
+        self._slots: List[tuple] = []                  # per run: its cache tensors, then its states
         ip = iter(pool.row_pages)
         st = iter(pool.state)
         for r in model.runs:
-            self._slots.append((next(ip),) if isinstance(r.mixer, LatentAttention) else (next(st), next(st)))
-        self._kinds = sorted({(r.mixer.heads, r.mixer.row) for r in model.runs if isinstance(r.mixer, LatentAttention)})
+            self._slots.append((*(next(ip) for _ in r.mixer.page_rows()), *(next(st) for _ in r.mixer.state_shapes())))
+        self._kinds: List[QueryTiling] = sorted({r.mixer.tiling() for r in model.runs} - {None})
         self.tap: Optional[List[torch.Tensor]] = None  # set to a list: the residual stream after every layer run is appended to it
         self._stage: List[list] = []                   # pinned staging buffers: [tensor, event]
         self._stage_i = 0
         self._sets: Dict[tuple, dict] = {}             # captured decode steps
 
     # ---- the step's layout -----------------------------------------------------------------------------------------------
-    def _split_of(self, n_tiles: int, row_tiles: int, heads: int, row: int, max_keys: int, T: int) -> int:
+    def _split_of(self, n_tiles: int, row_tiles: int, kind: QueryTiling, max_keys: int, T: int) -> int:
+        n_tiles *= kind.sets
         if n_tiles > 128:
             return 1
+        max_keys = min(max_keys, kind.chunk) if kind.chunk else max_keys
         want = min(self.FILL_WORKGROUPS[row_tiles] // max(n_tiles, 1), -(-max_keys // self.KEY_TILE))
-        fit = (256 << 20) // max(1, T * heads * (row + 2) * 4)             # (bytes of the partial results)
+        fit = (256 << 20) // max(1, T * kind.rep * kind.sets * (kind.width + 2) * 4)       # (bytes of the partial results)
         n = 1
         while 2 * n <= min(want, fit, 128):
             n *= 2
@@ -120,21 +115,27 @@ class HybridDecoder:
         sec["table"] = tab.reshape(-1)
         put("rows", max(len(rows), 1), rows, 0)
         plans = []
-        for heads, row in self._kinds:
-            longest = int(counts.max()) * heads
-            rt = ops.latent_row_tiles(row, 4 if longest > 32 else 2 if longest > 16 else 1, self.model.dtype)
-            per = -(-(counts * heads) // (16 * rt))
+        for kind in self._kinds:
+            rep, longest = kind.rep, int(counts.max()) * kind.rep
+            rt = kind.row_tiles(4 if longest > 32 else 2 if longest > 16 else 1, self.model.dtype)
+            per = -(-(counts * rep) // (16 * rt))
             ent = np.repeat(np.arange(b), per)
             first = (np.arange(int(per.sum())) - np.repeat(np.cumsum(per) - per, per)) * 16 * rt
             if b > 1 or len(first) > 1:       # longest first: the tail of the launch is short tiles
-                keys = a["ctx"][ent] + (first + 16 * rt - 1) // heads
-                order = np.argsort(-keys, kind="stable")
+                keys = a["ctx"][ent] + (first + 16 * rt - 1) // rep
+                order = np.argsort(-(keys % kind.chunk if kind.chunk else keys), kind="stable")
                 ent, first = ent[order], first[order]
-            nt = len(ent) + (B - b) * (-(-heads // (16 * rt)))
+            nt = len(ent) + (B - b) * (-(-rep // (16 * rt)))
             t = np.full((nt, 2), -1, dtype=np.int32)
             t[: len(ent), 0], t[: len(ent), 1] = ent, first
             sec[f"tiles{len(plans)}"] = t.reshape(-1)
-            plans.append((rt, self._split_of(nt, rt, heads, row, max_keys, T), nt))
+            plans.append((rt, self._split_of(nt, rt, kind, max_keys, T), nt))
+        if (counts > 1).any():                # runs of rows for the linear-attention layers
+            per = -(-counts // ops.CHUNK_ROWS)
+            at = np.cumsum(per) - per
+            put("chunk_start", B, at, 0)
+            ent = np.repeat(np.arange(b), per)
+            sec["chunks"] = np.stack([ent, (np.arange(int(per.sum())) - at[ent]) * ops.CHUNK_ROWS], axis=1).astype(np.int32).reshape(-1)
         offs, total = {}, 0
         for name, v in sec.items():
             offs[name] = (total, len(v))
@@ -167,6 +168,8 @@ class HybridDecoder:
     def _views(self, dev: torch.Tensor, offs, B: int, table_ld: int, plans):
         v = {k: dev[o: o + n] for k, (o, n) in offs.items()}
         v["table"] = v["table"].view(B, table_ld)
+        if "chunks" in v:
+            v["chunks"] = v["chunks"].view(-1, 2)
         plan = {kind: AttentionPlan(v[f"tiles{i}"].view(nt, 2), rt, sp) for i, (kind, (rt, sp, nt)) in enumerate(zip(self._kinds, plans))}
         return v, plan
 
@@ -179,10 +182,7 @@ class HybridDecoder:
         for r, held in zip(m.runs, self._slots):
             if r.enter is not None:
                 r.enter.run(res, x0)
-            if isinstance(r.mixer, LatentAttention):
-                r.mixer.run(res, step, plans[(r.mixer.heads, r.mixer.row)], held[0])
-            else:
-                r.mixer.run(res, step, held[0], held[1])
+            r.mixer.run(res, step, plans, held)
             if r.mlp is not None:
                 r.mlp.run(res, step)
             if self.tap is not None:

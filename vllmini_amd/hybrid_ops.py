@@ -1,33 +1,40 @@
-"""Operators of libvmi_hybrid.so (include/vmi_hybrid.h): what decoders with recurrent blocks and latent attention are made of.
+"""Operators of libvmi_hybrid.so (include/vmi_hybrid.h): what decoders that mix recurrences, linear and softmax attention are made of.
 
 Thin ctypes wrappers over csrc/hybrid_*.hip that check operands on the host (devices, dtypes, shapes, strides — a kernel never
 sees sizes that do not fit its buffers) and launch on torch's current stream.  There is no torch fallback: a missing library or
 an unsupported shape raises.  Two element types: torch.bfloat16 (what models are served in) and torch.float32 (every product in
 full 32 bits).
 
-    linear            y = epilogue(prologue(x) W^T): layer norm / concatenation in front, residual add / gated unit / head gate behind
-    embed, add_norm, glu, argmax
+    linear            y = epilogue(prologue(x) W^T): norm / concatenation in front, residual add / gated unit / head gate behind
+    embed, add_norm, merge, glu, argmax
     rglru             causal convolution + block-diagonal gates + gated linear recurrence + gelu(y) product
     latent_prep       RMS norm of the latent, rotary parts, cache write
     latent_attention  softmax attention in the latent space over the paged cache
+    linear_state      linear attention with a matrix state per head: retention, the gated delta rule
+    kv_prep           RMS norms of q and k, cache write
+    attention         grouped-query softmax attention over the paged cache: chunks, bias by distance, sink, output gate
 
-StepLayout describes the tokens of one step to the last three.
+StepLayout describes the tokens of one step to the latter ones.
 """
 from __future__ import annotations
 
 import ctypes
 import os
 import threading
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 
 from . import build as _build
 
-ABI_VERSION = 1
+ABI_VERSION = 2
 DTYPES = {torch.bfloat16: 0, torch.float32: 1}
 X_ROWS, X_NORM, X_CONCAT = 0, 1, 2
-E_STORE, E_RESIDUAL, E_FLOAT, E_GLU, E_GATED = 0, 1, 2, 3, 4
+E_STORE, E_RESIDUAL, E_FLOAT, E_GLU, E_GATED, E_STORE_GLU = 0, 1, 2, 3, 4, 5
+RETENTION, DELTA = 0, 1
+ACTS = {"sigmoid": 0, "silu": 1}
+CHUNK_ROWS = 16     # rows of a chunk of the linear-attention kernels
+STATE_DIMS = (32, 64, 96, 128, 192, 256, 512)       # key dimensions they are built for
 
 _vp, _i32, _i64, _f32 = ctypes.c_void_p, ctypes.c_int32, ctypes.c_int64, ctypes.c_float
 
@@ -36,22 +43,40 @@ def _struct(name, fields):
     return type(name, (ctypes.Structure,), {"_fields_": [(n, t) for t, names in fields for n in names.split()]})
 
 
-LinearArgs = _struct("LinearArgs", [(_vp, "x x2 rows norm_w w bias gate y"), (_i64, "ldx ldy ldg x_gstride y_gstride"),
-                                    (_i32, "M N K groups norm_n n_out"), (_f32, "eps scale"), (_i32, "x_kind epilogue dtype device")])
-StepArgs = _struct("StepArgs", [(_vp, "tok_seq tok_pos tok_slot q_start q_len ctx state_slot flip table"),
-                                (_i32, "T B table_ld page_size")])
+LinearArgs = _struct("LinearArgs", [(_vp, "x x2 rows norm_w w bias gate y y2"), (_i64, "ldx ldy ldg ldy2 x_gstride y_gstride"),
+                                    (_i32, "M N K groups norm_n n_out n_split rms"), (_f32, "eps scale glu_alpha glu_up"),
+                                    (_i32, "x_kind epilogue dtype device")])
+StepArgs = _struct("StepArgs", [(_vp, "tok_seq tok_pos tok_slot q_start q_len ctx state_slot flip table chunks chunk_start"),
+                                (_i32, "T B table_ld page_size n_chunks")])
 RglruArgs = _struct("RglruArgs", [(_vp, "yx out conv_w conv_b gates gate_b decay state tail scratch carry"), (_i64, "ldx ldo"),
                                   (_i32, "width blocks taps single spans dtype device")])
 PrepArgs = _struct("PrepArgs", [(_vp, "proj q cache norm_w freq"), (_i64, "ldp"), (_i32, "heads dim rot rank rot_n rank_n"),
                                 (_f32, "eps"), (_i32, "dtype device")])
 AttentionArgs = _struct("AttentionArgs", [(_vp, "q cache out tiles partial"), (_i32, "heads rank rot n_tiles row_tiles splits"),
                                           (_f32, "scale"), (_i32, "dtype device")])
+StateArgs = _struct("StateArgs", [(_vp, "proj beta z conv_w rate dt_bias decay log2_decay freq state tail o scratch out gate norm_w"),
+                                  (_i64, "ldp ldz ldo ldg"),
+                                  (_i32, "heads kv_heads dim vdim dim_n vdim_n taps rot_n kind single act"), (_f32, "eps"),
+                                  (_i32, "dtype device")])
+KvPrepArgs = _struct("KvPrepArgs", [(_vp, "proj q cache"), (_i64, "ldp"), (_i32, "heads kv_heads dim vdim dim_n"), (_f32, "eps"),
+                                    (_i32, "dtype device")])
+GqaArgs = _struct("GqaArgs", [(_vp, "q cache out bias sink gate tiles partial"), (_i64, "ldo ldg"),
+                              (_i32, "heads kv_heads dim vdim bias_n chunk n_tiles row_tiles splits"), (_f32, "scale"),
+                              (_i32, "dtype device")])
 
 SIGNATURES = {
     "vmi_hy_linear": (ctypes.c_int, [ctypes.POINTER(LinearArgs), _vp]),
     "vmi_hy_embed": (ctypes.c_int, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
-    "vmi_hy_add_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32, _vp]),
-    "vmi_hy_glu": (ctypes.c_int, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_add_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32, _i32, _vp]),
+    "vmi_hy_merge": (ctypes.c_int, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_glu": (ctypes.c_int, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _f32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_state_scratch": (_i64, [_i32, _i32, _i32]),
+    "vmi_hy_state_fuses": (_i32, [_i32, _i32]),
+    "vmi_hy_state": (ctypes.c_int, [ctypes.POINTER(StateArgs), ctypes.POINTER(StepArgs), _vp]),
+    "vmi_hy_head_norm_gate": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _i32, _i32, _vp]),
+    "vmi_hy_kv_prep": (ctypes.c_int, [ctypes.POINTER(KvPrepArgs), ctypes.POINTER(StepArgs), _vp]),
+    "vmi_hy_attention_row_tiles": (_i32, [_i32, _i32, _i32, _i32]),
+    "vmi_hy_attention": (ctypes.c_int, [ctypes.POINTER(GqaArgs), ctypes.POINTER(StepArgs), _vp]),
     "vmi_hy_concat": (ctypes.c_int, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _vp]),
     "vmi_hy_argmax": (ctypes.c_int, [_vp, _i64, _i32, _i32, _vp, _i32, _vp]),
     "vmi_hy_rglru": (ctypes.c_int, [ctypes.POINTER(RglruArgs), ctypes.POINTER(StepArgs), _vp]),
@@ -119,6 +144,33 @@ def pad32(n: int) -> int:
     return (n + 31) // 32 * 32
 
 
+def state_dim(n: int) -> int:
+    """The key dimension that the linear-attention kernels are built for and that holds n."""
+    for d in STATE_DIMS:
+        if n <= d:
+            return d
+    raise ValueError(f"key dimensions beyond {STATE_DIMS[-1]} are not built")
+
+
+class GatedUnit(NamedTuple):
+    """g' sigmoid(alpha g') (u' + up) with g' = min(g, limit), u' = u clamped to +- limit."""
+    limit: float
+    alpha: float
+    up: float
+
+    @classmethod
+    def clamped(cls, limit: float) -> "GatedUnit":
+        return cls(float(limit), 1.702, 1.0)
+
+
+SILU_UNIT = GatedUnit(float("inf"), 1.0, 0.0)      # silu(g) u
+NormArgs = Tuple       # weight, true columns, eps, and whether it is an RMS norm (default: a layer norm)
+
+
+def _rms(norm: Optional[NormArgs]) -> int:
+    return int(norm is not None and len(norm) > 3 and norm[3])
+
+
 class MatrixTiles:
     """Linear weights [N, K] (or a group of them, [G, N, K]) as the tiles the kernels stream, zero-padded to N % 32 == K % 32 == 0:
     tiles[g][s][t][kc * 16 + r][e] = w[g][16 s + r][32 t + 8 kc + e].  `dense=True` keeps the padded [N, K] as well (steps of many
@@ -134,21 +186,23 @@ class MatrixTiles:
         self.dense = p[0].contiguous() if dense and G == 1 else None
 
 
-def linear(x: torch.Tensor, w: MatrixTiles, *, norm: Optional[Tuple[torch.Tensor, int, float]] = None, x2: Optional[torch.Tensor] = None,
+def linear(x: torch.Tensor, w: MatrixTiles, *, norm: Optional[NormArgs] = None, x2: Optional[torch.Tensor] = None,
            rows: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
-           residual: bool = False, float_out: Optional[Tuple[int, float]] = None, glu_limit: Optional[float] = None,
-           gate: Optional[torch.Tensor] = None, x_gstride: int = 0, y_gstride: int = 0) -> torch.Tensor:
+           residual: bool = False, float_out: Optional[Tuple[int, float]] = None, glu: Optional[GatedUnit] = None,
+           glu_from: int = -1, glu_out: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, x_gstride: int = 0,
+           y_gstride: int = 0) -> torch.Tensor:
     """One linear layer over the rows of x.
-        input     x [M, K] of the element type | norm=(weight, n, eps): x float32, layer norm over its first n columns, optionally
+        input     x [M, K] of the element type | norm=(weight, n, eps, rms): x float32, normed over its first n columns, optionally
                   of `rows` only | x2: x and x2 float32 side by side
-        output    element type (+ bias) | residual=True: out (float32) += | float_out=(columns, scale): float32 | glu_limit: the
-                  clamped gated unit of interleaved (gate, up) columns | gate [M, groups ...]: times sigmoid of the group's column
+        output    element type (+ bias) | residual=True: out (float32) += | float_out=(columns, scale): float32 | glu: the
+                  gated unit of interleaved (gate, up) columns | gate [M, groups ...]: times sigmoid of the group's column |
+                  glu and glu_from=n, glu_out: columns below n as they are, the gated unit of the others into glu_out
         groups    group g reads x at column g * x_gstride, writes out at column g * y_gstride"""
     lib = load()
     device, stream = _on(x)
     T = w.tiles.dtype
     kind = X_NORM if norm is not None else X_CONCAT if x2 is not None else X_ROWS
-    epi = E_RESIDUAL if residual else E_FLOAT if float_out else E_GLU if glu_limit is not None else E_GATED if gate is not None else E_STORE
+    epi = E_RESIDUAL if residual else E_FLOAT if float_out else (E_GLU if glu_out is None else E_STORE_GLU) if glu is not None else E_GATED if gate is not None else E_STORE
     M = int(rows.numel()) if rows is not None else int(x.shape[0])
     K, N = w.K, w.N
     span = (w.groups - 1) * x_gstride + (K // 2 if kind == X_CONCAT else K)
@@ -165,17 +219,23 @@ def linear(x: torch.Tensor, w: MatrixTiles, *, norm: Optional[Tuple[torch.Tensor
         _need(bias.dtype == torch.float32 and bias.numel() >= N, "hybrid_ops.linear: bias float32 [N]")
     if gate is not None:
         _need(gate.dtype == T and gate.shape[0] == M and gate.stride(1) == 1 and gate.shape[1] >= w.groups, "hybrid_ops.linear: gate")
-    cols = float_out[0] if epi == E_FLOAT else N // 2 if epi == E_GLU else (w.groups - 1) * y_gstride + N
+    if epi == E_STORE_GLU:
+        _need(0 <= glu_from <= N and glu_from % 16 == 0 and glu_out.dtype == T and glu_out.dim() == 2 and glu_out.stride(1) == 1
+              and glu_out.shape[0] == M and glu_out.shape[1] >= (N - glu_from) // 2 and glu_out.device == x.device
+              and w.groups == 1, "hybrid_ops.linear: glu_out")
+    cols = float_out[0] if epi == E_FLOAT else N // 2 if epi == E_GLU else glu_from if epi == E_STORE_GLU else (w.groups - 1) * y_gstride + N
     odt = torch.float32 if epi in (E_RESIDUAL, E_FLOAT) else T
     if out is None:
         out = torch.empty((M, cols), dtype=odt, device=x.device)
     _need(out.dim() == 2 and out.shape[0] == M and out.shape[1] >= cols and out.stride(1) == 1 and out.dtype == odt
           and out.data_ptr() != x.data_ptr(), f"hybrid_ops.linear: out {tuple(out.shape)} {out.dtype} for {M} x {cols}")
     a = LinearArgs(x=x.data_ptr(), x2=_ptr(x2), rows=_ptr(rows), norm_w=norm[0].data_ptr() if norm else None, w=w.tiles.data_ptr(),
-                   bias=_ptr(bias), gate=_ptr(gate), y=out.data_ptr(), ldx=x.stride(0), ldy=out.stride(0),
-                   ldg=gate.stride(0) if gate is not None else 0, x_gstride=x_gstride, y_gstride=y_gstride, M=M, N=N, K=K,
+                   bias=_ptr(bias), gate=_ptr(gate), y=out.data_ptr(), y2=_ptr(glu_out), ldx=x.stride(0), ldy=out.stride(0),
+                   ldg=gate.stride(0) if gate is not None else 0, ldy2=glu_out.stride(0) if glu_out is not None else 0, x_gstride=x_gstride, y_gstride=y_gstride, M=M, N=N, K=K,
                    groups=w.groups, norm_n=norm[1] if norm else 0, n_out=float_out[0] if float_out else 0,
-                   eps=norm[2] if norm else 0.0, scale=float_out[1] if float_out else glu_limit if glu_limit is not None else 1.0,
+                   n_split=max(glu_from, 0), rms=_rms(norm), eps=norm[2] if norm else 0.0,
+                   scale=float_out[1] if float_out else glu.limit if glu is not None else 1.0,
+                   glu_alpha=glu.alpha if glu is not None else 0.0, glu_up=glu.up if glu is not None else 0.0,
                    x_kind=kind, epilogue=epi, dtype=DTYPES[T], device=device)
     _check(lib.vmi_hy_linear(ctypes.byref(a), stream))
     return out
@@ -192,9 +252,8 @@ def embed(ids: torch.Tensor, table: torch.Tensor, width: int, scale: float) -> t
     return x
 
 
-def add_norm(x: torch.Tensor, add: Optional[torch.Tensor], norm: Optional[Tuple[torch.Tensor, int, float]],
-             dtype: torch.dtype) -> Optional[torch.Tensor]:
-    """x += add (if given), then the layer norm of x in `dtype` (if asked for)."""
+def add_norm(x: torch.Tensor, add: Optional[torch.Tensor], norm: Optional[NormArgs], dtype: torch.dtype) -> Optional[torch.Tensor]:
+    """x += add (if given), then the norm of x in `dtype` (if asked for)."""
     device, stream = _on(x)
     T, ld = x.shape
     _need(x.dtype == torch.float32 and x.is_contiguous(), "hybrid_ops.add_norm: x float32, contiguous")
@@ -205,19 +264,38 @@ def add_norm(x: torch.Tensor, add: Optional[torch.Tensor], norm: Optional[Tuple[
         _need(norm[0].dtype == torch.float32 and norm[0].numel() >= ld, "hybrid_ops.add_norm: norm weight float32 [ld]")
         out = torch.empty((T, ld), dtype=dtype, device=x.device)
     _check(load().vmi_hy_add_norm(x.data_ptr(), _ptr(add), add.stride(0) if add is not None else 0, norm[0].data_ptr() if norm else None,
-                                  _ptr(out), T, norm[1] if norm else ld, ld, norm[2] if norm else 0.0, DTYPES[dtype], device, stream))
+                                  _ptr(out), T, norm[1] if norm else ld, ld, norm[2] if norm else 0.0, _rms(norm), DTYPES[dtype],
+                                  device, stream))
     return out
 
 
-def glu(x: torch.Tensor, limit: float) -> torch.Tensor:
-    """The clamped gated unit of interleaved (gate, up) columns: [T, 2 n] -> [T, n]."""
+def merge(x: torch.Tensor, a: torch.Tensor, wa: torch.Tensor, b: torch.Tensor, wb: torch.Tensor, add: Optional[torch.Tensor], *, n: int,
+          eps: float, scale: float) -> None:
+    """x += scale (RMS norm of a + RMS norm of b) + add, in place; x float32 [T, ld], norms over n columns."""
+    device, stream = _on(x)
+    T, ld = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous() and 0 < n <= ld, "hybrid_ops.merge: x float32, contiguous")
+    for t in (a, b) if add is None else (a, b, add):
+        _need(t.dtype == a.dtype and t.shape[0] == T and t.shape[1] >= ld and t.stride(1) == 1 and t.device == x.device, "hybrid_ops.merge: branches")
+    for t in (wa, wb):
+        _need(t.dtype == torch.float32 and t.numel() >= ld and t.is_contiguous(), "hybrid_ops.merge: weights float32 [ld]")
+    _check(load().vmi_hy_merge(x.data_ptr(), a.data_ptr(), a.stride(0), b.data_ptr(), b.stride(0), _ptr(add),
+                               add.stride(0) if add is not None else 0, wa.data_ptr(), wb.data_ptr(), T, n, ld, eps, scale,
+                               DTYPES[a.dtype], device, stream))
+
+
+def glu(x: torch.Tensor, unit: GatedUnit, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The gated unit of interleaved (gate, up) columns: [T, 2 n] -> [T, n]."""
     device, stream = _on(x)
     T, n = x.shape[0], x.shape[1] // 2
-    _need(x.stride(1) == 1 and x.dtype in DTYPES, "hybrid_ops.glu: rows of unit stride")
-    out = torch.empty((T, n), dtype=x.dtype, device=x.device)
+    _need(x.dim() == 2 and x.stride(1) == 1 and x.dtype in DTYPES, "hybrid_ops.glu: rows of unit stride")
+    if out is None:
+        out = torch.empty((T, n), dtype=x.dtype, device=x.device)
+    _need(out.shape == (T, n) and out.stride(1) == 1 and out.dtype == x.dtype, "hybrid_ops.glu: out [T, n]")
     for t in range(0, T, 65535):      # (a launch's grid holds that many rows)
         m = min(65535, T - t)
-        _check(load().vmi_hy_glu(x[t:].data_ptr(), x.stride(0), out[t:].data_ptr(), n, m, n, float(limit), DTYPES[x.dtype], device, stream))
+        _check(load().vmi_hy_glu(x[t:].data_ptr(), x.stride(0), out[t:].data_ptr(), out.stride(0), m, n, unit.limit, unit.alpha, unit.up,
+                                 DTYPES[x.dtype], device, stream))
     return out
 
 
@@ -254,12 +332,17 @@ class StepLayout:
             _need(fields[name].dtype == torch.int32 and fields[name].numel() >= B and fields[name].is_contiguous(), f"StepLayout: {name}")
         tab = fields["table"]
         _need(tab.dtype == torch.int32 and tab.dim() == 2 and tab.shape[0] >= B and tab.is_contiguous(), "StepLayout: table")
+        chunks = fields.get("chunks")      # [n, 2], with chunk_start [B]: steps whose portions are longer than a token, where a layer asks
+        if chunks is not None:
+            _need(chunks.dtype == torch.int32 and chunks.dim() == 2 and chunks.shape[1] == 2 and chunks.is_contiguous(), "StepLayout: chunks")
+            _need(fields["chunk_start"].dtype == torch.int32 and fields["chunk_start"].numel() >= B, "StepLayout: chunk_start")
+        self.n_chunks = 0 if chunks is None else int(chunks.shape[0])
         self.fields = fields      # (keeps the tensors alive)
         self.T, self.B, self.single, self.spans = T, B, single, spans
         self.max_len, self.max_keys = max_len, max_keys      # longest portion, most keys any token sees
         self.args = StepArgs(**{k: fields[k].data_ptr() for k in ("tok_seq", "tok_pos", "tok_slot", "q_start", "q_len", "ctx",
                                                                   "state_slot", "flip", "table")},
-                             T=T, B=B, table_ld=tab.shape[1], page_size=page_size)
+                             chunks=_ptr(chunks), chunk_start=_ptr(fields.get("chunk_start")), n_chunks=self.n_chunks, T=T, B=B, table_ld=tab.shape[1], page_size=page_size)
         self.ref = ctypes.byref(self.args)
 
 
@@ -323,3 +406,94 @@ def latent_attention(q: torch.Tensor, cache: torch.Tensor, step: StepLayout, til
                       dtype=DTYPES[q.dtype], device=device)
     _check(load().vmi_hy_latent_attention(ctypes.byref(a), step.ref, stream))
     return out
+
+
+def state_fuses(dim: int, vdim: int) -> bool:
+    """Whether a step of single tokens finishes its rows (norm and output gate) by itself."""
+    return bool(load().vmi_hy_state_fuses(dim, vdim))
+
+
+def linear_state(proj: torch.Tensor, step: StepLayout, *, kind: int, heads: int, kv_heads: int, dim: int, vdim: int, dim_n: int,
+                 vdim_n: int, state: torch.Tensor, gate: torch.Tensor, act: str, eps: float, out: torch.Tensor,
+                 norm_w: Optional[torch.Tensor] = None, freq: Optional[torch.Tensor] = None, decay: Optional[torch.Tensor] = None,
+                 log2_decay: Optional[torch.Tensor] = None, beta: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None,
+                 conv_w: Optional[torch.Tensor] = None, rate: Optional[torch.Tensor] = None, dt_bias: Optional[torch.Tensor] = None,
+                 tail: Optional[torch.Tensor] = None) -> None:
+    """Linear attention with a matrix state: proj [T, q | k | v ...] -> out [T, heads vdim], every head over its root mean square,
+    times norm_w and the activated gate; state float32 [slots, heads, dim, vdim] (and tail) are updated."""
+    device, stream = _on(proj)
+    who, T, C, dt = "hybrid_ops.linear_state: ", step.T, 2 * kv_heads * dim + heads * vdim, proj.dtype
+    _need(proj.shape[0] == T and proj.shape[1] >= C and proj.stride(1) == 1 and dt in DTYPES, who + "proj")
+    _need(state.dim() == 4 and state.shape[1:] == (heads, dim, vdim) and state.dtype == torch.float32 and state.is_contiguous(), who + "state")
+    _need(out.shape == (T, heads * vdim) and out.stride(1) == 1 and out.dtype == dt and gate.shape == (T, heads * vdim)
+          and gate.stride(1) == 1 and gate.dtype == dt, who + "out, gate")
+    _need(norm_w is None or (norm_w.dtype == torch.float32 and norm_w.numel() == vdim), who + "norm weight float32 [vdim]")
+    taps = 0
+    if kind == DELTA:
+        taps = conv_w.shape[0]
+        _need(conv_w.shape == (taps, C) and rate.numel() == heads and dt_bias.numel() == heads * dim and beta.dtype == dt
+              and beta.shape == (T, heads) and beta.stride() == (proj.stride(0), 1) and z.dtype == dt and z.shape == (T, heads * dim)
+              and z.stride(1) == 1, who + "gates")
+        for t in (conv_w, rate, dt_bias):
+            _need(t.dtype == torch.float32 and t.is_contiguous(), who + "float32 constants")
+        _need(taps == 1 or (tail is not None and tail.shape == (state.shape[0], 2, taps - 1, C) and tail.dtype == dt
+                            and tail.is_contiguous()), who + "tail [slots, 2, taps - 1, channels]")
+    else:
+        _need(freq.dtype == torch.float64 and 2 * freq.numel() <= dim and decay.numel() == log2_decay.numel() == heads
+              and decay.dtype == log2_decay.dtype == torch.float32, who + "freq, decay")
+    lib, single = load(), step.single
+    fused = single and state_fuses(dim, vdim)
+    o = scratch = None
+    if not fused:
+        o = torch.empty((T, heads * vdim), dtype=torch.float32, device=proj.device)
+    if not single:
+        _need(step.n_chunks > 0, who + "the step's layout has no chunks")
+        scratch = torch.empty(step.n_chunks * heads * lib.vmi_hy_state_scratch(kind, dim, vdim), dtype=torch.float32, device=proj.device)
+    a = StateArgs(proj=proj.data_ptr(), beta=_ptr(beta), z=_ptr(z), conv_w=_ptr(conv_w), rate=_ptr(rate), dt_bias=_ptr(dt_bias),
+                  decay=_ptr(decay), log2_decay=_ptr(log2_decay), freq=_ptr(freq), state=state.data_ptr(),
+                  tail=_ptr(tail) if taps > 1 else None, o=_ptr(o), scratch=_ptr(scratch), out=out.data_ptr() if fused else None,
+                  gate=gate.data_ptr(), norm_w=_ptr(norm_w), ldp=proj.stride(0), ldz=z.stride(0) if z is not None else 0,
+                  ldo=out.stride(0), ldg=gate.stride(0), heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, dim_n=dim_n, vdim_n=vdim_n,
+                  taps=taps, rot_n=2 * freq.numel() if freq is not None else 0, kind=kind, single=int(single), act=ACTS[act], eps=eps,
+                  dtype=DTYPES[dt], device=device)
+    _check(lib.vmi_hy_state(ctypes.byref(a), step.ref, stream))
+    if not fused:
+        _check(lib.vmi_hy_head_norm_gate(o.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(norm_w), out.data_ptr(), out.stride(0), T,
+                                         heads, vdim, vdim_n, eps, ACTS[act], DTYPES[dt], device, stream))
+
+
+def kv_prep(proj: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, step: StepLayout, *, heads: int, kv_heads: int, dim: int, vdim: int,
+            dim_n: int, eps: float) -> None:
+    """proj [T, q | k | v ...]: q and k over their root mean square, q to q, k and v to the cache."""
+    device, stream = _on(proj)
+    _need(proj.shape[0] == step.T and proj.shape[1] >= (heads + kv_heads) * dim + kv_heads * vdim and proj.stride(1) == 1
+          and q.shape == (step.T, heads * dim) and q.is_contiguous() and q.dtype == proj.dtype and cache.dtype == proj.dtype
+          and cache.shape[-1] == kv_heads * (dim + vdim) and cache.is_contiguous(), "hybrid_ops.kv_prep: operand sizes")
+    a = KvPrepArgs(proj=proj.data_ptr(), q=q.data_ptr(), cache=cache.data_ptr(), ldp=proj.stride(0), heads=heads, kv_heads=kv_heads,
+                   dim=dim, vdim=vdim, dim_n=dim_n, eps=eps, dtype=DTYPES[proj.dtype], device=device)
+    _check(load().vmi_hy_kv_prep(ctypes.byref(a), step.ref, stream))
+
+
+def attention_row_tiles(dim: int, vdim: int, want: int, dtype: torch.dtype) -> int:
+    return int(load().vmi_hy_attention_row_tiles(dim, vdim, want, DTYPES[dtype]))
+
+
+def attention(q: torch.Tensor, cache: torch.Tensor, step: StepLayout, tiles: torch.Tensor, *, heads: int, kv_heads: int, dim: int,
+              vdim: int, scale: float, row_tiles: int, splits: int, out: torch.Tensor, chunk: int = 0, bias: Optional[torch.Tensor] = None,
+              sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
+    """q [T, heads dim] -> out [T, heads vdim] over the cache's pages; bias [heads, distances] and sink [heads] times log2(e)."""
+    device, stream = _on(q)
+    who = "hybrid_ops.attention: "
+    _need(q.shape == (step.T, heads * dim) and q.is_contiguous() and cache.dtype == q.dtype and cache.dim() == 3
+          and cache.shape[1] == step.args.page_size and cache.shape[2] == kv_heads * (dim + vdim) and cache.is_contiguous()
+          and tiles.dtype == torch.int32 and tiles.dim() == 2 and tiles.shape[1] == 2 and tiles.is_contiguous()
+          and out.shape == (step.T, heads * vdim) and out.stride(1) == 1 and out.dtype == q.dtype, who + "operand sizes")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.dim() == 2 and bias.shape[0] == heads and bias.is_contiguous()), who + "bias")
+    _need(sink is None or (sink.dtype == torch.float32 and sink.numel() == heads), who + "sink")
+    _need(gate is None or (gate.dtype == q.dtype and gate.shape == (step.T, heads) and gate.stride(1) == 1), who + "gate")
+    partial = torch.empty((splits, step.T * heads, vdim + 2), dtype=torch.float32, device=q.device) if splits > 1 else None
+    a = GqaArgs(q=q.data_ptr(), cache=cache.data_ptr(), out=out.data_ptr(), bias=_ptr(bias), sink=_ptr(sink), gate=_ptr(gate),
+                tiles=tiles.data_ptr(), partial=_ptr(partial), ldo=out.stride(0), ldg=gate.stride(0) if gate is not None else 0,
+                heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, bias_n=bias.shape[1] if bias is not None else 0, chunk=chunk,
+                n_tiles=tiles.shape[0], row_tiles=row_tiles, splits=splits, scale=scale, dtype=DTYPES[q.dtype], device=device)
+    _check(load().vmi_hy_attention(ctypes.byref(a), step.ref, stream))

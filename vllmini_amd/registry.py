@@ -61,16 +61,28 @@ def load_decoder(model_dir: str, *, dtype: Optional[str] = None, max_tokens: int
                            max_tokens=max_tokens, max_seqs=max_seqs, max_length=max_length, **decoder_kw)
 
 
-@register("Voduvik")
-def _voduvik(config, tensors, dtype, device, *, max_tokens, max_seqs, max_length=None, page_size=64, **kw):
+def _hybrid(name, config_class, build_model, config, tensors, dtype, device, *, max_tokens, max_seqs, max_length=None, page_size=64, **kw):
     from .hybrid_decoder import HybridDecoder
-    from .voduvik import VoduvikConfig, build_model
 
     dtype = dtype or torch.bfloat16
     if dtype not in (torch.bfloat16, torch.float32):
-        raise UnsupportedDtype(f"Voduvik is built for bfloat16 and float32, not {dtype}")
-    model = build_model(VoduvikConfig.from_json(config), tensors(), dtype, device)
+        raise UnsupportedDtype(f"{name} is built for bfloat16 and float32, not {dtype}")
+    model = build_model(config_class.from_json(config), tensors(), dtype, device)
     return HybridDecoder(model, model.make_pool(max_tokens, max_seqs, page_size, max_length), **kw)
+
+
+@register("Voduvik")
+def _voduvik(config, *args, **kw):
+    from .voduvik import VoduvikConfig, build_model
+
+    return _hybrid("Voduvik", VoduvikConfig, build_model, config, *args, **kw)
+
+
+@register("Fetelorn")
+def _fetelorn(config, *args, **kw):
+    from .fetelorn import FetelornConfig, build_model
+
+    return _hybrid("Fetelorn", FetelornConfig, build_model, config, *args, **kw)
 
 
 @register("GPT2LMHeadModel", "gpt2")
