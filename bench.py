@@ -131,12 +131,13 @@ def build_parser():
     ap.add_argument("--serve-no-deferred-scatter", action="store_true", help="the reference's call pair per layer instead")
     ap.add_argument("--serve-eager", action="store_true", help="plain launches instead of hipGraph replay")
     ap.add_argument("--no-serve", action="store_true", help="skip the extra serving-loop measurement")
-    ap.add_argument("--design", default="", choices=("", "voduvik"),
-                    help="prefill and decode throughput of another registered design at sizes of a real model's layers, beside GPT-2 "
+    ap.add_argument("--design", default="", choices=("", "voduvik", "fetelorn"),
+                    help="prefill and decode throughput of another registered design at sizes of a real model's layers, beside the closest other model "
                          "of equal width and depth (random weights; its own JSON, not the headline line)")
     ap.add_argument("--design-width", type=int, default=0, help="one width only (default: 1024, 2048 and 4096)")
     ap.add_argument("--design-part", default="all", choices=("all", "decode", "prefill"))
-    ap.add_argument("--design-model", default="both", choices=("both", "design", "gpt2"))
+    ap.add_argument("--design-model", default="both", choices=("both", "design", "closest"),
+                    help="the design, the closest of the other models at equal size (GPT-2 for voduvik, voduvik for fetelorn), or both")
     ap.add_argument("--design-batch", type=int, default=0, help="one decode batch only (default: 1, 32 and 256)")
     ap.add_argument("--min-timed-ms", type=float, default=50.0,
                     help="repeat the K-step timed region until the regions hold this many ms in all; the line reports the MEDIAN region")
@@ -887,16 +888,36 @@ def voduvik_config(width):
             "loop": {"start": 0, "stop": 2, "times": 2}, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5}, "logit_scale": 1.0}
 
 
-def design_decoders(width, batch, dev, which):
-    """(name, decoder) of the design and of GPT-2 with the same width and as many layers as the design has runs; pools sized for
-    `batch` sequences of DESIGN_CONTEXT tokens and for the prompts."""
-    tokens = max(batch * (DESIGN_CONTEXT + 128), DESIGN_PROMPTS * (DESIGN_CONTEXT + 64))
-    if which == "design":
-        from vllmini_amd.hybrid_decoder import HybridDecoder
-        from vllmini_amd.voduvik import VoduvikConfig, build_model, random_tensors
+def fetelorn_config(width):
+    """Eight layers in the proportions of a small production model (heads of 128 throughout, four query heads per key head, chunks longer
+    than the contexts measured, a feed-forward of three widths): six of retention, two of the parallel mixer."""
+    heads = width // 128
+    ff = {"kind": "dense", "ff": 3 * width}
+    ret = {"type": "retention", "mlp": ff,
+           "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1 - 2.0 ** (-5 - 4 * i / heads) for i in range(heads)],
+                     "rot": {"base": 10000.0, "dims": 128}}}
+    par = {"type": "parallel", "mlp": ff,
+           "mixer": {"left": {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "bias_max": 2048,
+                              "mask": {"size": 2048}},
+                     "right": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}}}
+    return {"architecture": "Fetelorn", "vocab": DESIGN_VOCAB, "width": width, "layers": [ret, ret, par, ret, ret, ret, par, ret],
+            "norm": {"eps": 1e-6}}
 
-        cfg = VoduvikConfig.from_json(voduvik_config(width))
-        model = build_model(cfg, random_tensors(cfg, dev), torch.bfloat16, dev)
+
+CLOSEST = {"voduvik": "gpt2", "fetelorn": "voduvik"}
+
+
+def design_decoders(name, width, batch, dev):
+    """The decoder of a design, or of GPT-2, with eight layer runs of a width; pools sized for `batch` sequences of DESIGN_CONTEXT
+    tokens and for the prompts."""
+    tokens = max(batch * (DESIGN_CONTEXT + 128), DESIGN_PROMPTS * (DESIGN_CONTEXT + 64))
+    if name != "gpt2":
+        from vllmini_amd import fetelorn, voduvik
+        from vllmini_amd.hybrid_decoder import HybridDecoder
+
+        cfg, mod = ((voduvik.VoduvikConfig.from_json(voduvik_config(width)), voduvik) if name == "voduvik" else
+                    (fetelorn.FetelornConfig.from_json(fetelorn_config(width)), fetelorn))
+        model = mod.build_model(cfg, mod.random_tensors(cfg, dev), torch.bfloat16, dev)
         return HybridDecoder(model, model.make_pool(tokens, max(batch, DESIGN_PROMPTS), 64, DESIGN_CONTEXT + 128))
     from vllmini_amd.gpt2_decode import GPT2Dims, GPT2PagedDecoder, random_state_dict
     from vllmini_amd.kv_pool import PagedKVPool
@@ -957,11 +978,12 @@ def design_prefill(dec, dev, repeats=3):
 def run_design(args, dev):
     rows = []
     for width in [args.design_width] if args.design_width else [1024, 2048, 4096]:
-        for which in ("design", "gpt2") if args.design_model == "both" else (args.design_model,):
+        pair = {"both": (args.design, CLOSEST[args.design]), "design": (args.design,), "closest": (CLOSEST[args.design],)}
+        for name in pair[args.design_model]:
             for batch in [args.design_batch] if args.design_batch else [1, 32, 256]:
-                dec = design_decoders(width, batch, dev, which)
-                row = {"model": args.design if which == "design" else "gpt2", "width": width, "layer_runs": 8, "batch": batch,
-                       "context": DESIGN_CONTEXT, "dtype": "bf16" if which == "design" else "f16", "data": "synthetic"}
+                dec = design_decoders(name, width, batch, dev)
+                row = {"model": name, "width": width, "layer_runs": 8, "batch": batch,
+                       "context": DESIGN_CONTEXT, "dtype": "f16" if name == "gpt2" else "bf16", "data": "synthetic"}
                 if args.design_part != "prefill":
                     ms = design_decode(dec, batch, dev, min(args.steps, 30))
                     row.update(decode_ms_per_step=ms, decode_tokens_per_s=batch / ms * 1e3)

@@ -178,7 +178,7 @@ typedef struct {
   const float* dt_bias;    /* [heads dim] */
   const float* decay;      /* [heads]: RETENTION */
   const float* log2_decay; /* [heads] */
-  const double* freq;      /* [rot_n / 2] */
+  const float* turns;      /* [T][rot_n / 2][2]: what vmi_hy_rotations wrote */
   float* state;            /* [slots][heads][dim][vdim] */
   void* tail;              /* [slots][2][taps - 1][2 kv_heads dim + heads vdim] element type */
   float* o;
@@ -191,6 +191,8 @@ typedef struct {
   float eps;
   int32_t dtype, device;
 } vmi_hy_state_args;
+/* out [T][half][2] = cos, sin of tok_pos[t] * freq[i]: once per step for all layers of one set of frequencies */
+VMI_HY_API int vmi_hy_rotations(const double* freq, int32_t half, float* out, const vmi_hy_step* s, int32_t device, void* stream);
 VMI_HY_API int64_t vmi_hy_state_scratch(int32_t kind, int32_t dim, int32_t vdim);
 VMI_HY_API int32_t vmi_hy_state_fuses(int32_t dim, int32_t vdim);
 VMI_HY_API int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream);

@@ -10,18 +10,19 @@
 
 namespace vmi_hybrid {
 
-constexpr int BIAS_LDS = 8192;   // floats of the bias table kept in LDS (larger ones are read from memory)
+// distances that the rows of a tile (R of them, rep to a token) can have to the keys of one tile
+__host__ __device__ inline int bias_window(int KT, int R, int rep) { return KT + (R + rep - 1) / rep; }
 
 template <typename T, int KT, int RT>
-inline size_t gqa_lds(int dim, int vdim, int bias) {
+inline size_t gqa_lds(int dim, int vdim, int rep, bool bias) {
   constexpr int PAD = pad_of<T>();
   return ((size_t)KT * (dim + vdim + PAD) + (size_t)16 * RT * (dim + PAD) + (size_t)16 * RT * (KT + PAD)) * sizeof(T) +
-         (size_t)4 * 16 * RT * 4 + (size_t)bias * 4;
+         (size_t)4 * 16 * RT * 4 + (bias ? (size_t)rep * bias_window(KT, 16 * RT, rep) * 4 : 0);
 }
 
 // RT row tiles, NT value tiles (of 16 columns) per wave, U 8-element units of a cache row per thread
 template <typename T, int KT, int RT, int NT, int U>
-__global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p, const vmi_hy_step s, const int bias_lds) {
+__global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p, const vmi_hy_step s) {
   constexpr int R = 16 * RT, TPK = 256 / KT, PAD = pad_of<T>(), LDP = KT + PAD, SW = KT / 16;   // SW waves score
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int dim = p.dim, vdim = p.vdim, D = dim + vdim, LDK = D + PAD, LDQ = dim + PAD;
@@ -29,7 +30,7 @@ __global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p,
   T* qs = ks + (size_t)KT * LDK;                   // [R][LDQ]
   T* ps = qs + (size_t)R * LDQ;                    // [R][LDP]
   float* sx = reinterpret_cast<float*>(ps + (size_t)R * LDP);   // [4][R]
-  float* bl = sx + 4 * R;                          // [rep][bias_n]
+  float* bl = sx + 4 * R;                          // [rep][window]: the bias of the distances that occur in a tile
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), kc = lane >> 4, r16 = lane & 15;
   const int e = p.tiles[2 * blockIdx.x], r0 = p.tiles[2 * blockIdx.x + 1], split = blockIdx.y, g = blockIdx.z;
   if (e < 0) return;
@@ -73,8 +74,21 @@ __global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p,
     *reinterpret_cast<V8<T>*>(qs + m * LDQ + k) =
         load8(static_cast<const T*>(p.q) + ((int64_t)(tok0 + row / rep) * p.heads + h0 + row % rep) * dim + k);
   }
-  const float* bg = p.bias ? p.bias + (int64_t)h0 * p.bias_n : nullptr;
-  for (int u = tid; u < bias_lds; u += 256) bl[u] = bg[u];
+  // the window's entry (hh, w): head hh, distance first - (last key of the tile) + w
+  const int BW = bias_window(KT, R, rep), bn = p.bias ? rep * BW : 0;
+  const float* bg = p.bias + (int64_t)h0 * p.bias_n;
+  auto bias_at = [&](int kt, int u) {
+    const int hh = u / BW, w = u - hh * BW;
+    return bg[(int64_t)hh * p.bias_n + min(max(first - (kt * KT + KT - 1) + w, 0), p.bias_n - 1)];
+  };
+  constexpr int BU = 2;   // of a window, per thread, requested with the tile's keys
+  float br[BU] = {};
+  auto load_bias = [&](int kt) {
+#pragma unroll
+    for (int i = 0; i < BU; ++i)
+      if (bn) br[i] = bias_at(kt, min(tid + 256 * i, bn - 1));
+  };
+  load_bias(kt0);
 
   f32x4 o[RT][NT];
   float mrun[RT][4], lrun[RT][4];
@@ -94,7 +108,7 @@ __global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p,
       }
       lim[rt][r] = ctx + row / rep;
       low[rt][r] = p.chunk > 0 ? lim[rt][r] / p.chunk * p.chunk : 0;
-      boff[rt][r] = hh * p.bias_n;
+      boff[rt][r] = hh * BW + lim[rt][r] - first;
     }
   }
   const float sc2 = p.scale * 1.4426950408889634f;   // scores in units of log 2
@@ -103,7 +117,13 @@ __global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p,
 #pragma unroll
     for (int i = 0; i < U; ++i)   // (a clamped column is written again with the same values)
       *reinterpret_cast<V8<T>*>(ks + kj * LDK + min(kcol + i * TPK * 8, D - 8)) = kr[i];
+    if (bn) {
+#pragma unroll
+      for (int i = 0; i < BU; ++i) bl[min(tid + 256 * i, bn - 1)] = br[i];   // (a clamped entry is written again with the same value)
+      for (int u = tid + 256 * BU; u < bn; u += 256) bl[u] = bias_at(kt, u);
+    }
     if (kt + 1 < kt1) {
+      load_bias(kt + 1);
       load_tile(next_page, kt + 1);
       next_page = tab[key_of(min(kt + 2, kt1 - 1)) / s.page_size];
     }
@@ -125,10 +145,7 @@ __global__ __launch_bounds__(256) void gqa_kernel(const vmi_hy_attention_args p,
       for (int rt = 0; rt < RT; ++rt) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int dist = min(max(lim[rt][r] - key, 0), p.bias_n - 1) + boff[rt][r];
-          float b = 0.f;
-          if (bias_lds) b = bl[dist];
-          else if (bg) b = bg[dist];
+          const float b = bn ? bl[boff[rt][r] + KT - 1 - (wave * 16 + r16)] : 0.f;
           sc[rt][r] = key <= lim[rt][r] && key >= low[rt][r] ? fmaf(sc[rt][r], sc2, b) : -INFINITY;
           const float v = max16(sc[rt][r]);
           if (r16 == 0) sx[wave * R + rt * 16 + 4 * kc + r] = v;
@@ -264,11 +281,9 @@ __global__ __launch_bounds__(256) void kv_prep_kernel(const vmi_hy_kv_prep_args 
 template <typename T, int KT, int RT, int NT, int U>
 static int launch_gqa(const vmi_hy_attention_args& p, const vmi_hy_step& s, hipStream_t st) {
   auto* fn = gqa_kernel<T, KT, RT, NT, U>;
-  const int table = p.bias ? p.heads / p.kv_heads * p.bias_n : 0;
-  const int in_lds = table <= BIAS_LDS && gqa_lds<T, KT, RT>(p.dim, p.vdim, table) <= LDS_PER_CU ? table : 0;
-  const size_t lds = gqa_lds<T, KT, RT>(p.dim, p.vdim, in_lds);
+  const size_t lds = gqa_lds<T, KT, RT>(p.dim, p.vdim, p.heads / p.kv_heads, p.bias != nullptr);
   if (int rc = allow_lds(fn, lds, "vmi_hy_attention")) return rc;
-  hipLaunchKernelGGL(fn, dim3(p.n_tiles, p.splits, p.kv_heads), dim3(256), lds, st, p, s, in_lds);
+  hipLaunchKernelGGL(fn, dim3(p.n_tiles, p.splits, p.kv_heads), dim3(256), lds, st, p, s);
   if (p.splits > 1) launch_combine<T>(Combine{p.partial, p.out, p.gate, s.tok_seq, p.ldo, p.ldg, s.T, p.heads, p.vdim, p.splits}, st);
   return launched("vmi_hy_attention");
 }
@@ -278,6 +293,7 @@ static int gqa_width(const vmi_hy_attention_args& p, const vmi_hy_step& s, hipSt
   const int units = (p.dim + p.vdim + 2048 / KT - 1) / (2048 / KT);   // of 8 elements of a cache row, per thread
   constexpr int H = 64 / KT;                                          // (tiles of 32 keys: twice the threads per key)
   if (p.vdim <= 128 && units * H <= 4) return launch_gqa<T, KT, RT, 2, 4 / H>(p, s, st);
+  if (p.vdim <= 128 && units * H <= 8) return launch_gqa<T, KT, RT, 2, 8 / H>(p, s, st);
   if (p.vdim <= 256 && units * H <= 8) return launch_gqa<T, KT, RT, 4, 8 / H>(p, s, st);
   if constexpr (RT <= 2)
     if (p.vdim <= 512 && units * H <= 16) return launch_gqa<T, KT, RT, 8, 16 / H>(p, s, st);
@@ -303,7 +319,7 @@ static int run_gqa(const vmi_hy_attention_args& p, const vmi_hy_step& s, hipStre
     if (p.row_tiles == 4) return gqa_width<T, 64, 4>(p, s, st);
     if (p.row_tiles == 2) return gqa_width<T, 64, 2>(p, s, st);
   }
-  return gqa_lds<T, 64, 1>(p.dim, p.vdim, 0) <= LDS_PER_CU ? gqa_width<T, 64, 1>(p, s, st) : gqa_width<T, 32, 1>(p, s, st);
+  return gqa_lds<T, 64, 1>(p.dim, p.vdim, p.heads / p.kv_heads, p.bias != nullptr) <= LDS_PER_CU ? gqa_width<T, 64, 1>(p, s, st) : gqa_width<T, 32, 1>(p, s, st);
 }
 
 }  // namespace vmi_hybrid

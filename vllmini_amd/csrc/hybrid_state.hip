@@ -7,10 +7,12 @@
 //     S  <- e^{G_15} S + sum_j (k_j e^{G_15 - G_j}) u_j^T
 // (retention: u = v, no A).  state_prep_kernel makes, for every (chunk, head) independently, the triangular system's solutions
 // W = (I + beta A)^-1 beta (k e^G) and U0 = (I + beta A)^-1 beta v, q e^G, k e^{G_15 - G} and B; exponents are always of differences
-// i >= j, so nothing can overflow.  state_scan_kernel then walks a state's chunks: u = U0 - W S, o = q e^G S + B u, S update, on
-// v_mfma_f32_16x16x4_f32.  A wave owns 16 value columns of one head's state for the whole walk, in the matrix core's result layout
-// (lane (kc, r16): rows 4 kc + r of column r16), which is at the same time the operand layout of the next product: no LDS, no
-// barrier, and rows past a portion's end are zeros in every operand.
+// i >= j, so nothing can overflow (where a chunk decays little, products of e^{G_i} and e^{-G_j} on the matrix cores instead).
+// state_scan_kernel then walks a state's chunks: u = U0 - W S, o = q e^G S + B u, S update, on v_mfma_f32_16x16x4_f32.  A workgroup
+// owns 16 value columns of one head's state for the whole walk, each wave some of its rows, in the matrix core's result layout
+// (lane (kc, r16): rows 4 kc + r of column r16), which is at the same time the operand layout of the next product.  What the waves
+// exchange per chunk is their part of W S and q e^G S (16 x 16 each, one barrier); the operands of the next chunks are in flight
+// meanwhile, and rows past a portion's end are zeros in all of them.
 //
 // Steps of single tokens: state_step_kernel reads each state once, keeps it in registers between the correction and the read-out,
 // and writes it back; convolution, gates, norm and output gate ride along.
@@ -74,42 +76,82 @@ __device__ __forceinline__ void write_tail(const vmi_hy_state_args& p, const Por
   }
 }
 
-// cos, sin of position * frequency, the angle reduced in fp64: exact to fp32 at any position
-__device__ __forceinline__ f32x2 turn(double pos, double f) {
-  const double a = pos * f;
-  const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
-  return f32x2{cosf(r), sinf(r)};
+// cos, sin of position * frequency, the angle reduced in fp64: exact to fp32 at any position.  One row per token
+__global__ __launch_bounds__(64) void rotations_kernel(const double* __restrict__ freq, int half, float* __restrict__ out,
+                                                       const int* __restrict__ tok_pos) {
+  const int t = blockIdx.x;
+  const double pos = (double)tok_pos[t];
+  for (int i = threadIdx.x; i < half; i += 64) {
+    const double a = pos * freq[i];
+    const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
+    *reinterpret_cast<f32x2*>(out + ((int64_t)t * half + i) * 2) = f32x2{cosf(r), sinf(r)};
+  }
 }
 
-// q and k of one head, `rows` of them from packed row t0, rotated, k / sqrt(dim_n), into LDS
+// q and k of one head in packed row t, rotated, k / sqrt(dim_n), into LDS rows: the share of lane l of L
 template <typename T>
-__device__ __forceinline__ void rotated_rows(const vmi_hy_state_args& p, int t0, int pos0, int rows, int n, int h, int hk, float* ql,
-                                             float* kl, int ld, int tid) {
+__device__ __forceinline__ void rotated_row(const vmi_hy_state_args& p, int t, int hk, float* ql, float* kl, int l, int L) {
   const int half = p.rot_n >> 1;
   const float ks = 1.f / sqrtf((float)p.dim_n);
-  for (int u = tid; u < rows * p.dim; u += 256) {
-    const int m = u / p.dim, i = u - m * p.dim;
-    float q = 0.f, k = 0.f;
-    if (m < n && i < p.rot_n) {
-      if (i >= half) continue;
-      const T* qr = static_cast<const T*>(p.proj) + (int64_t)(t0 + m) * p.ldp + (int64_t)hk * p.dim;
-      const T* kr = qr + (int64_t)p.kv_heads * p.dim;
-      const f32x2 cs = turn((double)(pos0 + m), p.freq[i]);
+  const T* qr = static_cast<const T*>(p.proj) + (int64_t)t * p.ldp + (int64_t)hk * p.dim;
+  const T* kr = qr + (int64_t)p.kv_heads * p.dim;
+  const float* cs = p.turns + (int64_t)t * half * 2;
+  if ((half & 3) == 0) {   // four pairs at a time
+    for (int i = 4 * l; i < half; i += 4 * L) {
+      const V4<T> qa = *reinterpret_cast<const V4<T>*>(qr + i), qb = *reinterpret_cast<const V4<T>*>(qr + i + half);
+      const V4<T> ka = *reinterpret_cast<const V4<T>*>(kr + i), kb = *reinterpret_cast<const V4<T>*>(kr + i + half);
+      const f32x8 c = load8(cs + 2 * i);
+      f32x4 q0, q1, k0, k1;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const float co = c[2 * x], si = c[2 * x + 1];
+        q0[x] = (float)qa[x] * co - (float)qb[x] * si;
+        q1[x] = (float)qb[x] * co + (float)qa[x] * si;
+        k0[x] = ((float)ka[x] * co - (float)kb[x] * si) * ks;
+        k1[x] = ((float)kb[x] * co + (float)ka[x] * si) * ks;
+      }
+      *reinterpret_cast<f32x4*>(ql + i) = q0;
+      *reinterpret_cast<f32x4*>(ql + i + half) = q1;
+      *reinterpret_cast<f32x4*>(kl + i) = k0;
+      *reinterpret_cast<f32x4*>(kl + i + half) = k1;
+    }
+  } else {
+    for (int i = l; i < half; i += L) {
       const float qa = (float)qr[i], qb = (float)qr[i + half], ka = (float)kr[i], kb = (float)kr[i + half];
-      ql[m * ld + i] = qa * cs[0] - qb * cs[1];
-      ql[m * ld + i + half] = qb * cs[0] + qa * cs[1];
-      kl[m * ld + i] = (ka * cs[0] - kb * cs[1]) * ks;
-      kl[m * ld + i + half] = (kb * cs[0] + ka * cs[1]) * ks;
-      continue;
+      const float co = cs[2 * i], si = cs[2 * i + 1];
+      ql[i] = qa * co - qb * si;
+      ql[i + half] = qb * co + qa * si;
+      kl[i] = (ka * co - kb * si) * ks;
+      kl[i + half] = (kb * co + ka * si) * ks;
     }
-    if (m < n) {
-      const T* qr = static_cast<const T*>(p.proj) + (int64_t)(t0 + m) * p.ldp + (int64_t)hk * p.dim;
-      q = (float)qr[i];
-      k = (float)qr[(int64_t)p.kv_heads * p.dim + i] * ks;
-    }
-    ql[m * ld + i] = q;
-    kl[m * ld + i] = k;
   }
+  for (int i = p.rot_n + l; i < p.dim; i += L) {   // passes unrotated (padding: zeros)
+    ql[i] = (float)qr[i];
+    kl[i] = (float)kr[i] * ks;
+  }
+}
+
+__device__ __forceinline__ void mma4(f32x4& acc, const f32x4& a, const f32x4& b) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], acc, 0, 0, 0);
+}
+
+// this wave's part (every fourth 16 channels) of the 16 x 16 products of LDS rows a and b
+__device__ __forceinline__ f32x4 row_products(const float* a, const float* b, int ld, int dim, int wave, int lane) {
+  const int at = (lane & 15) * ld + 4 * (lane >> 4);
+  f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int c = 16 * wave; c < dim; c += 64)
+    mma4(acc, *reinterpret_cast<const f32x4*>(a + at + c), *reinterpret_cast<const f32x4*>(b + at + c));
+  return acc;
+}
+// ... and its place: part[wave][16][20], row i = 4 kc + r, column j
+__device__ __forceinline__ void put_products(float* part, const f32x4& v, int wave, int lane) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) part[(wave * CH + 4 * (lane >> 4) + r) * 20 + (lane & 15)] = v[r];
+}
+__device__ __forceinline__ float sum_products(const float* part, int i, int j) {
+  const float* v = part + i * 20 + j;
+  return (v[0] + v[CH * 20]) + (v[2 * CH * 20] + v[3 * CH * 20]);
 }
 
 // what one (chunk, head) hands to the walk, in floats
@@ -127,8 +169,12 @@ struct Scratch {
 };
 
 inline size_t prep_lds(int kind, int dim, int vdim) {
-  return ((size_t)CH * (dim + 4) * (kind == VMI_HY_DELTA ? 3 : 2) + (size_t)CH * (vdim + 4) + 2 * CH * 20 + CH) * sizeof(float);
+  const bool delta = kind == VMI_HY_DELTA;
+  return ((size_t)CH * (dim + 4) * (delta ? 3 : 2) + (size_t)CH * (vdim + 4) + (size_t)(delta ? 9 : 4) * CH * 20 + 2 * CH + (delta ? dim : 0)) *
+         sizeof(float);
 }
+
+constexpr float LITTLE_DECAY = 24.f;   // a chunk whose channels decay by at most e^-24 takes the matrix cores for A and B
 
 template <typename T, int KIND, int TAPS>
 __global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
@@ -138,70 +184,85 @@ __global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args
   float* kl = ql + CH * LD;                                    // [16][LD]
   float* gl = kl + CH * LD;                                    // [16][LD] (delta)
   float* vl = gl + (KIND == VMI_HY_DELTA ? CH * LD : 0);       // [16][LDV]
-  float* Al = vl + CH * LDV;                                   // [16][20] beta_i A_ij
-  float* Bl = Al + CH * 20;                                    // [16][20]
-  float* be = Bl + CH * 20;                                    // [16]
-  const int tid = threadIdx.x, h = blockIdx.y, hk = h / (p.heads / p.kv_heads);
+  float* pb = vl + CH * LDV;                                   // [4][16][20] parts of B
+  float* pa = pb + 4 * CH * 20;                                // [4][16][20] parts of A (delta)
+  float* Al = pa + (KIND == VMI_HY_DELTA ? 4 * CH * 20 : 0);   // [16][20] beta_i A_ij (delta)
+  float* be = Al + (KIND == VMI_HY_DELTA ? CH * 20 : 0);       // [16]: beta | (retention) powers of the decay
+  float* most = be + CH;                                       // [4]
+  float* dl = most + CH;                                       // [dim] e^{G_15} (delta)
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), m16 = tid >> 4, l16 = tid & 15;
+  const int h = blockIdx.y, hk = h / (p.heads / p.kv_heads);
   const int e = s.chunks[2 * blockIdx.x], first = s.chunks[2 * blockIdx.x + 1];
   const Portion r = portion(s, e);
   const int t0 = r.qs + first, n = min(CH, r.len - first), C = 2 * p.kv_heads * dim + p.heads * vdim;
   const int cq = hk * dim, ck = (p.kv_heads + hk) * dim, cv = 2 * p.kv_heads * dim + h * vdim;
   const Scratch sc(KIND, dim, vdim);
   float* out = p.scratch + ((int64_t)blockIdx.x * p.heads + h) * sc.size;
+  const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
 
   if constexpr (KIND == VMI_HY_DELTA) {
-    const int ud = dim >> 3, uv = vdim >> 3;
-    for (int u = tid; u < CH * (2 * ud + uv); u += 256) {
-      const int m = u / (2 * ud + uv);
-      int c = u - m * (2 * ud + uv);
-      float* dst;
-      int ch;
-      if (c < ud) dst = ql + m * LD + c * 8, ch = cq + c * 8;
-      else if (c < 2 * ud) c -= ud, dst = kl + m * LD + c * 8, ch = ck + c * 8;
-      else c -= 2 * ud, dst = vl + m * LDV + c * 8, ch = cv + c * 8;
-      f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (m < n) v = conv_silu8<T, TAPS>(p, r, C, t0 + m, ch);
-      *reinterpret_cast<f32x4*>(dst) = f32x4{v[0], v[1], v[2], v[3]};
-      *reinterpret_cast<f32x4*>(dst + 4) = f32x4{v[4], v[5], v[6], v[7]};
-    }
+    // row m16, 16 lanes: channels through the convolution
+    auto conv = [&](float* dst, int ch, int width) {
+      for (int c = 8 * l16; c < width; c += 128) {
+        f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        if (m16 < n) v = conv_silu8<T, TAPS>(p, r, C, t0 + m16, ch + c);
+        *reinterpret_cast<f32x4*>(dst + c) = f32x4{v[0], v[1], v[2], v[3]};
+        *reinterpret_cast<f32x4*>(dst + c + 4) = f32x4{v[4], v[5], v[6], v[7]};
+      }
+    };
+    conv(ql + m16 * LD, cq, dim);
+    conv(kl + m16 * LD, ck, dim);
+    conv(vl + m16 * LDV, cv, vdim);
     if (tid < CH) be[tid] = tid < n ? sigmoid((float)static_cast<const T*>(p.beta)[(int64_t)(t0 + tid) * p.ldp + h]) : 0.f;
-    const float rate = p.rate[h];
-    for (int c = tid; c < dim; c += 256) {
-      const float bias = p.dt_bias[(int64_t)h * dim + c];
-      float G = 0.f;
-#pragma unroll 4
-      for (int m = 0; m < CH; ++m) {
-        const float z = (float)static_cast<const T*>(p.z)[(int64_t)(t0 + min(m, n - 1)) * p.ldz + (int64_t)h * dim + c] + bias;
-        if (m < n) G -= rate * softplus(z);
-        gl[m * LD + c] = G;
+    {   // decays: the steps row by row, then their sums down the rows
+      const float rate = p.rate[h];
+      const T* z = static_cast<const T*>(p.z) + (int64_t)(t0 + min(m16, n - 1)) * p.ldz + (int64_t)h * dim;
+      const float* bias = p.dt_bias + (int64_t)h * dim;
+      for (int c = 4 * l16; c < dim; c += 64) {
+        const V4<T> zv = *reinterpret_cast<const V4<T>*>(z + c);
+        const f32x4 bv = *reinterpret_cast<const f32x4*>(bias + c);
+        f32x4 g;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) g[x] = m16 < n ? -rate * softplus((float)zv[x] + bv[x]) : 0.f;
+        *reinterpret_cast<f32x4*>(gl + m16 * LD + c) = g;
       }
     }
-    __syncthreads();
-    {   // unit lengths: 16 lanes a row
-      const int m = tid >> 4, l = tid & 15;
+    {   // unit lengths of the rows of this lane group's own making
+      float* q = ql + m16 * LD;
+      float* k = kl + m16 * LD;
       float a = 0.f, b = 0.f;
-      for (int c = l; c < dim; c += 16) {
-        a = fmaf(ql[m * LD + c], ql[m * LD + c], a);
-        b = fmaf(kl[m * LD + c], kl[m * LD + c], b);
-      }
+      for (int c = 8 * l16; c < dim; c += 128)
+#pragma unroll
+        for (int x = 0; x < 8; ++x) a = fmaf(q[c + x], q[c + x], a), b = fmaf(k[c + x], k[c + x], b);
 #pragma unroll
       for (int o = 8; o > 0; o >>= 1) a += __shfl_xor(a, o, 64), b += __shfl_xor(b, o, 64);
       a = 1.f / sqrtf((a + 1e-6f) * (float)p.dim_n);
       b = 1.f / sqrtf(b + 1e-6f);
-      for (int c = l; c < dim; c += 16) {
-        ql[m * LD + c] *= a;
-        kl[m * LD + c] *= b;
-      }
+      for (int c = 8 * l16; c < dim; c += 128)
+#pragma unroll
+        for (int x = 0; x < 8; ++x) q[c + x] *= a, k[c + x] *= b;
     }
     __syncthreads();
-    {
-      const int i = tid >> 4, j = tid & 15;
+    float deepest = 0.f;
+    for (int c = tid; c < dim; c += 256) {
+      float G = 0.f;
+#pragma unroll
+      for (int m = 0; m < CH; ++m) gl[m * LD + c] = G += gl[m * LD + c];
+      dl[c] = exp_hw(G);
+      deepest = fminf(deepest, G);
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) deepest = fminf(deepest, __shfl_xor(deepest, o, 64));
+    if (lane == 0) most[wave] = deepest;
+    __syncthreads();
+    const bool little = fminf(fminf(most[0], most[1]), fminf(most[2], most[3])) >= -LITTLE_DECAY;
+    if (!little) {   // exponents of differences, pair by pair
       float a = 0.f, b = 0.f;
-      if (j <= i) {
+      if (l16 <= m16) {
         for (int c = 0; c < dim; c += 4) {
-          const f32x4 qi = *reinterpret_cast<const f32x4*>(ql + i * LD + c), ki = *reinterpret_cast<const f32x4*>(kl + i * LD + c);
-          const f32x4 kj = *reinterpret_cast<const f32x4*>(kl + j * LD + c), gi = *reinterpret_cast<const f32x4*>(gl + i * LD + c);
-          const f32x4 gj = *reinterpret_cast<const f32x4*>(gl + j * LD + c);
+          const f32x4 qi = *reinterpret_cast<const f32x4*>(ql + m16 * LD + c), ki = *reinterpret_cast<const f32x4*>(kl + m16 * LD + c);
+          const f32x4 kj = *reinterpret_cast<const f32x4*>(kl + l16 * LD + c), gi = *reinterpret_cast<const f32x4*>(gl + m16 * LD + c);
+          const f32x4 gj = *reinterpret_cast<const f32x4*>(gl + l16 * LD + c);
 #pragma unroll
           for (int x = 0; x < 4; ++x) {
             const float w = kj[x] * exp_hw(gi[x] - gj[x]);
@@ -210,38 +271,76 @@ __global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args
           }
         }
       }
-      Al[i * 20 + j] = j < i ? a * be[i] : 0.f;
-      out[sc.b + i * CH + j] = j <= i ? b : 0.f;
+      Al[m16 * 20 + l16] = l16 < m16 ? a * be[m16] : 0.f;
+      out[sc.b + tid] = l16 <= m16 ? b : 0.f;
+      __syncthreads();
+    }
+    // q e^G; where it decays little also k e^G (in G's place) and k e^-G (in k's)
+    for (int c = 4 * l16; c < dim; c += 64) {
+      const int at = m16 * LD + c;
+      const f32x4 g = *reinterpret_cast<const f32x4*>(gl + at), k = *reinterpret_cast<const f32x4*>(kl + at);
+      f32x4 q = *reinterpret_cast<const f32x4*>(ql + at), kg, kn;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const float eg = exp_hw(g[x]);
+        q[x] *= eg;
+        kg[x] = k[x] * eg;
+        kn[x] = little ? k[x] * exp_hw(-g[x]) : k[x];
+      }
+      *reinterpret_cast<f32x4*>(ql + at) = q;
+      *reinterpret_cast<f32x4*>(out + sc.q + m16 * dim + c) = q;
+      *reinterpret_cast<f32x4*>(kl + at) = kn;
+      if (little) *reinterpret_cast<f32x4*>(gl + at) = kg;
+    }
+    __syncthreads();
+    if (little) {
+      put_products(pa, row_products(gl, kl, LD, dim, wave, lane), wave, lane);
+      put_products(pb, row_products(ql, kl, LD, dim, wave, lane), wave, lane);
+      __syncthreads();
+      Al[m16 * 20 + l16] = l16 < m16 ? sum_products(pa, m16, l16) * be[m16] : 0.f;
+      out[sc.b + tid] = l16 <= m16 ? sum_products(pb, m16, l16) : 0.f;
+    }
+    // k e^{G_15 - G}, transposed: 4 rows of a channel a thread
+    for (int c = tid >> 2; c < dim; c += 64) {
+      const int y = 4 * (tid & 3);
+      f32x4 k;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const float g = little ? dl[c] : exp_hw(gl[(CH - 1) * LD + c] - gl[(y + x) * LD + c]);
+        k[x] = kl[(y + x) * LD + c] * g;
+      }
+      *reinterpret_cast<f32x4*>(out + sc.k + c * CH + y) = k;
+    }
+    if (!little) {
+      __syncthreads();
+      for (int c = 4 * l16; c < dim; c += 64) {
+        const int at = m16 * LD + c;
+        const f32x4 g = *reinterpret_cast<const f32x4*>(gl + at), k = *reinterpret_cast<const f32x4*>(kl + at);
+        f32x4 kg;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) kg[x] = k[x] * exp_hw(g[x]);
+        *reinterpret_cast<f32x4*>(gl + at) = kg;
+      }
     }
     __syncthreads();
     // forward substitution, a column a thread: of W (dim of them), of U0 (vdim)
     for (int col = tid; col < dim + vdim; col += 256) {
       const bool isw = col < dim;
       const int c = isw ? col : col - dim;
+      const float* rhs = isw ? gl + c : vl + c;
+      const int ld = isw ? LD : LDV;
       float x[CH];
 #pragma unroll
       for (int i = 0; i < CH; ++i) {
-        float v = isw ? kl[i * LD + c] * exp_hw(gl[i * LD + c]) : vl[i * LDV + c];
-        v *= be[i];
+        float v = rhs[i * ld] * be[i];
 #pragma unroll
         for (int j = 0; j < i; ++j) v = fmaf(-Al[i * 20 + j], x[j], v);
         x[i] = v;
       }
       if (isw) {
-        const float G = gl[(CH - 1) * LD + c];
-        out[sc.d + c] = exp_hw(G);
+        out[sc.d + c] = dl[c];
 #pragma unroll
-        for (int i = 0; i < CH; ++i) {
-          out[sc.w + i * dim + c] = x[i];
-          out[sc.q + i * dim + c] = ql[i * LD + c] * exp_hw(gl[i * LD + c]);
-        }
-#pragma unroll
-        for (int i = 0; i < CH; i += 4) {
-          f32x4 k;
-#pragma unroll
-          for (int y = 0; y < 4; ++y) k[y] = kl[(i + y) * LD + c] * exp_hw(G - gl[(i + y) * LD + c]);
-          *reinterpret_cast<f32x4*>(out + sc.k + c * CH + i) = k;
-        }
+        for (int i = 0; i < CH; ++i) out[sc.w + i * dim + c] = x[i];
       } else {
 #pragma unroll
         for (int i = 0; i < CH; i += 4) *reinterpret_cast<f32x4*>(out + sc.u + c * CH + i) = f32x4{x[i], x[i + 1], x[i + 2], x[i + 3]};
@@ -255,125 +354,138 @@ __global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args
       }
     }
   } else {
-    rotated_rows<T>(p, t0, r.ctx + first, CH, n, h, hk, ql, kl, LD, tid);
-    for (int u = tid; u < CH * vdim; u += 256) {
-      const int m = u / vdim, c = u - m * vdim;
-      vl[m * LDV + c] = m < n ? (float)static_cast<const T*>(p.proj)[(int64_t)(t0 + m) * p.ldp + cv + c] : 0.f;
+    const float ld = p.log2_decay[h];
+    if (tid <= CH) be[tid] = exp2f(ld * (float)tid);   // d^0 .. d^16 (runs one past be, into most)
+    if (m16 < n) {
+      rotated_row<T>(p, t0 + m16, hk, ql + m16 * LD, kl + m16 * LD, l16, 16);
+    } else {
+      for (int c = 4 * l16; c < dim; c += 64)
+        *reinterpret_cast<f32x4*>(ql + m16 * LD + c) = *reinterpret_cast<f32x4*>(kl + m16 * LD + c) = zero;
+    }
+    for (int c = 4 * l16; c < vdim; c += 64) {
+      const V4<T> v = *reinterpret_cast<const V4<T>*>(static_cast<const T*>(p.proj) + (int64_t)(t0 + min(m16, n - 1)) * p.ldp + cv + c);
+      f32x4 f;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) f[x] = m16 < n ? (float)v[x] : 0.f;
+      *reinterpret_cast<f32x4*>(vl + m16 * LDV + c) = f;
     }
     __syncthreads();
-    const float ld = p.log2_decay[h];
-    {
-      const int i = tid >> 4, j = tid & 15;
-      float b = 0.f;
-      if (j <= i && i < n) {
-        for (int c = 0; c < dim; c += 4) {
-          const f32x4 qi = *reinterpret_cast<const f32x4*>(ql + i * LD + c), kj = *reinterpret_cast<const f32x4*>(kl + j * LD + c);
+    put_products(pb, row_products(ql, kl, LD, dim, wave, lane), wave, lane);
+    const float dq = be[m16 + 1];
+    for (int c = 4 * l16; c < dim; c += 64)
+      *reinterpret_cast<f32x4*>(out + sc.q + m16 * dim + c) = *reinterpret_cast<const f32x4*>(ql + m16 * LD + c) * dq;
+    const int y = 4 * (tid & 3);   // four rows of a channel a thread
+    f32x4 dk;
 #pragma unroll
-          for (int x = 0; x < 4; ++x) b = fmaf(qi[x], kj[x], b);
-        }
-        b *= exp2f(ld * (float)(i - j));
-      }
-      out[sc.b + i * CH + j] = b;
+    for (int x = 0; x < 4; ++x) dk[x] = be[max(n - 1 - y - x, 0)];
+    for (int c = tid >> 2; c < dim; c += 64) {
+      f32x4 k;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) k[x] = kl[(y + x) * LD + c] * dk[x];
+      *reinterpret_cast<f32x4*>(out + sc.k + c * CH + y) = k;
     }
-    for (int u = tid; u < CH * dim; u += 256) {
-      const int i = u / dim, c = u - i * dim;
-      out[sc.q + u] = ql[i * LD + c] * exp2f(ld * (float)(i + 1));
-      const int ck2 = u / CH, ik = u % CH;
-      out[sc.k + u] = kl[ik * LD + ck2] * exp2f(ld * (float)max(n - 1 - ik, 0));
+    for (int c = tid >> 2; c < vdim; c += 64) {
+      f32x4 v;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) v[x] = vl[(y + x) * LDV + c];
+      *reinterpret_cast<f32x4*>(out + sc.u + c * CH + y) = v;
     }
-    for (int u = tid; u < CH * vdim; u += 256) out[sc.u + u] = vl[(u % CH) * LDV + u / CH];
-    for (int c = tid; c < dim; c += 256) out[sc.d + c] = exp2f(ld * (float)n);
+    for (int c = tid; c < dim; c += 256) out[sc.d + c] = be[n];
+    __syncthreads();
+    out[sc.b + tid] = l16 <= m16 ? sum_products(pb, m16, l16) * be[max(m16 - l16, 0)] : 0.f;
   }
 }
 
-__device__ __forceinline__ void mma4(f32x4& acc, const f32x4& a, const f32x4& b) {
-#pragma unroll
-  for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], acc, 0, 0, 0);
-}
-
-// NT: 16-row tiles of the state.  One wave: 16 value columns of one (entry, head)
-template <int KIND, int NT>
-__global__ __launch_bounds__(256, 1) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+// NT: 16-row tiles of the state, dealt over RS waves.  One workgroup: 16 value columns of one (entry, head)
+template <int KIND, int NT, int RS>
+__global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+  constexpr int NW = NT / RS, DEPTH = NW <= 2 ? 3 : 2;   // tiles of a wave, chunks of operands in registers
+  constexpr bool DELTA = KIND == VMI_HY_DELTA;
+  __shared__ f32x4 red[2][DELTA ? 2 : 1][RS][64];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), kc = lane >> 4, r16 = lane & 15;
-  const int waves = blockDim.x >> 6, per = (p.vdim / 16 + waves - 1) / waves;
-  const int h = blockIdx.x / per, col0 = ((int)(blockIdx.x % per) * waves + wave) * 16, e = blockIdx.y;
-  if (col0 >= p.vdim) return;
+  const int cols = p.vdim >> 4, h = blockIdx.x / cols, col0 = (int)(blockIdx.x % cols) * 16, e = blockIdx.y;
   const Portion r = portion(s, e);
   if (r.len <= 0) return;
   constexpr int dim = NT * 16;
+  const int ct0 = wave * NW;
   const Scratch sc(KIND, dim, p.vdim);
   const int nch = (r.len + CH - 1) / CH;
   const int64_t step = (int64_t)p.heads * sc.size;
   const float* in = p.scratch + ((int64_t)s.chunk_start[e] * p.heads + h) * sc.size;
-  float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim) * p.vdim + col0 + r16;
-  f32x4 S[NT], w[KIND == VMI_HY_DELTA ? NT : 1], q[NT], k[NT];
+  float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim + 16 * ct0 + 4 * kc) * p.vdim + col0 + r16;
+  f32x4 S[NW];
 #pragma unroll
-  for (int ct = 0; ct < NT; ++ct)
+  for (int ct = 0; ct < NW; ++ct)
 #pragma unroll
-    for (int x = 0; x < 4; ++x) S[ct][x] = r.ctx > 0 ? st[(int64_t)(16 * ct + 4 * kc + x) * p.vdim] : 0.f;
+    for (int x = 0; x < 4; ++x) S[ct][x] = r.ctx > 0 ? st[(int64_t)(16 * ct + x) * p.vdim] : 0.f;
 
-  const int row = r16 * dim + 4 * kc, col = r16 * CH + 4 * kc;
-  auto load_w = [&](const float* c) {
-    if constexpr (KIND == VMI_HY_DELTA) {
+  struct Operands {
+    f32x4 w[DELTA ? NW : 1], q[NW], k[NW], d[NW], u, b;
+  };
+  const int row = r16 * dim + 16 * ct0 + 4 * kc, col = r16 * CH + 4 * kc;
+  auto load = [&](Operands& o, int c) {
+    const float* at = in + min(c, nch - 1) * step;   // (past the end: the last one again)
+    o.u = *reinterpret_cast<const f32x4*>(at + sc.u + col0 * CH + col);
 #pragma unroll
-      for (int ct = 0; ct < NT; ++ct) w[ct] = *reinterpret_cast<const f32x4*>(c + sc.w + row + 16 * ct);
+    for (int ct = 0; ct < NW; ++ct) {
+      if constexpr (DELTA) o.w[ct] = *reinterpret_cast<const f32x4*>(at + sc.w + row + 16 * ct);
+      o.q[ct] = *reinterpret_cast<const f32x4*>(at + sc.q + row + 16 * ct);
+    }
+    o.b = *reinterpret_cast<const f32x4*>(at + sc.b + col);
+#pragma unroll
+    for (int ct = 0; ct < NW; ++ct) {
+      o.d[ct] = *reinterpret_cast<const f32x4*>(at + sc.d + 16 * (ct0 + ct) + 4 * kc);
+      o.k[ct] = *reinterpret_cast<const f32x4*>(at + sc.k + 16 * (ct0 + ct) * CH + col);
     }
   };
-  auto load_q = [&](const float* c) {
+  float* out = p.o + (int64_t)r.qs * p.heads * p.vdim + (int64_t)h * p.vdim + col0 + r16;
+  auto chunk = [&](Operands& o, int c) {
+    auto& mine = red[c & 1];   // (two of them: a wave still reading chunk c's parts has passed the barrier of c, not of c + 1)
+    f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f}, b = a;
 #pragma unroll
-    for (int ct = 0; ct < NT; ++ct) q[ct] = *reinterpret_cast<const f32x4*>(c + sc.q + row + 16 * ct);
-  };
-  auto load_k = [&](const float* c) {
-#pragma unroll
-    for (int ct = 0; ct < NT; ++ct) k[ct] = *reinterpret_cast<const f32x4*>(c + sc.k + 16 * ct * CH + col);
-  };
-  f32x4 u0, b;
-  auto load_u = [&](const float* c) {
-    u0 = *reinterpret_cast<const f32x4*>(c + sc.u + col0 * CH + col);
-    b = *reinterpret_cast<const f32x4*>(c + sc.b + col);
-  };
-  load_u(in);
-  load_w(in);
-  load_q(in);
-  load_k(in);
-  float* o = p.o + (int64_t)r.qs * p.heads * p.vdim + (int64_t)h * p.vdim + col0 + r16;
-  for (int c = 0; c < nch; ++c) {
-    // every operand is asked for again, from the next chunk, as soon as its last use has been issued (the last chunk: from itself)
-    const float* next = c + 1 < nch ? in + step : in;
-    f32x4 u = u0, a0 = f32x4{0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    const f32x4 bb = b;
-    load_u(next);
-    if constexpr (KIND == VMI_HY_DELTA) {
-#pragma unroll
-      for (int ct = 0; ct < NT; ++ct) mma4(ct & 1 ? a1 : a0, w[ct], S[ct]);
-      u -= a0 + a1;
-      load_w(next);
+    for (int ct = 0; ct < NW; ++ct) {
+      if constexpr (DELTA) mma4(a, o.w[ct], S[ct]);
+      mma4(b, o.q[ct], S[ct]);
     }
-    f32x4 o0 = f32x4{0.f, 0.f, 0.f, 0.f}, o1 = o0;
+    if constexpr (DELTA) mine[1][wave][lane] = a;
+    mine[0][wave][lane] = b;
+    __syncthreads();
+    f32x4 u = o.u;
+    if constexpr (DELTA) {
 #pragma unroll
-    for (int ct = 0; ct < NT; ++ct) mma4(ct & 1 ? o1 : o0, q[ct], S[ct]);
-    load_q(next);
-    mma4(o0, bb, u);
-#pragma unroll
-    for (int ct = 0; ct < NT; ++ct) {
-      const f32x4 d = *reinterpret_cast<const f32x4*>(in + sc.d + 16 * ct + 4 * kc);
-#pragma unroll
-      for (int x = 0; x < 4; ++x) S[ct][x] *= d[x];
-      mma4(S[ct], k[ct], u);
+      for (int w = 0; w < RS; ++w) u -= mine[1][w][lane];
     }
-    load_k(next);
-    o0 += o1;
+    if (wave == c % RS) {   // the waves take turns finishing o
+      f32x4 y = mine[0][0][lane];
 #pragma unroll
-    for (int x = 0; x < 4; ++x) {
-      const int m = c * CH + 4 * kc + x;
-      if (m < r.len) o[(int64_t)m * p.heads * p.vdim] = o0[x];
+      for (int w = 1; w < RS; ++w) y += mine[0][w][lane];
+      mma4(y, o.b, u);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const int m = c * CH + 4 * kc + x;
+        if (m < r.len) out[(int64_t)m * p.heads * p.vdim] = y[x];
+      }
     }
-    in = next;
+#pragma unroll
+    for (int ct = 0; ct < NW; ++ct) {
+#pragma unroll
+      for (int x = 0; x < 4; ++x) S[ct][x] *= o.d[ct][x];
+      mma4(S[ct], o.k[ct], u);
+    }
+    load(o, c + DEPTH);
+  };
+  Operands ops[DEPTH];
+#pragma unroll
+  for (int i = 0; i < DEPTH; ++i) load(ops[i], i);
+  for (int c = 0; c < nch; c += DEPTH) {
+#pragma unroll
+    for (int i = 0; i < DEPTH; ++i)
+      if (c + i < nch) chunk(ops[i], c + i);
   }
 #pragma unroll
-  for (int ct = 0; ct < NT; ++ct)
+  for (int ct = 0; ct < NW; ++ct)
 #pragma unroll
-    for (int x = 0; x < 4; ++x) st[(int64_t)(16 * ct + 4 * kc + x) * p.vdim] = S[ct][x];
+    for (int x = 0; x < 4; ++x) st[(int64_t)(16 * ct + x) * p.vdim] = S[ct][x];
 }
 
 // the columns of a state that one workgroup of the single-token step takes, and the rows a thread then holds
@@ -448,7 +560,7 @@ __global__ __launch_bounds__(256) void state_step_kernel(const vmi_hy_state_args
       for (int c = tid & 63; c < dim; c += 64) x[c] *= a;
     }
   } else {
-    rotated_rows<T>(p, t, r.ctx, 1, 1, h, hk, ql, kl, dim, tid);
+    if (tid < 64) rotated_row<T>(p, t, hk, ql, kl, tid, 64);
     for (int c = tid; c < width; c += 256) vl[c] = (float)static_cast<const T*>(p.proj)[(int64_t)t * p.ldp + cv + c];
     beta = p.decay[h];   // (the one decay of the head)
   }
@@ -525,9 +637,8 @@ static int run_step(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_
 
 template <int KIND, int NT>
 static void launch_scan(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
-  const int waves = p.vdim >= 64 ? 4 : p.vdim / 16;
-  hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT>), dim3(p.heads * ((p.vdim / 16 + waves - 1) / waves), s.B), dim3(64 * waves),
-                     0, st, p, s);
+  constexpr int RS = NT % 4 == 0 ? 4 : 2;
+  hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT, RS>), dim3(p.heads * (p.vdim / 16), s.B), dim3(64 * RS), 0, st, p, s);
 }
 
 template <typename T, int KIND>
@@ -565,6 +676,15 @@ int64_t vmi_hy_state_scratch(int32_t kind, int32_t dim, int32_t vdim) { return S
 
 int32_t vmi_hy_state_fuses(int32_t dim, int32_t vdim) { return step_slice(dim, vdim) == vdim; }
 
+int vmi_hy_rotations(const double* freq, int32_t half, float* out, const vmi_hy_step* s, int32_t device, void* stream) {
+  static const char* who = "vmi_hy_rotations";
+  if (!freq || !out || !s || !s->tok_pos || s->T <= 0 || half <= 0) return fail(VMI_HY_E_ARG, who, "null pointer or non-positive size");
+  DeviceScope dev(device);
+  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
+  hipLaunchKernelGGL(rotations_kernel, dim3(s->T), dim3(64), 0, static_cast<hipStream_t>(stream), freq, half, out, s->tok_pos);
+  return launched(who);
+}
+
 int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream) {
   static const char* who = "vmi_hy_state";
   if (!a || !s || !a->proj || !a->state || (!a->o && !a->out) || !s->q_start || !s->q_len || !s->ctx || !s->state_slot || !s->flip ||
@@ -574,7 +694,7 @@ int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream)
   if (a->kind == VMI_HY_DELTA && (!a->beta || !a->z || !a->conv_w || !a->rate || !a->dt_bias || a->taps < 1 || a->taps > MAX_TAPS ||
                                   (a->taps > 1 && !a->tail)))
     return fail(VMI_HY_E_ARG, who, "the delta rule needs its gates and a convolution of 1 to 16 taps");
-  if (a->kind == VMI_HY_RETENTION && (!a->freq || !a->decay || !a->log2_decay || a->rot_n < 0 || a->rot_n > a->dim || (a->rot_n & 1)))
+  if (a->kind == VMI_HY_RETENTION && ((a->rot_n > 0 && !a->turns) || !a->decay || !a->log2_decay || a->rot_n < 0 || a->rot_n > a->dim || (a->rot_n & 1)))
     return fail(VMI_HY_E_ARG, who, "retention needs decays and an even number of rotated dimensions");
   if (!a->single && (!a->scratch || !a->o || !s->chunks || !s->chunk_start || s->n_chunks <= 0))
     return fail(VMI_HY_E_ARG, who, "portions need chunks and scratch");

@@ -67,7 +67,7 @@ class FetelornConfig:
         return out
 
 
-def random_tensors(cfg: FetelornConfig, device, seed: int = 0, rank: int = 64, buckets: int = 32) -> Dict[str, torch.Tensor]:
+def random_tensors(cfg: FetelornConfig, device, seed: int = 0, rank: int = 128, buckets: int = 32) -> Dict[str, torch.Tensor]:
     """Random bfloat16 weights of a configuration, scaled so that activations keep their size (no checkpoint exists)."""
     g = torch.Generator(device=device).manual_seed(seed)
     out = {}

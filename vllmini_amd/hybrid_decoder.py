@@ -176,6 +176,7 @@ class HybridDecoder:
     # ---- the forward pass --------------------------------------------------------------------------------------------------
     def _forward(self, ids: torch.Tensor, step: ops.StepLayout, plans, rows: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
         m = self.model
+        step.begin()
         x0 = ops.embed(ids, m.embed, m.width, m.embed_scale)
         loops = any(r.enter is not None for r in m.runs)
         res = Residual(x0.clone() if loops and m.runs[0].enter is None else x0, m.dtype)

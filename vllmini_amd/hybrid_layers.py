@@ -317,7 +317,7 @@ class Retention:
         self.log2_decay = torch.tensor([max(math.log2(d), -1e30) if d > 0 else -1e30 for d in map(float, decay)], dtype=torch.float32,
                                        device=dev)
         i = torch.arange(rot_dims // 2, dtype=torch.float64)
-        self.freq = (float(rot_base) ** (-2.0 * i / max(rot_dims, 1))).to(dev)
+        self.freq, self.turn_key = (float(rot_base) ** (-2.0 * i / max(rot_dims, 1))).to(dev), (float(rot_base), rot_dims)
 
     def page_rows(self) -> List[int]:
         return []
@@ -331,7 +331,7 @@ class Retention:
 
     def run(self, proj: torch.Tensor, out: torch.Tensor, step: StepLayout, plans: Plans, held: Sequence[torch.Tensor]) -> None:
         ops.linear_state(proj, step, kind=ops.RETENTION, state=held[0], gate=proj[:, self.gate_at:self.gate_at + out.shape[1]], act="silu",
-                         out=out, freq=self.freq, decay=self.decay, log2_decay=self.log2_decay, **self.sizes)
+                         out=out, turns=step.rotations(self.freq, self.turn_key), decay=self.decay, log2_decay=self.log2_decay, **self.sizes)
 
 
 class GatedDelta:

@@ -54,7 +54,7 @@ PrepArgs = _struct("PrepArgs", [(_vp, "proj q cache norm_w freq"), (_i64, "ldp")
                                 (_f32, "eps"), (_i32, "dtype device")])
 AttentionArgs = _struct("AttentionArgs", [(_vp, "q cache out tiles partial"), (_i32, "heads rank rot n_tiles row_tiles splits"),
                                           (_f32, "scale"), (_i32, "dtype device")])
-StateArgs = _struct("StateArgs", [(_vp, "proj beta z conv_w rate dt_bias decay log2_decay freq state tail o scratch out gate norm_w"),
+StateArgs = _struct("StateArgs", [(_vp, "proj beta z conv_w rate dt_bias decay log2_decay turns state tail o scratch out gate norm_w"),
                                   (_i64, "ldp ldz ldo ldg"),
                                   (_i32, "heads kv_heads dim vdim dim_n vdim_n taps rot_n kind single act"), (_f32, "eps"),
                                   (_i32, "dtype device")])
@@ -70,6 +70,7 @@ SIGNATURES = {
     "vmi_hy_add_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _i32, _i32, _vp]),
     "vmi_hy_merge": (ctypes.c_int, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _i32, _i32, _i32, _f32, _f32, _i32, _i32, _vp]),
     "vmi_hy_glu": (ctypes.c_int, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _f32, _f32, _i32, _i32, _vp]),
+    "vmi_hy_rotations": (ctypes.c_int, [_vp, _i32, _vp, ctypes.POINTER(StepArgs), _i32, _vp]),
     "vmi_hy_state_scratch": (_i64, [_i32, _i32, _i32]),
     "vmi_hy_state_fuses": (_i32, [_i32, _i32]),
     "vmi_hy_state": (ctypes.c_int, [ctypes.POINTER(StateArgs), ctypes.POINTER(StepArgs), _vp]),
@@ -344,6 +345,23 @@ class StepLayout:
                                                                   "state_slot", "flip", "table")},
                              chunks=_ptr(chunks), chunk_start=_ptr(fields.get("chunk_start")), n_chunks=self.n_chunks, T=T, B=B, table_ld=tab.shape[1], page_size=page_size)
         self.ref = ctypes.byref(self.args)
+        self._turns: dict = {}
+
+    def begin(self) -> None:
+        """A forward pass over this layout starts: what earlier passes derived from its positions is void (a captured pass has to
+        derive it again)."""
+        self._turns.clear()
+
+    def rotations(self, freq: torch.Tensor, key) -> torch.Tensor:
+        """float32 [T, n, 2]: cos and sin of position times frequency; one launch per pass for all layers that name the same key."""
+        if key not in self._turns:
+            device, stream = _on(freq)
+            _need(freq.dtype == torch.float64 and freq.is_contiguous(), "StepLayout.rotations: float64 frequencies")
+            out = torch.empty((self.T, freq.numel(), 2), dtype=torch.float32, device=freq.device)
+            if freq.numel():
+                _check(load().vmi_hy_rotations(freq.data_ptr(), freq.numel(), out.data_ptr(), self.ref, device, stream))
+            self._turns[key] = out
+        return self._turns[key]
 
 
 def rglru(yx: torch.Tensor, step: StepLayout, *, conv_w: torch.Tensor, conv_b: torch.Tensor, gates: torch.Tensor, gate_b: torch.Tensor,
@@ -415,7 +433,7 @@ def state_fuses(dim: int, vdim: int) -> bool:
 
 def linear_state(proj: torch.Tensor, step: StepLayout, *, kind: int, heads: int, kv_heads: int, dim: int, vdim: int, dim_n: int,
                  vdim_n: int, state: torch.Tensor, gate: torch.Tensor, act: str, eps: float, out: torch.Tensor,
-                 norm_w: Optional[torch.Tensor] = None, freq: Optional[torch.Tensor] = None, decay: Optional[torch.Tensor] = None,
+                 norm_w: Optional[torch.Tensor] = None, turns: Optional[torch.Tensor] = None, decay: Optional[torch.Tensor] = None,
                  log2_decay: Optional[torch.Tensor] = None, beta: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None,
                  conv_w: Optional[torch.Tensor] = None, rate: Optional[torch.Tensor] = None, dt_bias: Optional[torch.Tensor] = None,
                  tail: Optional[torch.Tensor] = None) -> None:
@@ -439,8 +457,9 @@ def linear_state(proj: torch.Tensor, step: StepLayout, *, kind: int, heads: int,
         _need(taps == 1 or (tail is not None and tail.shape == (state.shape[0], 2, taps - 1, C) and tail.dtype == dt
                             and tail.is_contiguous()), who + "tail [slots, 2, taps - 1, channels]")
     else:
-        _need(freq.dtype == torch.float64 and 2 * freq.numel() <= dim and decay.numel() == log2_decay.numel() == heads
-              and decay.dtype == log2_decay.dtype == torch.float32, who + "freq, decay")
+        _need(turns.dtype == torch.float32 and turns.dim() == 3 and turns.shape[0] == T and 2 * turns.shape[1] <= dim
+              and turns.is_contiguous() and decay.numel() == log2_decay.numel() == heads
+              and decay.dtype == log2_decay.dtype == torch.float32, who + "turns, decay")
     lib, single = load(), step.single
     fused = single and state_fuses(dim, vdim)
     o = scratch = None
@@ -450,11 +469,11 @@ def linear_state(proj: torch.Tensor, step: StepLayout, *, kind: int, heads: int,
         _need(step.n_chunks > 0, who + "the step's layout has no chunks")
         scratch = torch.empty(step.n_chunks * heads * lib.vmi_hy_state_scratch(kind, dim, vdim), dtype=torch.float32, device=proj.device)
     a = StateArgs(proj=proj.data_ptr(), beta=_ptr(beta), z=_ptr(z), conv_w=_ptr(conv_w), rate=_ptr(rate), dt_bias=_ptr(dt_bias),
-                  decay=_ptr(decay), log2_decay=_ptr(log2_decay), freq=_ptr(freq), state=state.data_ptr(),
+                  decay=_ptr(decay), log2_decay=_ptr(log2_decay), turns=_ptr(turns), state=state.data_ptr(),
                   tail=_ptr(tail) if taps > 1 else None, o=_ptr(o), scratch=_ptr(scratch), out=out.data_ptr() if fused else None,
                   gate=gate.data_ptr(), norm_w=_ptr(norm_w), ldp=proj.stride(0), ldz=z.stride(0) if z is not None else 0,
                   ldo=out.stride(0), ldg=gate.stride(0), heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, dim_n=dim_n, vdim_n=vdim_n,
-                  taps=taps, rot_n=2 * freq.numel() if freq is not None else 0, kind=kind, single=int(single), act=ACTS[act], eps=eps,
+                  taps=taps, rot_n=2 * turns.shape[1] if turns is not None else 0, kind=kind, single=int(single), act=ACTS[act], eps=eps,
                   dtype=DTYPES[dt], device=device)
     _check(lib.vmi_hy_state(ctypes.byref(a), step.ref, stream))
     if not fused:
