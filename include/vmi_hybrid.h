@@ -219,7 +219,7 @@ VMI_HY_API int vmi_hy_kv_prep(const vmi_hy_kv_prep_args* a, const vmi_hy_step* s
 /* score = scale q . k + bias[h][min(i - j, bias_n - 1)]; token i sees the j <= i of its own chunk of `chunk` tokens (0: all);
  * sink[h] adds exp(sink) to the denominator; out = softmax . v * sigmoid(gate[t, h]).  bias, sink and gate may be NULL; bias and
  * sink come times log2(e).  Query rows of an entry and key head are (token, head of the group) pairs, head fastest, in tiles of
- * 16 * row_tiles (1, 2 or 4; float32: 1): tiles [n_tiles][2] = (entry, first row), entry -1: none.  splits > 1: a tile's keys are dealt to that
+ * 16 * row_tiles (1 or 4, vmi_hy_attention_row_tiles): tiles [n_tiles][2] = (entry, first row), entry -1: none.  splits > 1: a tile's keys are dealt to that
  * many workgroups, partial float32 [splits][T * heads][vdim + 2]. */
 typedef struct {
   const void* q;

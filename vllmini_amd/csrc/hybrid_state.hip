@@ -403,7 +403,8 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
   constexpr bool DELTA = KIND == VMI_HY_DELTA;
   __shared__ f32x4 red[2][DELTA ? 2 : 1][RS][64];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), kc = lane >> 4, r16 = lane & 15;
-  const int cols = p.vdim >> 4, h = blockIdx.x / cols, col0 = (int)(blockIdx.x % cols) * 16, e = blockIdx.y;
+  // (heads vary fastest: the column blocks of one head, which read the same operands, then share an XCD's L2)
+  const int h = blockIdx.x % p.heads, col0 = (int)(blockIdx.x / p.heads) * 16, e = blockIdx.y;
   const Portion r = portion(s, e);
   if (r.len <= 0) return;
   constexpr int dim = NT * 16;
