@@ -165,8 +165,8 @@ VMI_HY_API int vmi_hy_latent_attention(const vmi_hy_latent_attention_args* a, co
  *                     g = exp(-rate_h softplus(z + dt_bias))
  * A step of single tokens (`single`) is one pass over the states; otherwise portions are cut into chunks of 16 rows whose inner
  * products are prepared independently (scratch: vmi_hy_state_scratch floats per (chunk, head)) and walked once per state.
- * The result is o (float32 [T, heads vdim]), or, where out is given and `single` and one workgroup holds a head
- * (vmi_hy_state_fuses), the finished out = o / rms(o) * norm_w * act(gate) in the element type. */
+ * out = o / rms(o) (over vdim_n) * norm_w (NULL: 1) * act(gate), per head.  A step of single tokens finishes its rows by itself where
+ * one workgroup holds a head (vmi_hy_state_fuses); where not, o (float32 [T, heads vdim]) holds them in between. */
 enum { VMI_HY_RETENTION = 0, VMI_HY_DELTA = 1 };
 enum { VMI_HY_ACT_SIGMOID = 0, VMI_HY_ACT_SILU = 1 };
 typedef struct {
@@ -181,9 +181,9 @@ typedef struct {
   const float* turns;      /* [T][rot_n / 2][2]: what vmi_hy_rotations wrote */
   float* state;            /* [slots][heads][dim][vdim] */
   void* tail;              /* [slots][2][taps - 1][2 kv_heads dim + heads vdim] element type */
-  float* o;
-  float* scratch;
-  void* out;
+  float* o;                /* single and not fused */
+  float* scratch;          /* not single */
+  void* out;               /* [T, ldo] heads vdim columns */
   const void* gate;        /* [T, ldg] heads vdim columns */
   const float* norm_w;     /* [vdim] or NULL */
   int64_t ldp, ldz, ldo, ldg;
@@ -196,11 +196,6 @@ VMI_HY_API int vmi_hy_rotations(const double* freq, int32_t half, float* out, co
 VMI_HY_API int64_t vmi_hy_state_scratch(int32_t kind, int32_t dim, int32_t vdim);
 VMI_HY_API int32_t vmi_hy_state_fuses(int32_t dim, int32_t vdim);
 VMI_HY_API int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream);
-
-/* out[t, h] = o[t, h] / rms(o[t, h]) (over vdim_n) * norm_w (NULL: 1) * act(gate[t, h]); o float32 [T, heads vdim] */
-VMI_HY_API int vmi_hy_head_norm_gate(const float* o, const void* gate, int64_t ldg, const float* norm_w, void* out, int64_t ldo,
-                                     int32_t T, int32_t heads, int32_t vdim, int32_t vdim_n, float eps, int32_t act, int32_t dtype,
-                                     int32_t device, void* stream);
 
 /* Grouped-query softmax attention over a paged cache of rows [kv_heads][dim | vdim] (csrc/hybrid_attention.hip).
  * prep: proj [T, ldp] = q [heads dim] | k [kv_heads dim] | v [kv_heads vdim]; q and k over their root mean square (dim_n true

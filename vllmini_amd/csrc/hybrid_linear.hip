@@ -440,42 +440,6 @@ __global__ __launch_bounds__(256) void merge_kernel(float* x, const T* a, int64_
   }
 }
 
-// every head's o over its root mean square, times a weight and the activated gate; 16 lanes per (token, head)
-template <typename T>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate, int64_t ldg,
-                                                             const float* __restrict__ norm_w, T* __restrict__ out, int64_t ldo,
-                                                             int64_t rows, int heads, int vdim, int vdim_n, float eps, int act) {
-  const int64_t row = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
-  if (row >= rows) return;
-  const int64_t t = row / heads;
-  const int h = (int)(row - t * heads), l = threadIdx.x & 15;
-  o += row * vdim;
-  gate += t * ldg + (int64_t)h * vdim;
-  out += t * ldo + (int64_t)h * vdim;
-  float ss = 0.f;
-  for (int k = l * 4; k < vdim; k += 64) {
-    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
-  }
-#pragma unroll
-  for (int m = 8; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
-  const float r = 1.f / sqrtf(ss / (float)vdim_n + eps);
-  for (int k = l * 4; k < vdim; k += 64) {
-    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
-    const V4<T> g = *reinterpret_cast<const V4<T>*>(gate + k);
-    f32x4 w = f32x4{1.f, 1.f, 1.f, 1.f};
-    if (norm_w) w = *reinterpret_cast<const f32x4*>(norm_w + k);
-    V4<T> y;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float z = (float)g[e];
-      y[e] = (T)(v[e] * r * w[e] * (act == VMI_HY_ACT_SILU ? silu(z) : sigmoid(z)));
-    }
-    *reinterpret_cast<V4<T>*>(out + k) = y;
-  }
-}
-
 // out [T, 2 n] = (x | x2) in the element type
 template <typename T>
 __global__ __launch_bounds__(256) void concat_kernel(const float* __restrict__ x, const float* __restrict__ x2, T* __restrict__ out, int n) {
@@ -609,26 +573,6 @@ int vmi_hy_merge(float* x, const void* a, int64_t ld_a, const void* b, int64_t l
   else
     hipLaunchKernelGGL(merge_kernel<float>, dim3(T), dim3(256), 0, st, x, static_cast<const float*>(a), ld_a, static_cast<const float*>(b),
                        ld_b, static_cast<const float*>(add), ld_add, wa, wb, n, ld, eps, scale);
-  return launched(who);
-}
-
-int vmi_hy_head_norm_gate(const float* o, const void* gate, int64_t ldg, const float* norm_w, void* out, int64_t ldo, int32_t T,
-                          int32_t heads, int32_t vdim, int32_t vdim_n, float eps, int32_t act, int32_t dtype, int32_t device,
-                          void* stream) {
-  static const char* who = "vmi_hy_head_norm_gate";
-  if (!o || !gate || !out || T <= 0 || heads <= 0 || vdim <= 0 || (vdim & 3) || (ldg & 3) || (ldo & 3) || vdim_n <= 0 || vdim_n > vdim)
-    return fail(VMI_HY_E_ARG, who, "bad argument");
-  DeviceScope dev(device);
-  if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");
-  hipStream_t st = static_cast<hipStream_t>(stream);
-  const int64_t rows = (int64_t)T * heads;
-  const dim3 grid((rows + 15) / 16);
-  if (dtype == VMI_HY_BF16)
-    hipLaunchKernelGGL(head_norm_gate_kernel<b16>, grid, dim3(256), 0, st, o, static_cast<const b16*>(gate), ldg, norm_w,
-                       static_cast<b16*>(out), ldo, rows, heads, vdim, vdim_n, eps, act);
-  else
-    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, st, o, static_cast<const float*>(gate), ldg, norm_w,
-                       static_cast<float*>(out), ldo, rows, heads, vdim, vdim_n, eps, act);
   return launched(who);
 }
 

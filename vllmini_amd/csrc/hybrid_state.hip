@@ -11,8 +11,8 @@
 // state_scan_kernel then walks a state's chunks: u = U0 - W S, o = q e^G S + B u, S update, on v_mfma_f32_16x16x4_f32.  A workgroup
 // owns 16 value columns of one head's state for the whole walk, each wave some of its rows, in the matrix core's result layout
 // (lane (kc, r16): rows 4 kc + r of column r16), which is at the same time the operand layout of the next product.  What the waves
-// exchange per chunk is their part of W S and q e^G S (16 x 16 each, one barrier); the operands of the next chunks are in flight
-// meanwhile, and rows past a portion's end are zeros in all of them.
+// exchange per chunk is their part of W S and, a chunk later, of o (16 x 16 each, one barrier); the operands of the next chunks are in
+// flight meanwhile, and rows past a portion's end are zeros in all of them.
 //
 // Steps of single tokens: state_step_kernel reads each state once, keeps it in registers between the correction and the read-out,
 // and writes it back; convolution, gates, norm and output gate ride along.
@@ -156,7 +156,7 @@ __device__ __forceinline__ float sum_products(const float* part, int i, int j) {
 
 // what one (chunk, head) hands to the walk, in floats
 struct Scratch {
-  int q, w, k, u, b, d, size;
+  int q, w, k, u, b, d, o, size;
   __host__ __device__ Scratch(int kind, int dim, int vdim) {
     q = 0;                                                // [16][dim]   q e^G
     w = q + CH * dim;                                     // [16][dim]   W (delta only)
@@ -164,7 +164,8 @@ struct Scratch {
     u = k + CH * dim;                                     // [vdim][16]  U0
     b = u + CH * vdim;                                    // [16][16]    B
     d = b + CH * CH;                                      // [dim]       e^{G_15}
-    size = d + dim;
+    o = d + dim;                                          // [16][vdim]  what the walk leaves: o
+    size = o + CH * vdim;
   }
 };
 
@@ -401,7 +402,9 @@ template <int KIND, int NT, int RS>
 __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
   constexpr int NW = NT / RS, DEPTH = NW <= 2 ? 3 : 2;   // tiles of a wave, chunks of operands in registers
   constexpr bool DELTA = KIND == VMI_HY_DELTA;
-  __shared__ f32x4 red[2][DELTA ? 2 : 1][RS][64];
+  constexpr int EW = 4 / RS;                             // elements of a lane's four that a wave finishes of o
+  __shared__ f32x4 reda[DELTA ? 2 : 1][DELTA ? RS : 1][64];
+  __shared__ float redo[2][RS][4][64];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), kc = lane >> 4, r16 = lane & 15;
   // (heads vary fastest: the column blocks of one head, which read the same operands, then share an XCD's L2)
   const int h = blockIdx.x % p.heads, col0 = (int)(blockIdx.x / p.heads) * 16, e = blockIdx.y;
@@ -412,7 +415,7 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
   const Scratch sc(KIND, dim, p.vdim);
   const int nch = (r.len + CH - 1) / CH;
   const int64_t step = (int64_t)p.heads * sc.size;
-  const float* in = p.scratch + ((int64_t)s.chunk_start[e] * p.heads + h) * sc.size;
+  float* const base = p.scratch + ((int64_t)s.chunk_start[e] * p.heads + h) * sc.size;
   float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim + 16 * ct0 + 4 * kc) * p.vdim + col0 + r16;
   f32x4 S[NW];
 #pragma unroll
@@ -421,51 +424,57 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
     for (int x = 0; x < 4; ++x) S[ct][x] = r.ctx > 0 ? st[(int64_t)(16 * ct + x) * p.vdim] : 0.f;
 
   struct Operands {
-    f32x4 w[DELTA ? NW : 1], q[NW], k[NW], d[NW], u, b;
+    f32x4 w[DELTA ? NW : 1], q[NW], k[NW], d[NW], u;
+    float b[EW];
   };
   const int row = r16 * dim + 16 * ct0 + 4 * kc, col = r16 * CH + 4 * kc;
+  // (no branch stands in a chunk: every path issues the same loads and stores, so the waits count them exactly)
   auto load = [&](Operands& o, int c) {
-    const float* at = in + min(c, nch - 1) * step;   // (past the end: the last one again)
-    o.u = *reinterpret_cast<const f32x4*>(at + sc.u + col0 * CH + col);
+    const float* at = base + min(c, nch - 1) * step;   // (past the end: the last one again)
 #pragma unroll
     for (int ct = 0; ct < NW; ++ct) {
       if constexpr (DELTA) o.w[ct] = *reinterpret_cast<const f32x4*>(at + sc.w + row + 16 * ct);
       o.q[ct] = *reinterpret_cast<const f32x4*>(at + sc.q + row + 16 * ct);
     }
-    o.b = *reinterpret_cast<const f32x4*>(at + sc.b + col);
+    o.u = *reinterpret_cast<const f32x4*>(at + sc.u + col0 * CH + col);
+#pragma unroll
+    for (int i = 0; i < EW; ++i) o.b[i] = at[sc.b + col + wave + RS * i];
 #pragma unroll
     for (int ct = 0; ct < NW; ++ct) {
       o.d[ct] = *reinterpret_cast<const f32x4*>(at + sc.d + 16 * (ct0 + ct) + 4 * kc);
       o.k[ct] = *reinterpret_cast<const f32x4*>(at + sc.k + 16 * (ct0 + ct) * CH + col);
     }
   };
-  float* out = p.o + (int64_t)r.qs * p.heads * p.vdim + (int64_t)h * p.vdim + col0 + r16;
+  f32x4 part = f32x4{0.f, 0.f, 0.f, 0.f};   // this wave's part of the last chunk's o
+  auto publish = [&](int c) {               // (two places: a wave still reading those of c has passed the barrier of c, not of c + 1)
+#pragma unroll
+    for (int x = 0; x < 4; ++x) redo[c & 1][wave][x][lane] = part[x];
+  };
+  auto finish = [&](int c) {                // the elements wave, wave + RS, .. of every lane's four of chunk c - 1
+    float* out = base + max(c - 1, 0) * step + sc.o + 4 * kc * p.vdim + col0 + r16;
+#pragma unroll
+    for (int i = 0; i < EW; ++i) {
+      const int x = wave + RS * i;
+      float y = redo[c & 1][0][x][lane];
+#pragma unroll
+      for (int w = 1; w < RS; ++w) y += redo[c & 1][w][x][lane];
+      out[x * p.vdim] = y;                  // (c = 0: zeros, which the next chunk overwrites)
+    }
+  };
   auto chunk = [&](Operands& o, int c) {
-    auto& mine = red[c & 1];   // (two of them: a wave still reading chunk c's parts has passed the barrier of c, not of c + 1)
     f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f}, b = a;
+    publish(c);
 #pragma unroll
     for (int ct = 0; ct < NW; ++ct) {
       if constexpr (DELTA) mma4(a, o.w[ct], S[ct]);
       mma4(b, o.q[ct], S[ct]);
     }
-    if constexpr (DELTA) mine[1][wave][lane] = a;
-    mine[0][wave][lane] = b;
+    if constexpr (DELTA) reda[c & 1][wave][lane] = a;
     __syncthreads();
     f32x4 u = o.u;
     if constexpr (DELTA) {
 #pragma unroll
-      for (int w = 0; w < RS; ++w) u -= mine[1][w][lane];
-    }
-    if (wave == c % RS) {   // the waves take turns finishing o
-      f32x4 y = mine[0][0][lane];
-#pragma unroll
-      for (int w = 1; w < RS; ++w) y += mine[0][w][lane];
-      mma4(y, o.b, u);
-#pragma unroll
-      for (int x = 0; x < 4; ++x) {
-        const int m = c * CH + 4 * kc + x;
-        if (m < r.len) out[(int64_t)m * p.heads * p.vdim] = y[x];
-      }
+      for (int w = 0; w < RS; ++w) u -= reda[c & 1][w][lane];
     }
 #pragma unroll
     for (int ct = 0; ct < NW; ++ct) {
@@ -473,20 +482,77 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
       for (int x = 0; x < 4; ++x) S[ct][x] *= o.d[ct][x];
       mma4(S[ct], o.k[ct], u);
     }
+#pragma unroll
+    for (int i = 0; i < EW; ++i) {          // B u, a share of its inner rows a wave
+      float ux = u[RS * i];
+#pragma unroll
+      for (int w = 1; w < RS; ++w) ux = wave == w ? u[w + RS * i] : ux;
+      b = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[i], ux, b, 0, 0, 0);
+    }
+    part = b;
+    finish(c);
     load(o, c + DEPTH);
   };
   Operands ops[DEPTH];
 #pragma unroll
   for (int i = 0; i < DEPTH; ++i) load(ops[i], i);
-  for (int c = 0; c < nch; c += DEPTH) {
+  int c = 0;
+  for (; c + DEPTH <= nch; c += DEPTH) {
 #pragma unroll
-    for (int i = 0; i < DEPTH; ++i)
-      if (c + i < nch) chunk(ops[i], c + i);
+    for (int i = 0; i < DEPTH; ++i) chunk(ops[i], c + i);
   }
+#pragma unroll
+  for (int i = 0; i + 1 < DEPTH; ++i)
+    if (c + i < nch) chunk(ops[i], c + i);
+  publish(nch);
+  __syncthreads();
+  finish(nch);
 #pragma unroll
   for (int ct = 0; ct < NW; ++ct)
 #pragma unroll
     for (int x = 0; x < 4; ++x) st[(int64_t)(16 * ct + x) * p.vdim] = S[ct][x];
+}
+
+// every head's o over its root mean square, times a weight and the activated gate; 16 lanes per (token, head).  o: rows of p.o, or
+// (portions) where the walk left them
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+  const int64_t row = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  if (row >= (int64_t)s.T * p.heads) return;
+  const int64_t t = row / p.heads;
+  const int h = (int)(row - t * p.heads), l = threadIdx.x & 15, vdim = p.vdim;
+  const float* o = p.o + row * vdim;
+  if (!p.single) {
+    const int e = s.tok_seq[t];
+    if (e < 0) return;
+    const int m = (int)t - s.q_start[e];
+    const Scratch sc(p.kind, p.dim, vdim);
+    o = p.scratch + ((int64_t)(s.chunk_start[e] + m / CH) * p.heads + h) * sc.size + sc.o + (m % CH) * vdim;
+  }
+  const T* gate = static_cast<const T*>(p.gate) + t * p.ldg + (int64_t)h * vdim;
+  T* out = static_cast<T*>(p.out) + t * p.ldo + (int64_t)h * vdim;
+  float ss = 0.f;
+  for (int k = l * 4; k < vdim; k += 64) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+#pragma unroll
+  for (int m = 8; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  const float r = 1.f / sqrtf(ss / (float)p.vdim_n + p.eps);
+  for (int k = l * 4; k < vdim; k += 64) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(o + k);
+    const V4<T> g = *reinterpret_cast<const V4<T>*>(gate + k);
+    f32x4 w = f32x4{1.f, 1.f, 1.f, 1.f};
+    if (p.norm_w) w = *reinterpret_cast<const f32x4*>(p.norm_w + k);
+    V4<T> y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float z = (float)g[e];
+      y[e] = (T)(v[e] * r * w[e] * (p.act == VMI_HY_ACT_SILU ? silu(z) : sigmoid(z)));
+    }
+    *reinterpret_cast<V4<T>*>(out + k) = y;
+  }
 }
 
 // the columns of a state that one workgroup of the single-token step takes, and the rows a thread then holds
@@ -609,7 +675,7 @@ __global__ __launch_bounds__(256) void state_step_kernel(const vmi_hy_state_args
     }
   }
   const float o = gather(part);
-  if (!p.out) {
+  if (slice < p.vdim) {
     if (tid < width) p.o[((int64_t)t * p.heads + h) * p.vdim + c0 + tid] = o;
     return;
   }
@@ -623,6 +689,11 @@ __global__ __launch_bounds__(256) void state_step_kernel(const vmi_hy_state_args
   }
 }
 
+template <typename T>
+static void launch_norm_gate(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
+  hipLaunchKernelGGL(head_norm_gate_kernel<T>, dim3(((int64_t)s.T * p.heads + 15) / 16), dim3(256), 0, st, p, s);
+}
+
 template <typename T, int KIND>
 static int run_step(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
   const int slice = step_slice(p.dim, p.vdim), rows = step_rows(p.dim, slice);
@@ -633,6 +704,7 @@ static int run_step(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_
   else if (rows <= 16) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 16>), grid, dim3(256), lds, st, p, s, slice);
   else if (rows <= 32) hipLaunchKernelGGL(HIP_KERNEL_NAME(state_step_kernel<T, KIND, 32>), grid, dim3(256), lds, st, p, s, slice);
   else return fail(VMI_HY_E_SHAPE, "vmi_hy_state", "heads this large are not built");
+  if (slice < p.vdim) launch_norm_gate<T>(p, s, st);
   return launched("vmi_hy_state");
 }
 
@@ -658,6 +730,7 @@ static int run_chunks(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStrea
     case 512: launch_scan<KIND, 32>(p, s, st); break;
     default: return fail(VMI_HY_E_SHAPE, "vmi_hy_state", "key dimensions of 32, 64, 96, 128, 192, 256 and 512 are built");
   }
+  launch_norm_gate<T>(p, s, st);
   return launched("vmi_hy_state");
 }
 
@@ -688,7 +761,7 @@ int vmi_hy_rotations(const double* freq, int32_t half, float* out, const vmi_hy_
 
 int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream) {
   static const char* who = "vmi_hy_state";
-  if (!a || !s || !a->proj || !a->state || (!a->o && !a->out) || !s->q_start || !s->q_len || !s->ctx || !s->state_slot || !s->flip ||
+  if (!a || !s || !a->proj || !a->state || !a->out || !a->gate || !s->q_start || !s->q_len || !s->ctx || !s->state_slot || !s->flip ||
       s->T <= 0 || s->B <= 0 || a->heads <= 0 || a->kv_heads <= 0 || a->dim <= 0 || a->vdim <= 0 || a->dim_n <= 0 || a->dim_n > a->dim ||
       a->vdim_n <= 0 || a->vdim_n > a->vdim || a->heads % a->kv_heads || a->kind < 0 || a->kind > 1 || a->dtype < 0 || a->dtype > 1)
     return fail(VMI_HY_E_ARG, who, "null pointer or a size out of range");
@@ -697,11 +770,10 @@ int vmi_hy_state(const vmi_hy_state_args* a, const vmi_hy_step* s, void* stream)
     return fail(VMI_HY_E_ARG, who, "the delta rule needs its gates and a convolution of 1 to 16 taps");
   if (a->kind == VMI_HY_RETENTION && ((a->rot_n > 0 && !a->turns) || !a->decay || !a->log2_decay || a->rot_n < 0 || a->rot_n > a->dim || (a->rot_n & 1)))
     return fail(VMI_HY_E_ARG, who, "retention needs decays and an even number of rotated dimensions");
-  if (!a->single && (!a->scratch || !a->o || !s->chunks || !s->chunk_start || s->n_chunks <= 0))
-    return fail(VMI_HY_E_ARG, who, "portions need chunks and scratch");
-  if (a->out && (!a->single || !a->gate || !vmi_hy_state_fuses(a->dim, a->vdim)))
-    return fail(VMI_HY_E_ARG, who, "only a step of single tokens with whole heads writes finished rows");
-  if ((a->dim & 31) || (a->vdim & 31) || (a->ldp & 7) || ((uintptr_t)a->proj & 15) || a->dim > 512 || s->B > 65535 || a->heads > 65535)
+  if (a->single ? !a->o && !vmi_hy_state_fuses(a->dim, a->vdim)
+                : !a->scratch || !s->tok_seq || !s->chunks || !s->chunk_start || s->n_chunks <= 0)
+    return fail(VMI_HY_E_ARG, who, "portions need chunks and scratch, single tokens of heads this large a place for o");
+  if ((a->dim & 31) || (a->vdim & 31) || (a->ldp & 7) || ((uintptr_t)a->proj & 15) || (a->ldg & 3) || (a->ldo & 3) || a->dim > 512 || s->B > 65535 || a->heads > 65535)
     return fail(VMI_HY_E_SHAPE, who, "needs sizes that are multiples of 32, key dimensions up to 512 and aligned rows");
   DeviceScope dev(a->device);
   if (!dev.ok) return fail(VMI_HY_E_HIP, who, "hipSetDevice failed");

@@ -74,7 +74,6 @@ SIGNATURES = {
     "vmi_hy_state_scratch": (_i64, [_i32, _i32, _i32]),
     "vmi_hy_state_fuses": (_i32, [_i32, _i32]),
     "vmi_hy_state": (ctypes.c_int, [ctypes.POINTER(StateArgs), ctypes.POINTER(StepArgs), _vp]),
-    "vmi_hy_head_norm_gate": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _i32, _i32, _vp]),
     "vmi_hy_kv_prep": (ctypes.c_int, [ctypes.POINTER(KvPrepArgs), ctypes.POINTER(StepArgs), _vp]),
     "vmi_hy_attention_row_tiles": (_i32, [_i32, _i32, _i32, _i32]),
     "vmi_hy_attention": (ctypes.c_int, [ctypes.POINTER(GqaArgs), ctypes.POINTER(StepArgs), _vp]),
@@ -461,24 +460,20 @@ def linear_state(proj: torch.Tensor, step: StepLayout, *, kind: int, heads: int,
               and turns.is_contiguous() and decay.numel() == log2_decay.numel() == heads
               and decay.dtype == log2_decay.dtype == torch.float32, who + "turns, decay")
     lib, single = load(), step.single
-    fused = single and state_fuses(dim, vdim)
     o = scratch = None
-    if not fused:
-        o = torch.empty((T, heads * vdim), dtype=torch.float32, device=proj.device)
     if not single:
         _need(step.n_chunks > 0, who + "the step's layout has no chunks")
         scratch = torch.empty(step.n_chunks * heads * lib.vmi_hy_state_scratch(kind, dim, vdim), dtype=torch.float32, device=proj.device)
+    elif not state_fuses(dim, vdim):
+        o = torch.empty((T, heads * vdim), dtype=torch.float32, device=proj.device)
     a = StateArgs(proj=proj.data_ptr(), beta=_ptr(beta), z=_ptr(z), conv_w=_ptr(conv_w), rate=_ptr(rate), dt_bias=_ptr(dt_bias),
                   decay=_ptr(decay), log2_decay=_ptr(log2_decay), turns=_ptr(turns), state=state.data_ptr(),
-                  tail=_ptr(tail) if taps > 1 else None, o=_ptr(o), scratch=_ptr(scratch), out=out.data_ptr() if fused else None,
+                  tail=_ptr(tail) if taps > 1 else None, o=_ptr(o), scratch=_ptr(scratch), out=out.data_ptr(),
                   gate=gate.data_ptr(), norm_w=_ptr(norm_w), ldp=proj.stride(0), ldz=z.stride(0) if z is not None else 0,
                   ldo=out.stride(0), ldg=gate.stride(0), heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, dim_n=dim_n, vdim_n=vdim_n,
                   taps=taps, rot_n=2 * turns.shape[1] if turns is not None else 0, kind=kind, single=int(single), act=ACTS[act], eps=eps,
                   dtype=DTYPES[dt], device=device)
     _check(lib.vmi_hy_state(ctypes.byref(a), step.ref, stream))
-    if not fused:
-        _check(lib.vmi_hy_head_norm_gate(o.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(norm_w), out.data_ptr(), out.stride(0), T,
-                                         heads, vdim, vdim_n, eps, ACTS[act], DTYPES[dt], device, stream))
 
 
 def kv_prep(proj: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, step: StepLayout, *, heads: int, kv_heads: int, dim: int, vdim: int,
