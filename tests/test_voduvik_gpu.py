@@ -49,6 +49,10 @@ def layout(counts, ctx, tables, page, slots=None, flips=None, pos_slots=True):
     f = dict(tok_seq=i32(seq), tok_pos=i32(pos), tok_slot=i32(slot), q_start=i32(starts), q_len=i32(counts), ctx=i32(ctx),
              state_slot=i32(range(len(counts)) if slots is None else slots), flip=i32([0] * len(counts) if flips is None else flips),
              table=i32(tables))
+    if (counts > 1).any():
+        per = -(-counts // ops.CHUNK_ROWS)
+        f["chunk_start"] = i32(np.cumsum(per) - per)
+        f["chunks"] = i32([(b, 16 * c) for b in range(len(counts)) for c in range(per[b])])
     spans = bool((starts // ops.ROW_TILE != (starts + counts - 1) // ops.ROW_TILE).any())
     return ops.StepLayout(f, int(counts.sum()), len(counts), page, bool((counts == 1).all()), spans, int(counts.max()),
                           int((ctx + counts).max()))

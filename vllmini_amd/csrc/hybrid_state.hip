@@ -397,17 +397,17 @@ __global__ __launch_bounds__(256) void state_prep_kernel(const vmi_hy_state_args
   }
 }
 
-// NT: 16-row tiles of the state, dealt over RS waves.  One workgroup: 16 value columns of one (entry, head)
-template <int KIND, int NT, int RS>
-__global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
-  constexpr int NW = NT / RS, DEPTH = NW <= 2 ? 3 : 2;   // tiles of a wave, chunks of operands in registers
+// NT: 16-row tiles of the state, dealt over RS waves.  One workgroup: CT tiles of 16 value columns of one (entry, head)
+template <int KIND, int NT, int RS, int CT>
+__global__ __launch_bounds__(64 * RS, CT > 1 && NT <= 8 ? 2 : 1) void state_scan_kernel(const vmi_hy_state_args p, const vmi_hy_step s) {
+  constexpr int NW = NT / RS, DEPTH = NW <= 2 && CT == 1 ? 3 : 2;   // tiles of a wave, chunks of operands in registers
   constexpr bool DELTA = KIND == VMI_HY_DELTA;
   constexpr int EW = 4 / RS;                             // elements of a lane's four that a wave finishes of o
-  __shared__ f32x4 reda[DELTA ? 2 : 1][DELTA ? RS : 1][64];
-  __shared__ float redo[2][RS][4][64];
+  __shared__ f32x4 reda[DELTA ? 2 : 1][CT][DELTA ? RS : 1][64];
+  __shared__ float redo[2][CT][RS][4][64];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), kc = lane >> 4, r16 = lane & 15;
   // (heads vary fastest: the column blocks of one head, which read the same operands, then share an XCD's L2)
-  const int h = blockIdx.x % p.heads, col0 = (int)(blockIdx.x / p.heads) * 16, e = blockIdx.y;
+  const int h = blockIdx.x % p.heads, col0 = (int)(blockIdx.x / p.heads) * 16 * CT, e = blockIdx.y;
   const Portion r = portion(s, e);
   if (r.len <= 0) return;
   constexpr int dim = NT * 16;
@@ -417,14 +417,16 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
   const int64_t step = (int64_t)p.heads * sc.size;
   float* const base = p.scratch + ((int64_t)s.chunk_start[e] * p.heads + h) * sc.size;
   float* st = p.state + (((int64_t)r.slot * p.heads + h) * dim + 16 * ct0 + 4 * kc) * p.vdim + col0 + r16;
-  f32x4 S[NW];
+  f32x4 S[NW][CT];
 #pragma unroll
-  for (int ct = 0; ct < NW; ++ct)
+  for (int t = 0; t < NW; ++t)
 #pragma unroll
-    for (int x = 0; x < 4; ++x) S[ct][x] = r.ctx > 0 ? st[(int64_t)(16 * ct + x) * p.vdim] : 0.f;
+    for (int c = 0; c < CT; ++c)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) S[t][c][x] = r.ctx > 0 ? st[(int64_t)(16 * t + x) * p.vdim + 16 * c] : 0.f;
 
   struct Operands {
-    f32x4 w[DELTA ? NW : 1], q[NW], k[NW], d[NW], u;
+    f32x4 w[DELTA ? NW : 1], q[NW], k[NW], d[NW], u[CT];
     float b[EW];
   };
   const int row = r16 * dim + 16 * ct0 + 4 * kc, col = r16 * CH + 4 * kc;
@@ -432,64 +434,86 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
   auto load = [&](Operands& o, int c) {
     const float* at = base + min(c, nch - 1) * step;   // (past the end: the last one again)
 #pragma unroll
-    for (int ct = 0; ct < NW; ++ct) {
-      if constexpr (DELTA) o.w[ct] = *reinterpret_cast<const f32x4*>(at + sc.w + row + 16 * ct);
-      o.q[ct] = *reinterpret_cast<const f32x4*>(at + sc.q + row + 16 * ct);
+    for (int t = 0; t < NW; ++t) {
+      if constexpr (DELTA) o.w[t] = *reinterpret_cast<const f32x4*>(at + sc.w + row + 16 * t);
+      o.q[t] = *reinterpret_cast<const f32x4*>(at + sc.q + row + 16 * t);
     }
-    o.u = *reinterpret_cast<const f32x4*>(at + sc.u + col0 * CH + col);
+#pragma unroll
+    for (int j = 0; j < CT; ++j) o.u[j] = *reinterpret_cast<const f32x4*>(at + sc.u + (col0 + 16 * j) * CH + col);
 #pragma unroll
     for (int i = 0; i < EW; ++i) o.b[i] = at[sc.b + col + wave + RS * i];
 #pragma unroll
-    for (int ct = 0; ct < NW; ++ct) {
-      o.d[ct] = *reinterpret_cast<const f32x4*>(at + sc.d + 16 * (ct0 + ct) + 4 * kc);
-      o.k[ct] = *reinterpret_cast<const f32x4*>(at + sc.k + 16 * (ct0 + ct) * CH + col);
+    for (int t = 0; t < NW; ++t) {
+      o.d[t] = *reinterpret_cast<const f32x4*>(at + sc.d + 16 * (ct0 + t) + 4 * kc);
+      o.k[t] = *reinterpret_cast<const f32x4*>(at + sc.k + 16 * (ct0 + t) * CH + col);
     }
   };
-  f32x4 part = f32x4{0.f, 0.f, 0.f, 0.f};   // this wave's part of the last chunk's o
+  f32x4 part[CT];                           // this wave's part of the last chunk's o
+#pragma unroll
+  for (int j = 0; j < CT; ++j) part[j] = f32x4{0.f, 0.f, 0.f, 0.f};
   auto publish = [&](int c) {               // (two places: a wave still reading those of c has passed the barrier of c, not of c + 1)
 #pragma unroll
-    for (int x = 0; x < 4; ++x) redo[c & 1][wave][x][lane] = part[x];
+    for (int j = 0; j < CT; ++j)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) redo[c & 1][j][wave][x][lane] = part[j][x];
   };
   auto finish = [&](int c) {                // the elements wave, wave + RS, .. of every lane's four of chunk c - 1
     float* out = base + max(c - 1, 0) * step + sc.o + 4 * kc * p.vdim + col0 + r16;
 #pragma unroll
-    for (int i = 0; i < EW; ++i) {
-      const int x = wave + RS * i;
-      float y = redo[c & 1][0][x][lane];
+    for (int j = 0; j < CT; ++j)
 #pragma unroll
-      for (int w = 1; w < RS; ++w) y += redo[c & 1][w][x][lane];
-      out[x * p.vdim] = y;                  // (c = 0: zeros, which the next chunk overwrites)
-    }
+      for (int i = 0; i < EW; ++i) {
+        const int x = wave + RS * i;
+        float y = redo[c & 1][j][0][x][lane];
+#pragma unroll
+        for (int w = 1; w < RS; ++w) y += redo[c & 1][j][w][x][lane];
+        out[x * p.vdim + 16 * j] = y;       // (c = 0: zeros, which the next chunk overwrites)
+      }
   };
   auto chunk = [&](Operands& o, int c) {
-    f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f}, b = a;
+    f32x4 a[CT], b[CT], u[CT];
     publish(c);
 #pragma unroll
-    for (int ct = 0; ct < NW; ++ct) {
-      if constexpr (DELTA) mma4(a, o.w[ct], S[ct]);
-      mma4(b, o.q[ct], S[ct]);
-    }
-    if constexpr (DELTA) reda[c & 1][wave][lane] = a;
-    __syncthreads();
-    f32x4 u = o.u;
+    for (int j = 0; j < CT; ++j) a[j] = b[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < NW; ++t)
+#pragma unroll
+      for (int j = 0; j < CT; ++j) {
+        if constexpr (DELTA) mma4(a[j], o.w[t], S[t][j]);
+        mma4(b[j], o.q[t], S[t][j]);
+      }
     if constexpr (DELTA) {
 #pragma unroll
-      for (int w = 0; w < RS; ++w) u -= reda[c & 1][w][lane];
+      for (int j = 0; j < CT; ++j) reda[c & 1][j][wave][lane] = a[j];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < CT; ++j) {
+      u[j] = o.u[j];
+      if constexpr (DELTA) {
+#pragma unroll
+        for (int w = 0; w < RS; ++w) u[j] -= reda[c & 1][j][w][lane];
+      }
     }
 #pragma unroll
-    for (int ct = 0; ct < NW; ++ct) {
+    for (int t = 0; t < NW; ++t)
 #pragma unroll
-      for (int x = 0; x < 4; ++x) S[ct][x] *= o.d[ct][x];
-      mma4(S[ct], o.k[ct], u);
+      for (int j = 0; j < CT; ++j) {
+#pragma unroll
+        for (int x = 0; x < 4; ++x) S[t][j][x] *= o.d[t][x];
+        mma4(S[t][j], o.k[t], u[j]);
+      }
+#pragma unroll
+    for (int j = 0; j < CT; ++j) {
+#pragma unroll
+      for (int i = 0; i < EW; ++i) {        // B u, a share of its inner rows a wave
+        float ux = u[j][RS * i];
+#pragma unroll
+        for (int w = 1; w < RS; ++w) ux = wave == w ? u[j][w + RS * i] : ux;
+        b[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[i], ux, b[j], 0, 0, 0);
+      }
+      part[j] = b[j];
     }
-#pragma unroll
-    for (int i = 0; i < EW; ++i) {          // B u, a share of its inner rows a wave
-      float ux = u[RS * i];
-#pragma unroll
-      for (int w = 1; w < RS; ++w) ux = wave == w ? u[w + RS * i] : ux;
-      b = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[i], ux, b, 0, 0, 0);
-    }
-    part = b;
     finish(c);
     load(o, c + DEPTH);
   };
@@ -508,9 +532,11 @@ __global__ __launch_bounds__(64 * RS) void state_scan_kernel(const vmi_hy_state_
   __syncthreads();
   finish(nch);
 #pragma unroll
-  for (int ct = 0; ct < NW; ++ct)
+  for (int t = 0; t < NW; ++t)
 #pragma unroll
-    for (int x = 0; x < 4; ++x) st[(int64_t)(16 * ct + x) * p.vdim] = S[ct][x];
+    for (int j = 0; j < CT; ++j)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) st[(int64_t)(16 * t + x) * p.vdim + 16 * j] = S[t][j][x];
 }
 
 // every head's o over its root mean square, times a weight and the activated gate; 16 lanes per (token, head).  o: rows of p.o, or
@@ -711,7 +737,13 @@ static int run_step(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_
 template <int KIND, int NT>
 static void launch_scan(const vmi_hy_state_args& p, const vmi_hy_step& s, hipStream_t st) {
   constexpr int RS = NT % 4 == 0 ? 4 : 2;
-  hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT, RS>), dim3(p.heads * (p.vdim / 16), s.B), dim3(64 * RS), 0, st, p, s);
+  const int tiles = p.vdim / 16;   // (even: vdim is a multiple of 32)
+  // states enough for the chip: a workgroup takes two column tiles, which halves what is read per column
+  if (NT <= 16 && (int64_t)p.heads * tiles * s.B >= 1024)
+    hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT, RS, NT <= 16 ? 2 : 1>), dim3(p.heads * (tiles / 2), s.B), dim3(64 * RS), 0,
+                       st, p, s);
+  else
+    hipLaunchKernelGGL(HIP_KERNEL_NAME(state_scan_kernel<KIND, NT, RS, 1>), dim3(p.heads * tiles, s.B), dim3(64 * RS), 0, st, p, s);
 }
 
 template <typename T, int KIND>

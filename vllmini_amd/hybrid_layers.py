@@ -386,9 +386,11 @@ def distance_buckets(n: int, buckets: int, far: float) -> torch.Tensor:
     """The row of a learned distance bias for distances 0 .. n - 1: one row each below half the rows, logarithmically wider ones up to
     `far` above, the last one beyond."""
     half = buckets // 2
-    if half < 1 or not float(far) > half:
-        raise ValueError(f"a distance bias of {buckets} rows needs a largest distance beyond {half}")
     d = torch.arange(n, dtype=torch.float64)
+    if buckets == 1 or n <= half:
+        return torch.clamp(d, max=buckets - 1).long()
+    if not float(far) > half:
+        raise ValueError(f"a distance bias of {buckets} rows needs a largest distance beyond {half}")
     # (a distance that lies on an edge belongs above it, whatever the logarithms round to)
     up = torch.floor(torch.log(torch.clamp(d, min=1) / half) / math.log(float(far) / half) * (buckets - half) + 1e-9)
     return torch.where(d < half, d, torch.clamp(half + up, max=buckets - 1)).long()
