@@ -164,7 +164,7 @@ def test_joined_projections_keep_the_products():
     assert torch.equal(runs[2].mixer.w_out[0].dense[:E, :2 * 96].reshape(E, 2, 96)[:, :, :72], w["l2.mix.o"].view(E, 2, 72))
 
 
-@pytest.mark.parametrize("buckets,far,n", [(16, 240.0, 700), (9, 64.0, 100), (2, 1.5, 40), (32, 1000.0, 5000), (6, 27.0, 60), (16, 128.0, 300)])
+@pytest.mark.parametrize("buckets,far,n", [(16, 250.0, 700), (9, 64.0, 100), (2, 1.5, 40), (32, 1000.0, 5000), (6, 27.0, 60), (16, 128.0, 300)])
 def test_bias_table_of_distances(buckets, far, n):
     from vllmini_amd.hybrid_layers import distance_buckets
 

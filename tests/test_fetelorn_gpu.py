@@ -350,8 +350,10 @@ def test_attention_without_some_of_its_parts(parts):
 def test_attention_sees_just_inside_its_chunk_and_not_just_outside(dtype, decoded):
     """One score stands out: at the chunk's first and last key, at page borders inside it, at the query's own position — and one token
     outside either end, where it must not be seen."""
-    chunk, page = 120, 16
-    for i, p in ((239, 120), (239, 119), (240, 239), (240, 240), (250, 240), (250, 239), (359, 351), (359, 352), (359, 240), (300, 300), (300, 301)):
+    c = chunk = 136
+    page = 16
+    for i, p in ((2 * c - 1, c), (2 * c - 1, c - 1), (2 * c, 2 * c - 1), (2 * c, 2 * c), (2 * c + 10, 2 * c), (2 * c + 10, 2 * c - 1),
+                 (3 * c - 1, 399), (3 * c - 1, 400), (3 * c - 1, 2 * c), (2 * c + 60, 2 * c + 60), (2 * c + 60, 2 * c + 61)):
         n = 1 if decoded else 40
         if decoded and p > i:
             continue
